@@ -16,7 +16,8 @@
 // one run is finished here (with the sink term, if any); a row with more runs leaves (max, sum,
 // unnormalised output) per run, and the merge kernel adds the runs in ascending order and applies
 // the sink.  Runs start at multiples of RUN whatever the batch, so a row's sums depend on
-// (position, RUN) alone.
+// (position, RUN, window) alone.  With a sliding window a block begins at the first run in which one of
+// its rows sees a key, and a row's runs are counted from the first in which it sees one itself.
 #include "common.h"
 
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
@@ -38,13 +39,16 @@ __device__ __forceinline__ uint32_t pack_bf16(float a, float b) {
   return (uint32_t)f32_to_bf16(a).bits | ((uint32_t)f32_to_bf16(b).bits << 16);
 }
 
+// the first key a query at position p sees (window 0: all earlier ones)
+__device__ __forceinline__ int first_seen(int p, int window) { return window > 0 && p >= window ? p - window + 1 : 0; }
+
 template <int MAXD32, int MAXR16>
 __global__ __launch_bounds__(kLmWaves* kLmHalves* kWave) void attn_latent_mfma_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ rows, const int* __restrict__ block_table,
     const int* __restrict__ entry_of_token, const int* __restrict__ positions, const int* __restrict__ tiles,
     const int* __restrict__ token_list, int tile_subs, const float* __restrict__ sink, bf16_t* __restrict__ out,
     float* __restrict__ part_o, float* __restrict__ part_ml, float scale, LmGeom gm, int run_keys, int max_runs,
-    int page_size, int max_blocks, int num_pages) {
+    int page_size, int max_blocks, int num_pages, int window) {
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
   bf16_t* kt = reinterpret_cast<bf16_t*>(smem);                    // [32][ldk]
   bf16_t* vt = kt + kLmChunk * gm.ldk;                             // [R][kLmVtLd], keys in the order the second product wants
@@ -72,9 +76,12 @@ __global__ __launch_bounds__(kLmWaves* kLmHalves* kWave) void attn_latent_mfma_k
   }
   if (cnt <= 0) return;
   const int p0 = positions[tok0];
-  const int run = blockIdx.y;
-  const int k_begin = run * run_keys;
-  const int k_end = min(k_begin + run_keys, p0 + cnt);
+  // runs are counted from the first that holds a key some row of the block sees; keys before that
+  // row's window are not read (a whole number of chunks is left out, so that chunks begin at the same keys)
+  const int see0 = first_seen(p0, window);
+  const int run = see0 / run_keys + blockIdx.y;
+  const int k_end = min(run * run_keys + run_keys, p0 + cnt);
+  const int k_begin = max(run * run_keys, see0 & ~(kLmChunk - 1));
   if (k_begin >= k_end) return;
   const int* bt = block_table + (size_t)e * max_blocks;
 
@@ -85,6 +92,7 @@ __global__ __launch_bounds__(kLmWaves* kLmHalves* kWave) void attn_latent_mfma_k
   const bool row_ok = ti < cnt && head < gm.H;
   const int token = tok0 + (row_ok ? ti : 0);
   const int p_row = p0 + ti;
+  const int k_row = first_seen(p_row, window);      // the first key this row sees
   const bool wave_ok = __any(row_ok);
 
   bf16x8 qf[MAXD32];
@@ -179,7 +187,7 @@ __global__ __launch_bounds__(kLmWaves* kLmHalves* kWave) void attn_latent_mfma_k
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const int key = c0 + 16 * u + 4 * g + i;
-        const bool ok = row_ok && key < k_end && key <= p_row;
+        const bool ok = row_ok && key < k_end && key <= p_row && key >= k_row;
         sv[4 * u + i] = ok ? s[u][i] * scale : -INFINITY;
         mx = fmaxf(mx, sv[4 * u + i]);
       }
@@ -223,8 +231,8 @@ __global__ __launch_bounds__(kLmWaves* kLmHalves* kWave) void attn_latent_mfma_k
   }
 
   if (!row_ok) return;
-  const int n_runs = p_row / run_keys + 1;      // runs that hold keys of this row
-  if (run >= n_runs) return;
+  const int run0 = k_row / run_keys, n_runs = p_row / run_keys + 1 - run0;      // runs that hold keys of this row
+  if (run < run0 || run >= run0 + n_runs) return;
   const size_t rh = (size_t)token * gm.H + head;
   if (n_runs == 1) {
     float M = m_run, denom = l_run;
@@ -246,14 +254,14 @@ __global__ __launch_bounds__(kLmWaves* kLmHalves* kWave) void attn_latent_mfma_k
     }
     return;
   }
-  float* po = part_o + (rh * max_runs + run) * gm.R + 16 * r_lo;
+  float* po = part_o + (rh * max_runs + run - run0) * gm.R + 16 * r_lo;
 #pragma unroll
   for (int d = 0; d < MAXH; ++d) {
     if (d < r_n) *reinterpret_cast<float4*>(po + 16 * d + 4 * g) = make_float4(acc[d][0], acc[d][1], acc[d][2], acc[d][3]);
   }
   if (g == 0 && half == 0) {
-    part_ml[(rh * max_runs + run) * 2] = m_run;
-    part_ml[(rh * max_runs + run) * 2 + 1] = l_run;
+    part_ml[(rh * max_runs + run - run0) * 2] = m_run;
+    part_ml[(rh * max_runs + run - run0) * 2 + 1] = l_run;
   }
 }
 
@@ -265,12 +273,12 @@ constexpr int kLmMergeWaves = 4;
 __global__ __launch_bounds__(kLmMergeWaves* kWave) void attn_latent_merge_kernel(
     const float* __restrict__ part_o, const float* __restrict__ part_ml, const int* __restrict__ positions,
     const int* __restrict__ token_list, const float* __restrict__ sink, bf16_t* __restrict__ out, int H, int R,
-    int run_keys, int max_runs) {
+    int run_keys, int max_runs, int window) {
   const int token = token_list ? token_list[blockIdx.x] : blockIdx.x;
   const int head = blockIdx.y * kLmMergeWaves + (threadIdx.x >> 6);
   const int lane = threadIdx.x & (kWave - 1);
   if (head >= H) return;
-  const int n_runs = positions[token] / run_keys + 1;
+  const int n_runs = positions[token] / run_keys + 1 - first_seen(positions[token], window) / run_keys;
   if (n_runs <= 1) return;
   const size_t rh = (size_t)token * H + head;
   bf16_t* orow = out + rh * R;
@@ -344,23 +352,27 @@ SHARPI_EXPORT int sharpi_attention_latent_mfma_block_tokens(int H) {
 // first token, rows <= tile_tokens) of consecutive tokens of one request, or n_items single tokens
 // (token_list int32 [n_items], or null: tokens 0 .. n_items - 1).  part_o float [T * H * max_runs * R],
 // part_ml float [T * H * max_runs * 2]: scratch for rows with keys in more than one run of run_keys
-// (a multiple of 32); max_runs runs cover every token's keys.  out [T, H, R] bfloat16.
+// (a multiple of 32); max_runs runs cover every token's keys.  window > 0: a query at position p sees the keys
+// p - window + 1 .. p only; grid_runs runs (>= max_runs) cover the keys that any row of a block's tokens sees.  out
+// [T, H, R] bfloat16.
 SHARPI_EXPORT int sharpi_attention_latent_mfma(const void* q, const void* rows, const int* block_table,
                                                const int* entry_of_token, const int* positions, const int* tiles,
                                                const int* token_list, int n_items, int tile_tokens,
                                                const float* sink, void* out, float* part_o, float* part_ml,
                                                float scale, int H, int R, int dr, int run_keys, int max_runs,
-                                               int page_size, int max_blocks, int num_pages, hipStream_t stream) {
+                                               int page_size, int max_blocks, int num_pages, int window, int grid_runs,
+                                               hipStream_t stream) {
   if (n_items <= 0) return SHARPI_OK;
   if (!sharpi_attention_latent_mfma_takes(R, dr) || H <= 0) return SHARPI_ERR_ARG;
   if (run_keys <= 0 || run_keys % kLmChunk || max_runs <= 0 || max_runs > 65535) return SHARPI_ERR_ARG;
   if (page_size <= 0 || max_blocks <= 0 || num_pages <= 0 || (tiles && tile_tokens <= 0)) return SHARPI_ERR_ARG;
+  if (window < 0 || grid_runs < max_runs || grid_runs > 65535) return SHARPI_ERR_ARG;
   const LmGeom g = lm_geom(H, R, dr);
   const int tpb = g.tgb * g.tb;
   const int subs = tiles ? ceil_div(tile_tokens, tpb) : 1;
   const int head_blocks = ceil_div(ceil_div(H, g.hpw), g.htb);
   if (head_blocks > 65535) return SHARPI_ERR_ARG;
-  dim3 grid(n_items * subs, max_runs, head_blocks), block(kLmWaves * kLmHalves * kWave);
+  dim3 grid(n_items * subs, grid_runs, head_blocks), block(kLmWaves * kLmHalves * kWave);
   const size_t lds = ((size_t)kLmChunk * g.ldk + (size_t)R * kLmVtLd) * sizeof(bf16_t);
 #define LM_LAUNCH(MD, MR)                                                                                         \
   do {                                                                                                            \
@@ -373,7 +385,7 @@ SHARPI_EXPORT int sharpi_attention_latent_mfma(const void* q, const void* rows, 
     }                                                                                                             \
     kern<<<grid, block, lds, stream>>>((const bf16_t*)q, (const bf16_t*)rows, block_table, entry_of_token,        \
                                        positions, tiles, token_list, subs, sink, (bf16_t*)out, part_o, part_ml,   \
-                                       scale, g, run_keys, max_runs, page_size, max_blocks, num_pages);           \
+                                       scale, g, run_keys, max_runs, page_size, max_blocks, num_pages, window);   \
   } while (0)
   if (g.d32 <= 5 && g.r16 <= 8) LM_LAUNCH(5, 8);
   else if (g.d32 <= 10 && g.r16 <= 16) LM_LAUNCH(10, 16);
@@ -387,12 +399,12 @@ SHARPI_EXPORT int sharpi_attention_latent_mfma(const void* q, const void* rows, 
 // The merge of the rows with more than one run: n_tokens tokens (token_list, or 0 .. n_tokens - 1).
 SHARPI_EXPORT int sharpi_attention_latent_merge(const float* part_o, const float* part_ml, const int* positions,
                                                 const int* token_list, int n_tokens, const float* sink, void* out,
-                                                int H, int R, int run_keys, int max_runs, hipStream_t stream) {
+                                                int H, int R, int run_keys, int max_runs, int window, hipStream_t stream) {
   if (n_tokens <= 0 || max_runs <= 1) return SHARPI_OK;
   if (H <= 0 || H > 65535 || R <= 0 || R % 4 || run_keys <= 0) return SHARPI_ERR_ARG;
   dim3 grid(n_tokens, ceil_div(H, kLmMergeWaves)), block(kLmMergeWaves * kWave);
   attn_latent_merge_kernel<<<grid, block, 0, stream>>>(part_o, part_ml, positions, token_list, sink, (bf16_t*)out, H, R,
-                                                       run_keys, max_runs);
+                                                       run_keys, max_runs, window);
   SHARPI_CHECK_LAUNCH();
   return SHARPI_OK;
 }

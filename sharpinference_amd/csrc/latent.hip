@@ -5,7 +5,8 @@
 //                  sum still to be formed (rows of the experts' outputs, their places and weights).
 // latent_prep:     per token: the latent c = rms_norm(first R of the down projection) and the one
 //                  rotated key part, stored side by side as the token's cache row [R + dr]; the
-//                  rotated parts of the queries go to the tails of the query rows [H, R + dr].
+//                  rotated parts of the queries go to the tails of the query rows [H, R + dr]; a query
+//                  latent, where queries come through one, is normed into rows of its own.
 // head_gemm:       out[t, h, n] = sum_k x[t, h, k] * w[h, n, k], one product per head, with an
 //                  optional sigmoid gate on the result (float FMA chains in ascending k: a row's
 //                  bits do not depend on the batch).
@@ -85,71 +86,89 @@ __device__ __forceinline__ float rotated_elem(const T* __restrict__ src, int j, 
   return (j & 1) ? b * cs[i] + a * sn[i] : a * cs[i] - b * sn[i];
 }
 
+// What a token's launch does, each part optional: the query latent c_q = rms_norm(Rq columns) into rows of its own,
+// the cache row (latent and rotated key part), the rotated parts of the queries.
+struct LatentPrep {
+  const void* q; int ldq, q_off;             // queries [H, dn + dr] (null: none)
+  const void* kv; int ldkv, kv_off;          // down projection [R + dr] (null: none)
+  const void* cq; int ldcq, cq_off, Rq;      // query latent before its norm (null: none)
+  void *q_full, *k_cache, *cq_out;
+  const float *norm_w, *cq_norm_w, *inv_freq;
+  const int *slots, *positions;
+  int n_pairs, H, dn, dr, R;
+  float eps, magnitude;
+};
+
 template <typename T>
-__global__ __launch_bounds__(256) void latent_prep_kernel(const T* __restrict__ proj, int ld, int q_off, int kv_off,
-                                                          T* __restrict__ q_full, T* __restrict__ k_cache,
-                                                          const int* __restrict__ slots,
-                                                          const int* __restrict__ positions,
-                                                          const float* __restrict__ inv_freq, int n_pairs,
-                                                          const float* __restrict__ norm_w, float eps, int H, int dn,
-                                                          int dr, int R) {
+__global__ __launch_bounds__(256) void latent_prep_kernel(LatentPrep a) {
   __shared__ float red[16];
   __shared__ float cs[kMaxPairs], sn[kMaxPairs];
   const int t = blockIdx.x;
-  const float p = (float)positions[t];
-  for (int i = threadIdx.x; i < n_pairs; i += blockDim.x) {
-    const float ang = p * inv_freq[i];
-    cs[i] = cosf(ang);
-    sn[i] = sinf(ang);
+  const float p = (float)a.positions[t];
+  for (int i = threadIdx.x; i < a.n_pairs; i += blockDim.x) {
+    const float ang = p * a.inv_freq[i];
+    cs[i] = cosf(ang) * a.magnitude;
+    sn[i] = sinf(ang) * a.magnitude;
   }
   __syncthreads();
-  const T* row = proj + (size_t)t * ld;
-  const int D = R + dr;
-  for (int idx = threadIdx.x; idx < H * dr; idx += blockDim.x) {
-    const int h = idx / dr, j = idx - h * dr;
-    const T* qr = row + q_off + (size_t)h * (dn + dr) + dn;
-    q_full[((size_t)t * H + h) * D + R + j] = from_f32<T>(rotated_elem<T>(qr, j, n_pairs, cs, sn));
+  const int D = a.R + a.dr;
+  if (a.q) {
+    const T* row = (const T*)a.q + (size_t)t * a.ldq + a.q_off;
+    for (int idx = threadIdx.x; idx < a.H * a.dr; idx += blockDim.x) {
+      const int h = idx / a.dr, j = idx - h * a.dr;
+      ((T*)a.q_full)[((size_t)t * a.H + h) * D + a.R + j] =
+          from_f32<T>(rotated_elem<T>(row + (size_t)h * (a.dn + a.dr) + a.dn, j, a.n_pairs, cs, sn));
+    }
   }
-  if (kv_off < 0) return;                  // (the same for every thread)
-  const T* kv = row + kv_off;
+  if (a.cq) {                                // (the same for every thread)
+    const T* src = (const T*)a.cq + (size_t)t * a.ldcq + a.cq_off;
+    float ss = 0.f;
+    for (int c = threadIdx.x; c < a.Rq; c += blockDim.x) {
+      const float x = to_f32<T>(src[c]);
+      ss += x * x;
+    }
+    const float s = 1.0f / sqrtf(block_sum(ss, red) / (float)a.Rq + a.eps);
+    T* dst = (T*)a.cq_out + (size_t)t * a.Rq;
+    for (int c = threadIdx.x; c < a.Rq; c += blockDim.x) dst[c] = from_f32<T>((to_f32<T>(src[c]) * s) * a.cq_norm_w[c]);
+  }
+  if (!a.kv) return;                         // (the same for every thread)
+  const T* kv = (const T*)a.kv + (size_t)t * a.ldkv + a.kv_off;
   float ss = 0.f;
-  for (int c = threadIdx.x; c < R; c += blockDim.x) {
+  for (int c = threadIdx.x; c < a.R; c += blockDim.x) {
     const float x = to_f32<T>(kv[c]);
     ss += x * x;
   }
   const float total = block_sum(ss, red);
-  const int slot = slots[t];
+  const int slot = a.slots[t];
   if (slot < 0) return;
-  const float s = 1.0f / sqrtf(total / (float)R + eps);
-  T* dst = k_cache + (size_t)slot * D;
-  for (int c = threadIdx.x; c < R; c += blockDim.x) dst[c] = from_f32<T>((to_f32<T>(kv[c]) * s) * norm_w[c]);
-  for (int j = threadIdx.x; j < dr; j += blockDim.x) dst[R + j] = from_f32<T>(rotated_elem<T>(kv + R, j, n_pairs, cs, sn));
+  const float s = 1.0f / sqrtf(total / (float)a.R + a.eps);
+  T* dst = (T*)a.k_cache + (size_t)slot * D;
+  for (int c = threadIdx.x; c < a.R; c += blockDim.x) dst[c] = from_f32<T>((to_f32<T>(kv[c]) * s) * a.norm_w[c]);
+  for (int j = threadIdx.x; j < a.dr; j += blockDim.x) dst[a.R + j] = from_f32<T>(rotated_elem<T>(kv + a.R, j, a.n_pairs, cs, sn));
 }
 
-// proj [T, ld]: queries at column q_off as [H, dn + dr], the down projection [R + dr] at column
-// kv_off (< 0: this layer makes no latent).  q_full [T, H, R + dr] receives the rotated query parts
-// (columns R ..); k_cache rows [R + dr] at `slots` (< 0: nothing stored) receive the latent and the
-// rotated key part.  inv_freq float [n_pairs], norm_w float [R].
-SHARPI_EXPORT int sharpi_latent_prep(const void* proj, int dtype, int ld, int q_off, int kv_off, void* q_full,
-                                     void* k_cache, const int* slots, const int* positions, const float* inv_freq,
-                                     int n_pairs, const float* norm_w, float eps, int n_tokens, int H, int dn, int dr,
+// Each of q, kv and cq may be null.  q [T, ldq]: queries at column q_off as [H, dn + dr]; q_full [T, H, R + dr] receives the
+// rotated query parts (columns R ..).  kv [T, ldkv]: the down projection [R + dr] at column kv_off; k_cache rows [R + dr]
+// at `slots` (< 0: nothing stored) receive the latent and the rotated key part.  cq [T, ldcq]: Rq columns at cq_off,
+// normed with cq_norm_w into cq_out [T, Rq].  inv_freq float [n_pairs]; cos and sin are multiplied by `magnitude`;
+// norm weights float.
+SHARPI_EXPORT int sharpi_latent_prep(const void* q, int ldq, int q_off, const void* kv, int ldkv, int kv_off, const void* cq,
+                                     int ldcq, int cq_off, int Rq, int dtype, void* q_full, void* k_cache, void* cq_out,
+                                     const int* slots, const int* positions, const float* inv_freq, int n_pairs, float magnitude,
+                                     const float* norm_w, const float* cq_norm_w, float eps, int n_tokens, int H, int dn, int dr,
                                      int R, hipStream_t stream) {
   if (n_tokens <= 0) return SHARPI_OK;
   if (H <= 0 || dn <= 0 || dr <= 0 || R <= 0 || n_pairs < 0 || n_pairs > kMaxPairs || 2 * n_pairs > dr) return SHARPI_ERR_ARG;
-  if (q_off < 0 || q_off + H * (dn + dr) > ld || (kv_off >= 0 && kv_off + R + dr > ld)) return SHARPI_ERR_ARG;
-  if (kv_off >= 0 && (!k_cache || !slots || !norm_w || !(eps > 0.f))) return SHARPI_ERR_ARG;
-  if (n_pairs > 0 && !inv_freq) return SHARPI_ERR_ARG;
+  if (q && (q_off < 0 || q_off + H * (dn + dr) > ldq || !q_full)) return SHARPI_ERR_ARG;
+  if (kv && (kv_off < 0 || kv_off + R + dr > ldkv || !k_cache || !slots || !norm_w || !(eps > 0.f))) return SHARPI_ERR_ARG;
+  if (cq && (cq_off < 0 || Rq <= 0 || cq_off + Rq > ldcq || !cq_out || !cq_norm_w || !(eps > 0.f))) return SHARPI_ERR_ARG;
+  if ((n_pairs > 0 && !inv_freq) || !positions) return SHARPI_ERR_ARG;
+  const LatentPrep a{q, ldq, q_off, kv, ldkv, kv_off, cq, ldcq, cq_off, Rq, q_full, k_cache, cq_out, norm_w, cq_norm_w, inv_freq,
+                     slots, positions, n_pairs, H, dn, dr, R, eps, magnitude};
   dim3 grid(n_tokens), block(256);
-  if (dtype == DT_F32)
-    latent_prep_kernel<float><<<grid, block, 0, stream>>>((const float*)proj, ld, q_off, kv_off, (float*)q_full,
-                                                          (float*)k_cache, slots, positions, inv_freq, n_pairs,
-                                                          norm_w, eps, H, dn, dr, R);
-  else if (dtype == DT_BF16)
-    latent_prep_kernel<bf16_t><<<grid, block, 0, stream>>>((const bf16_t*)proj, ld, q_off, kv_off, (bf16_t*)q_full,
-                                                           (bf16_t*)k_cache, slots, positions, inv_freq, n_pairs,
-                                                           norm_w, eps, H, dn, dr, R);
-  else
-    return SHARPI_ERR_ARG;
+  if (dtype == DT_F32) latent_prep_kernel<float><<<grid, block, 0, stream>>>(a);
+  else if (dtype == DT_BF16) latent_prep_kernel<bf16_t><<<grid, block, 0, stream>>>(a);
+  else return SHARPI_ERR_ARG;
   SHARPI_CHECK_LAUNCH();
   return SHARPI_OK;
 }

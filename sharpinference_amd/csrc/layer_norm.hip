@@ -1,0 +1,373 @@
+// Layers whose branches end in a layer norm and begin with a short convolution over the residual sum; the
+// embedding with a second table indexed by a pair of tokens.
+//
+// layer_norm:      x = h[r] (+ LN(delta[r]) w + b); the new x back into h; and, by what is asked for, x itself, LN of
+//                  x (a model's last norm), or x + conv(x) (what the next branch reads; steps of single
+//                  tokens) in the activations' storage type.  delta is a tensor or an expert sum still to be formed.
+// residual_conv:   out[t] = h[t] + sum_j w[:, j] h[t - taps + 1 + j], for steps that bring longer entries.
+// embed_bigram:    out[t] = table[id] * scale + pairs[(previous id * a + id * b) mod buckets].
+//
+// A convolution's last inputs lie in a ring [slots, taps, channels] of floats, position p at p mod taps; what lies
+// before position 0 is never read.  Statistics, sums and the residual sum are float.
+#include "common.h"
+
+constexpr int kLnMaxTaps = 8;
+
+struct LnDelta {
+  const void* y;                 // [T, hidden], or the experts' rows
+  const int* pos;                // [T, k]: places of a token's rows (null: y is a tensor)
+  const float* w;                // [T, k] or null
+  const void* shared;            // [T, hidden] or null (expert sums only)
+  int k;
+};
+
+template <typename TD, int V>
+__device__ __forceinline__ void ln_load(const TD* p, float* v) {
+  if constexpr (V == 8) load8(p, v);
+  else v[0] = to_f32<TD>(*p);
+}
+template <typename TO, int V>
+__device__ __forceinline__ void ln_store(TO* p, const float* v) {
+  if constexpr (V == 8) store8(p, v);
+  else *p = from_f32<TO>(v[0]);
+}
+
+template <typename TD, int V>
+__device__ __forceinline__ void ln_delta(const LnDelta& d, size_t r, int hidden, int c, float* v) {
+  if (!d.pos) {
+    ln_load<TD, V>((const TD*)d.y + r * hidden + c, v);
+    return;
+  }
+#pragma unroll
+  for (int i = 0; i < V; ++i) v[i] = 0.f;
+  for (int q = 0; q < d.k; ++q) {
+    float x[V];
+    ln_load<TD, V>((const TD*)d.y + (size_t)d.pos[r * d.k + q] * hidden + c, x);
+    const float wq = d.w ? d.w[r * d.k + q] : 1.0f;
+#pragma unroll
+    for (int i = 0; i < V; ++i) v[i] = fmaf(wq, x[i], v[i]);
+  }
+  if (d.shared) {
+    float x[V];
+    ln_load<TD, V>((const TD*)d.shared + r * hidden + c, x);
+#pragma unroll
+    for (int i = 0; i < V; ++i) v[i] += x[i];
+  }
+}
+
+enum : int { LN_COPY = 0, LN_NORM = 1, LN_CONV = 2 };    // what `out` is
+
+struct LnConv {
+  const float* w;                // [hidden, taps]
+  float* ring;                   // [slots, taps, hidden] (null with one tap)
+  int taps;
+  const int *positions, *state_slots, *entry_of_token;
+};
+
+template <typename TD, typename TO, int V>
+__global__ __launch_bounds__(1024) void layer_norm_kernel(float* __restrict__ h, LnDelta delta, const float* __restrict__ w,
+                                                          const float* __restrict__ b, float eps, const int* __restrict__ rows,
+                                                          int write_back, TO* __restrict__ out, int mode,
+                                                          const float* __restrict__ w2, const float* __restrict__ b2, float eps2,
+                                                          LnConv cv, int hidden) {
+  extern __shared__ __attribute__((aligned(16))) float row[];
+  __shared__ float red[16];
+  const size_t i = blockIdx.x, r = rows ? rows[i] : i;
+  float* hr = h + r * hidden;
+  const int step = blockDim.x * V, c_first = threadIdx.x * V;
+  float x[V], y[V], wv[V], bv[V];
+  if (delta.y) {
+    float s = 0.f;
+    for (int c = c_first; c < hidden; c += step) {
+      ln_delta<TD, V>(delta, r, hidden, c, y);
+      ln_store<float, V>(row + c, y);
+#pragma unroll
+      for (int k = 0; k < V; ++k) s += y[k];
+    }
+    const float mean = block_sum(s, red) / (float)hidden;
+    s = 0.f;
+    for (int c = c_first; c < hidden; c += step) {     // (a thread reads what it wrote)
+      ln_load<float, V>(row + c, y);
+#pragma unroll
+      for (int k = 0; k < V; ++k) s = fmaf(y[k] - mean, y[k] - mean, s);
+    }
+    const float inv = 1.0f / sqrtf(block_sum(s, red) / (float)hidden + eps);
+    for (int c = c_first; c < hidden; c += step) {
+      ln_load<float, V>(row + c, y);
+      ln_load<float, V>(hr + c, x);
+      ln_load<float, V>(w + c, wv);
+      ln_load<float, V>(b + c, bv);
+#pragma unroll
+      for (int k = 0; k < V; ++k) x[k] += fmaf((y[k] - mean) * inv, wv[k], bv[k]);
+      if (write_back) ln_store<float, V>(hr + c, x);
+      if (out) ln_store<float, V>(row + c, x);
+    }
+  } else {
+    for (int c = c_first; c < hidden; c += step) {
+      ln_load<float, V>(hr + c, x);
+      ln_store<float, V>(row + c, x);
+    }
+  }
+  if (!out) return;
+  TO* o = out + i * hidden;
+  if (mode == LN_COPY) {
+    for (int c = c_first; c < hidden; c += step) {
+      ln_load<float, V>(row + c, x);
+      ln_store<TO, V>(o + c, x);
+    }
+  } else if (mode == LN_NORM) {
+    float s = 0.f;
+    for (int c = c_first; c < hidden; c += step) {
+      ln_load<float, V>(row + c, x);
+#pragma unroll
+      for (int k = 0; k < V; ++k) s += x[k];
+    }
+    const float mean = block_sum(s, red) / (float)hidden;
+    s = 0.f;
+    for (int c = c_first; c < hidden; c += step) {
+      ln_load<float, V>(row + c, x);
+#pragma unroll
+      for (int k = 0; k < V; ++k) s = fmaf(x[k] - mean, x[k] - mean, s);
+    }
+    const float inv = 1.0f / sqrtf(block_sum(s, red) / (float)hidden + eps2);
+    for (int c = c_first; c < hidden; c += step) {
+      ln_load<float, V>(row + c, x);
+      ln_load<float, V>(w2 + c, wv);
+      ln_load<float, V>(b2 + c, bv);
+#pragma unroll
+      for (int k = 0; k < V; ++k) x[k] = fmaf((x[k] - mean) * inv, wv[k], bv[k]);
+      ln_store<TO, V>(o + c, x);
+    }
+  } else {
+    const int p = cv.positions[r];
+    float* ring = cv.ring ? cv.ring + (size_t)cv.state_slots[cv.entry_of_token[r]] * cv.taps * hidden : nullptr;
+    for (int c = c_first; c < hidden; c += step) {
+      ln_load<float, V>(row + c, x);
+#pragma unroll
+      for (int k = 0; k < V; ++k) y[k] = 0.f;
+      for (int back = cv.taps - 1; back > 0; --back)
+        if (p >= back) {
+          float u[V];
+          ln_load<float, V>(ring + (size_t)((p - back) % cv.taps) * hidden + c, u);
+#pragma unroll
+          for (int k = 0; k < V; ++k) y[k] = fmaf(cv.w[(size_t)(c + k) * cv.taps + cv.taps - 1 - back], u[k], y[k]);
+        }
+      if (ring) ln_store<float, V>(ring + (size_t)(p % cv.taps) * hidden + c, x);
+#pragma unroll
+      for (int k = 0; k < V; ++k) x[k] += fmaf(cv.w[(size_t)(c + k) * cv.taps + cv.taps - 1], x[k], y[k]);
+      ln_store<TO, V>(o + c, x);
+    }
+  }
+}
+
+// h [T, hidden] float.  With delta (y of d_dtype; pos/sum_w/k/shared describe an expert sum): x = h + LN(delta) w + b,
+// back into h unless `rows` (int32 [n_rows]: only those rows, h unchanged) is given.  out (o_dtype, or null), mode 0:
+// x; 1: LN(x) w2 + b2; 2: x + conv(x) with conv_w float [hidden, taps] and the entries' rings (every entry of
+// the step one token: row = token).
+SHARPI_EXPORT int sharpi_layer_norm(float* h, const void* delta, int d_dtype, const int* pos, const float* sum_w, int k,
+                                    const void* shared, const float* w, const float* b, float eps, const int* rows, int n_rows,
+                                    int hidden, void* out, int o_dtype, int mode, const float* w2, const float* b2, float eps2,
+                                    const float* conv_w, float* ring, int taps, const int* positions, const int* state_slots,
+                                    const int* entry_of_token, hipStream_t stream) {
+  if (n_rows <= 0) return SHARPI_OK;
+  if (hidden <= 0 || (size_t)hidden * sizeof(float) > 60 * 1024) return SHARPI_ERR_ARG;
+  if (delta && (!w || !b || !(eps > 0.f) || (pos && k <= 0))) return SHARPI_ERR_ARG;
+  if (!delta && !out) return SHARPI_OK;
+  if (mode < 0 || mode > 2 || (mode == LN_NORM && (!w2 || !b2 || !(eps2 > 0.f)))) return SHARPI_ERR_ARG;
+  if (mode == LN_CONV && out && (!conv_w || taps < 1 || taps > kLnMaxTaps || (taps > 1 && !ring) || !positions || !state_slots || !entry_of_token || rows))
+    return SHARPI_ERR_ARG;
+  if ((d_dtype != DT_F32 && d_dtype != DT_BF16) || (out && o_dtype != DT_F32 && o_dtype != DT_BF16)) return SHARPI_ERR_ARG;
+  auto aligned = [](const void* p) { return ((uintptr_t)p & 31) == 0; };
+  const bool wide = hidden % 8 == 0 && aligned(h) && aligned(delta) && aligned(shared) && aligned(w) && aligned(b) && aligned(out) &&
+                    aligned(w2) && aligned(b2) && aligned(ring);
+  const LnDelta d{delta, pos, sum_w, shared, k};
+  const LnConv cv{conv_w, taps > 1 ? ring : nullptr, taps, positions, state_slots, entry_of_token};
+  const int runs = wide ? hidden / 8 : hidden;
+  int threads = ceil_div(runs, kWave) * kWave;
+  if (threads > (wide ? 1024 : 256)) threads = wide ? 1024 : 256;
+  const size_t lds = (size_t)hidden * sizeof(float);
+  const int wb = rows ? 0 : 1;
+#define LN(TD, TO)                                                                                                                    \
+  do {                                                                                                                                \
+    if (wide) layer_norm_kernel<TD, TO, 8><<<n_rows, threads, lds, stream>>>(h, d, w, b, eps, rows, wb, (TO*)out, mode, w2, b2, eps2, cv, hidden); \
+    else layer_norm_kernel<TD, TO, 1><<<n_rows, threads, lds, stream>>>(h, d, w, b, eps, rows, wb, (TO*)out, mode, w2, b2, eps2, cv, hidden);      \
+  } while (0)
+  const bool of = !out || o_dtype == DT_F32;
+  if (d_dtype == DT_F32) {
+    if (of) LN(float, float);
+    else LN(float, bf16_t);
+  } else {
+    if (of) LN(bf16_t, float);
+    else LN(bf16_t, bf16_t);
+  }
+#undef LN
+  SHARPI_CHECK_LAUNCH();
+  return SHARPI_OK;
+}
+
+// ---------------------------------------------------------------------------
+// The convolution over the residual sum in steps of longer entries.  A block: `tok` tokens x 256 V channels, a thread
+// V channels with the last TAPS - 1 inputs in registers.  Only an entry's first TAPS - 1 tokens reach back
+// beyond the step, into the ring; all of them are taken by the block in which the entry begins (also where they
+// run past its tokens), whose threads then bring the ring up to date: no other block reads it.
+// ---------------------------------------------------------------------------
+template <typename TO, int TAPS, int V>
+__global__ __launch_bounds__(256) void residual_conv_kernel(const float* __restrict__ h, const float* __restrict__ w,
+                                                            float* __restrict__ ring_all, const int* __restrict__ positions,
+                                                            const int* __restrict__ state_slots, const int* __restrict__ entry_of_token,
+                                                            const int* __restrict__ cu_tokens, TO* __restrict__ out, int n_tokens,
+                                                            int hidden, int tok) {
+  const int c = (blockIdx.y * blockDim.x + threadIdx.x) * V;
+  if (c >= hidden) return;
+  const int t0 = blockIdx.x * tok, t1 = min(t0 + tok, n_tokens);
+  float wt[TAPS][V];
+#pragma unroll
+  for (int back = 0; back < TAPS; ++back)
+#pragma unroll
+    for (int k = 0; k < V; ++k) wt[back][k] = w[(size_t)(c + k) * TAPS + TAPS - 1 - back];
+  int t = t0;
+  {
+    const int first = cu_tokens[entry_of_token[t0]];
+    if (first < t0 && t0 - first < TAPS - 1) t = min(first + TAPS - 1, cu_tokens[entry_of_token[t0] + 1]);   // taken by an earlier block
+  }
+  float past[TAPS][V];                     // past[b]: the input b tokens back (b >= 1)
+  bool fresh = true;                       // the window has to be read anew
+  int e = -1, first = 0, end = 0;
+  for (; t < n_tokens; ++t) {
+    if (e < 0 || t >= end) {
+      e = entry_of_token[t];
+      first = cu_tokens[e];
+      end = cu_tokens[e + 1];
+      fresh = true;
+    }
+    const int local = t - first;
+    if (t >= t1 && !(local < TAPS - 1 && first >= t0 && first < t1)) break;
+    if (fresh) {
+      fresh = false;
+      const int p = positions[t];
+      float* ring = TAPS > 1 ? ring_all + (size_t)state_slots[e] * TAPS * hidden + c : nullptr;
+#pragma unroll
+      for (int back = 1; back < TAPS; ++back) {
+#pragma unroll
+        for (int k = 0; k < V; ++k) past[back][k] = 0.f;
+        if (back <= local) ln_load<float, V>(h + (size_t)(t - back) * hidden + c, past[back]);
+        else if (back <= p) ln_load<float, V>(ring + (size_t)((p - back) % TAPS) * hidden, past[back]);
+      }
+      if (local == 0) {                    // the entry begins here: its last inputs into the ring (read above, by this thread)
+        const int len = end - first;
+#pragma unroll
+        for (int back = 0; back < TAPS - 1; ++back)
+          if (back < len) {
+            float u[V];
+            ln_load<float, V>(h + (size_t)(end - 1 - back) * hidden + c, u);
+            ln_store<float, V>(ring + (size_t)((p + len - 1 - back) % TAPS) * hidden, u);
+          }
+      }
+    }
+    float x[V], y[V];
+    ln_load<float, V>(h + (size_t)t * hidden + c, x);
+#pragma unroll
+    for (int k = 0; k < V; ++k) y[k] = 0.f;
+#pragma unroll
+    for (int back = TAPS - 1; back >= 1; --back)
+#pragma unroll
+      for (int k = 0; k < V; ++k) y[k] = fmaf(wt[back][k], past[back][k], y[k]);
+#pragma unroll
+    for (int k = 0; k < V; ++k) y[k] = x[k] + fmaf(wt[0][k], x[k], y[k]);
+    ln_store<TO, V>(out + (size_t)t * hidden + c, y);
+#pragma unroll
+    for (int back = TAPS - 1; back >= 2; --back)
+#pragma unroll
+      for (int k = 0; k < V; ++k) past[back][k] = past[back - 1][k];
+    if (TAPS > 1) {
+#pragma unroll
+      for (int k = 0; k < V; ++k) past[TAPS > 1 ? 1 : 0][k] = x[k];
+    }
+  }
+}
+
+template <typename TO, int V>
+static int launch_residual_conv(const float* h, const float* w, int taps, float* ring, const int* positions, const int* state_slots,
+                                const int* entry_of_token, const int* cu_tokens, void* out, int n_tokens, int hidden, int tok, hipStream_t stream) {
+  const int threads = hidden / V >= 256 ? 256 : ceil_div(ceil_div(hidden, V), kWave) * kWave;
+  dim3 grid(ceil_div(n_tokens, tok), ceil_div(ceil_div(hidden, V), threads));
+#define RC(N)                                                                                                                        \
+  case N:                                                                                                                            \
+    residual_conv_kernel<TO, N, V><<<grid, threads, 0, stream>>>(h, w, ring, positions, state_slots, entry_of_token, cu_tokens, (TO*)out, \
+                                                                 n_tokens, hidden, tok);                                             \
+    break
+  switch (taps) {
+    RC(1); RC(2); RC(3); RC(4); RC(5); RC(6); RC(7); RC(8);
+    default: return SHARPI_ERR_ARG;
+  }
+#undef RC
+  SHARPI_CHECK_LAUNCH();
+  return SHARPI_OK;
+}
+
+// h float [T, hidden]; w float [hidden, taps]; ring float [slots, taps, hidden] (null with one tap); out [T, hidden] of o_dtype.
+SHARPI_EXPORT int sharpi_residual_conv(const float* h, const float* w, int taps, float* ring, const int* positions,
+                                       const int* state_slots, const int* entry_of_token, const int* cu_tokens, void* out, int o_dtype,
+                                       int n_tokens, int hidden, hipStream_t stream) {
+  if (n_tokens <= 0) return SHARPI_OK;
+  if (hidden <= 0 || taps < 1 || taps > kLnMaxTaps || (taps > 1 && !ring) || !out) return SHARPI_ERR_ARG;
+  if (o_dtype != DT_F32 && o_dtype != DT_BF16) return SHARPI_ERR_ARG;
+  const int tok = n_tokens >= 1024 ? 8 : n_tokens >= 128 ? 4 : 1;
+  const bool by8 = hidden % 8 == 0 && ((uintptr_t)h & 31) == 0 && ((uintptr_t)out & 31) == 0 && ((uintptr_t)ring & 31) == 0;
+  if (o_dtype == DT_F32) {
+    if (by8) return launch_residual_conv<float, 8>(h, w, taps, ring, positions, state_slots, entry_of_token, cu_tokens, out, n_tokens, hidden, tok, stream);
+    return launch_residual_conv<float, 1>(h, w, taps, ring, positions, state_slots, entry_of_token, cu_tokens, out, n_tokens, hidden, tok, stream);
+  }
+  if (by8) return launch_residual_conv<bf16_t, 8>(h, w, taps, ring, positions, state_slots, entry_of_token, cu_tokens, out, n_tokens, hidden, tok, stream);
+  return launch_residual_conv<bf16_t, 1>(h, w, taps, ring, positions, state_slots, entry_of_token, cu_tokens, out, n_tokens, hidden, tok, stream);
+}
+
+// ---------------------------------------------------------------------------
+// out[t] = table[id] * scale + pairs[row], row = (previous id * mul_prev + id * mul_cur) mod buckets, or `buckets` at
+// position 0.  The previous id of an entry's first token lies in its request's slot, [slots, 2] int32, position p at
+// p mod 2; the block of that token reads it and then leaves there the id of the entry's last token.
+// ---------------------------------------------------------------------------
+template <typename T, typename TP>
+__global__ __launch_bounds__(256) void embed_bigram_kernel(const int* __restrict__ ids, const T* __restrict__ table, float scale,
+                                                           const TP* __restrict__ pairs, long long mul_prev, long long mul_cur,
+                                                           long long buckets, int* __restrict__ before, const int* __restrict__ positions,
+                                                           const int* __restrict__ state_slots, const int* __restrict__ entry_of_token,
+                                                           const int* __restrict__ cu_tokens, float* __restrict__ out, int hidden) {
+  __shared__ long long row_s;
+  const int t = blockIdx.x;
+  if (threadIdx.x == 0) {
+    const int e = entry_of_token[t], first = cu_tokens[e], p = positions[t];
+    int* mine = before + 2 * state_slots[e];
+    long long row = buckets;
+    if (p > 0) row = ((long long)(t > first ? ids[t - 1] : mine[(p - 1) & 1]) * mul_prev + (long long)ids[t] * mul_cur) % buckets;
+    row_s = row < 0 ? row + buckets : row;
+    if (t == first) {
+      const int last = cu_tokens[e + 1] - 1;
+      mine[positions[last] & 1] = ids[last];
+    }
+  }
+  __syncthreads();
+  const T* a = table + (size_t)ids[t] * hidden;
+  const TP* b = pairs + (size_t)row_s * hidden;
+  float* o = out + (size_t)t * hidden;
+  for (int i = threadIdx.x; i < hidden; i += blockDim.x) o[i] = fmaf(to_f32<T>(a[i]), scale, to_f32<TP>(b[i]));
+}
+
+SHARPI_EXPORT int sharpi_embed_bigram(const int* ids, const void* table, int t_dtype, float scale, const void* pairs, int p_dtype,
+                                      long long mul_prev, long long mul_cur, int buckets, int* before, const int* positions,
+                                      const int* state_slots, const int* entry_of_token, const int* cu_tokens, float* out, int n_tokens,
+                                      int hidden, hipStream_t stream) {
+  if (n_tokens <= 0) return SHARPI_OK;
+  if (hidden <= 0 || buckets <= 0 || !before || !pairs) return SHARPI_ERR_ARG;
+#define EB(T, TP)                                                                                                                  \
+  embed_bigram_kernel<T, TP><<<n_tokens, 256, 0, stream>>>(ids, (const T*)table, scale, (const TP*)pairs, mul_prev, mul_cur, buckets, \
+                                                           before, positions, state_slots, entry_of_token, cu_tokens, out, hidden)
+  if (t_dtype == DT_F32 && p_dtype == DT_F32) EB(float, float);
+  else if (t_dtype == DT_BF16 && p_dtype == DT_BF16) EB(bf16_t, bf16_t);
+  else if (t_dtype == DT_BF16 && p_dtype == DT_F32) EB(bf16_t, float);
+  else if (t_dtype == DT_F32 && p_dtype == DT_BF16) EB(float, bf16_t);
+  else return SHARPI_ERR_ARG;
+#undef EB
+  SHARPI_CHECK_LAUNCH();
+  return SHARPI_OK;
+}

@@ -177,7 +177,7 @@ __global__ __launch_bounds__(1024) void router_topk_kernel(const T* __restrict__
                                                            float* __restrict__ gate_out, int n_tokens, int hidden,
                                                            int n_experts, int k, int gate, int renorm,
                                                            const float* __restrict__ corr, int n_groups, int keep,
-                                                           int split_choice, const float* __restrict__ bias) {
+                                                           int split_choice, const float* __restrict__ bias, float w_scale) {
   // TT tokens per block: a router row is fetched once for all of them.
   __shared__ float g[TT][kMaxExperts];
   extern __shared__ float choice_s[];        // [TT][n_experts + n_groups] when the choice has scores of its own
@@ -202,6 +202,8 @@ __global__ __launch_bounds__(1024) void router_topk_kernel(const T* __restrict__
     gate_and_pick(g[threadIdx.x], n_experts, k, gate, renorm, topk_ids + (size_t)t * k, topk_w + (size_t)t * k,
                   gate_out ? gate_out + (size_t)t * n_experts : nullptr,
                   split_choice ? choice_s + (size_t)threadIdx.x * (n_experts + n_groups) : nullptr, corr, n_groups, keep);
+    if (w_scale != 1.0f)
+      for (int j = 0; j < k; ++j) topk_w[(size_t)t * k + j] *= w_scale;
   }
 }
 
@@ -295,10 +297,11 @@ SHARPI_EXPORT int sharpi_add_rmsnorm_router(float* h, const void* delta, const v
 // picks come from the `keep` best of n_groups equal groups of neighbouring experts (1, 1: no groups).
 // bias (float [n_experts] or null): added to the logits.  gate 0: sigmoid; 1: softmax over all experts;
 // 2: the largest logits are picked and their weights are the softmax over the picked logits alone.
+// w_scale multiplies the picks' weights at the end.
 SHARPI_EXPORT int sharpi_router_topk(const void* x, int x_dtype, const void* wr, int w_dtype, int* topk_ids,
                                      float* topk_w, float* gate_out, int n_tokens, int hidden, int n_experts,
                                      int k, int gate, int renorm, const float* corr, int n_groups, int keep,
-                                     const float* bias, hipStream_t stream) {
+                                     const float* bias, float w_scale, hipStream_t stream) {
   if (n_tokens <= 0) return SHARPI_OK;
   if (hidden <= 0 || n_experts <= 0 || n_experts > kMaxExperts || k <= 0 || k > n_experts) return SHARPI_ERR_ARG;
   if (gate < 0 || gate > 2) return SHARPI_ERR_ARG;
@@ -314,11 +317,11 @@ SHARPI_EXPORT int sharpi_router_topk(const void* x, int x_dtype, const void* wr,
     if (tt == 4)                                                                                                 \
       router_topk_kernel<TX, TWT, 4><<<grid, block, lds, stream>>>((const TX*)x, (const TWT*)wr, topk_ids, topk_w, \
                                                                  gate_out, n_tokens, hidden, n_experts, k, gate, \
-                                                                 renorm, corr, n_groups, keep, split_choice, bias);    \
+                                                                 renorm, corr, n_groups, keep, split_choice, bias, w_scale); \
     else                                                                                                         \
       router_topk_kernel<TX, TWT, 1><<<grid, block, lds, stream>>>((const TX*)x, (const TWT*)wr, topk_ids, topk_w, \
                                                                  gate_out, n_tokens, hidden, n_experts, k, gate, \
-                                                                 renorm, corr, n_groups, keep, split_choice, bias);    \
+                                                                 renorm, corr, n_groups, keep, split_choice, bias, w_scale); \
   } while (0)
   if (x_dtype == DT_F32 && w_dtype == DT_F32) ROUTER_LAUNCH(float, float);
   else if (x_dtype == DT_BF16 && w_dtype == DT_BF16) ROUTER_LAUNCH(bf16_t, bf16_t);

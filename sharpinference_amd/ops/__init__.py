@@ -460,22 +460,33 @@ def norm_add(h: torch.Tensor, delta, weight: torch.Tensor, eps: float,
     return out
 
 
-def latent_prep(proj: torch.Tensor, q_off: int, kv_off: Optional[int], q_full: torch.Tensor,
+def latent_prep(proj: Optional[torch.Tensor], q_off: int, kv_off: Optional[int], q_full: Optional[torch.Tensor],
                 rows: Optional[torch.Tensor], slot_mapping: Optional[torch.Tensor], positions: torch.Tensor,
                 inv_freq: Optional[torch.Tensor], norm_w: Optional[torch.Tensor], eps: float, nh: int, dn: int, dr: int,
-                rank: int) -> None:
+                rank: int, magnitude: float = 1.0, kv: Optional[torch.Tensor] = None,
+                q_latent: Optional[Tuple[torch.Tensor, int, torch.Tensor]] = None) -> Optional[torch.Tensor]:
     """Per token of proj [T, ld] (queries [nh, dn + dr] at column q_off, the down projection
-    [rank + dr] at column kv_off, None: this layer makes no latent): the rotated query parts go to
-    columns rank.. of every head of q_full [T, nh, rank + dr]; the latent rms_norm(first rank
-    elements) * norm_w and the rotated key part go side by side into the cache rows
-    [pages, 1, page_size, rank + dr] at slot_mapping (-1: nothing stored).  inv_freq float32
-    [pairs]: pairs (2i, 2i + 1) of the rotated parts turn by position * inv_freq[i]."""
-    _dev(proj, q_full, rows, slot_mapping, positions, inv_freq, norm_w)
+    [rank + dr] at column kv_off of `kv` (proj unless given), None: this layer makes no latent): the
+    rotated query parts go to columns rank.. of every head of q_full [T, nh, rank + dr] (None: no
+    queries yet); the latent rms_norm(first rank elements) * norm_w and the rotated key part go side
+    by side into the cache rows [pages, 1, page_size, rank + dr] at slot_mapping (-1: nothing stored).
+    inv_freq float32 [pairs]: pairs (2i, 2i + 1) of the rotated parts turn by position * inv_freq[i],
+    cos and sin times ``magnitude``.  ``q_latent`` = (source [T, ld], column, weight float32 [n]): the
+    latent that queries come through, rms_norm(its n columns) * weight, is returned as [T, n]."""
+    src = proj if q_full is not None else None
+    kv_src = None if kv_off is None else (kv if kv is not None else proj)
+    cq_src, cq_off, cq_w = q_latent if q_latent is not None else (None, 0, None)
+    _dev(src, kv_src, cq_src, cq_w, q_full, rows, slot_mapping, positions, inv_freq, norm_w)
     _i32(slot_mapping, "slot_mapping")
     _i32(positions, "positions")
-    T, ld = proj.shape
+    some = src if src is not None else kv_src if kv_src is not None else cq_src
+    _need(some is not None, "latent_prep: nothing to do")
+    T = some.shape[0]
     D = rank + dr
-    _need(q_full.shape == (T, nh * D) and q_full.dtype == proj.dtype, "latent_prep: q_full must be [T, nh * (rank + dr)] of proj's dtype")
+    _need(all(x is None or (x.dim() == 2 and x.shape[0] == T and x.dtype == some.dtype) for x in (src, kv_src, cq_src)),
+          "latent_prep: sources of one type, [T, ..]")
+    if q_full is not None:
+        _need(q_full.shape == (T, nh * D) and q_full.dtype == some.dtype, "latent_prep: q_full must be [T, nh * (rank + dr)] of proj's dtype")
     _need(positions.shape == (T,), "latent_prep: positions must be [T]")
     n_pairs = 0
     if inv_freq is not None:
@@ -483,14 +494,23 @@ def latent_prep(proj: torch.Tensor, q_off: int, kv_off: Optional[int], q_full: t
               "latent_prep: inv_freq must be float32 [pairs], 2 * pairs <= dr")
         n_pairs = inv_freq.shape[0]
     if kv_off is not None:
-        _need(rows is not None and rows.dim() == 4 and rows.shape[1] == 1 and rows.shape[3] == D and rows.dtype == proj.dtype,
+        _need(rows is not None and rows.dim() == 4 and rows.shape[1] == 1 and rows.shape[3] == D and rows.dtype == some.dtype,
               "latent_prep: cache rows must be [pages, 1, page_size, rank + dr] of proj's dtype")
         _need(slot_mapping is not None and slot_mapping.shape == (T,), "latent_prep: slot_mapping must be [T]")
         _need(norm_w is not None and norm_w.dtype == torch.float32 and norm_w.shape == (rank,), "latent_prep: norm_w must be float32 [rank]")
-    _run("sharpi_latent_prep", _ptr(proj), _code(proj.dtype), ld, int(q_off), -1 if kv_off is None else int(kv_off),
-         _ptr(q_full), _ptr(rows) if kv_off is not None else None, _ptr(slot_mapping) if kv_off is not None else None,
-         _ptr(positions), _ptr(inv_freq), n_pairs, _ptr(norm_w) if kv_off is not None else None, float(eps), T, nh, dn, dr,
-         rank, _stream())
+    cq = None
+    if cq_src is not None:
+        n = cq_w.shape[0]
+        _need(cq_w.dtype == torch.float32 and cq_w.dim() == 1 and 0 <= cq_off and cq_off + n <= cq_src.shape[1],
+              "latent_prep: the query latent's columns must lie inside its source, its weight be float32 [n]")
+        cq = torch.empty(T, n, dtype=some.dtype, device=some.device)
+    ld = lambda x: 0 if x is None else x.shape[1]
+    _run("sharpi_latent_prep", _ptr(src), ld(src), int(q_off), _ptr(kv_src), ld(kv_src), 0 if kv_off is None else int(kv_off),
+         _ptr(cq_src), ld(cq_src), int(cq_off), 0 if cq is None else cq.shape[1], _code(some.dtype), _ptr(q_full),
+         _ptr(rows) if kv_off is not None else None, _ptr(cq), _ptr(slot_mapping) if kv_off is not None else None, _ptr(positions),
+         _ptr(inv_freq), n_pairs, float(magnitude), _ptr(norm_w) if kv_off is not None else None, _ptr(cq_w), float(eps), T, nh, dn,
+         dr, rank, _stream())
+    return cq
 
 
 def head_gemm(x: torch.Tensor, x_off: int, sx: int, w: torch.Tensor, out: torch.Tensor, out_off: int, so: int,
@@ -537,14 +557,27 @@ def latent_run_keys(max_context: int, prompt_step: bool) -> int:
 
 
 def latent_mfma_ok(dtype: torch.dtype, rank: int, dr: int, window_kind: int = WINDOW_NONE) -> bool:
-    return dtype == torch.bfloat16 and window_kind == WINDOW_NONE and _lib.latent_attention_takes(rank, dr)
+    return dtype == torch.bfloat16 and window_kind in (WINDOW_NONE, WINDOW_SLIDING) and _lib.latent_attention_takes(rank, dr)
+
+
+LATENT_BLOCK_TOKENS = 64         # the most tokens of one request that a block of the matrix-core latent kernel works on
+
+
+def latent_runs(max_context: int, window: int, run: int) -> Tuple[int, int]:
+    """(runs that hold keys of one row, runs that hold keys of any row of a block) at most, for runs of `run` keys
+    and a sliding window (0: none)."""
+    every = (max_context + run - 1) // run
+    if not window:
+        return every, every
+    spans = lambda keys: (keys - 1 + run - 1) // run + 1          # runs that `keys` adjacent keys can touch
+    return min(every, spans(window)), min(every, spans(window + LATENT_BLOCK_TOKENS - 1))
 
 
 def attention_latent(q: torch.Tensor, rows: torch.Tensor, group, ctx, scale: float, nh: int, rank: int, dr: int,
                      sink: Optional[torch.Tensor] = None, window_kind: int = WINDOW_NONE, window: int = 0,
                      kernel: Optional[str] = None) -> torch.Tensor:
     """Attention of nh query heads over one shared cache row per key (rows [pages, 1, page_size,
-    rank + dr]): score = scale * q . row over all rank + dr elements, value = the row's first rank
+    rank + dr]; all earlier keys, or a window of them): score = scale * q . row over all rank + dr elements, value = the row's first rank
     elements, softmax in float with exp(sink[h]) as one more term of the denominator where sinks
     (float32 [nh]) are given.  q [T, nh * (rank + dr)] -> [T, nh * rank].  bfloat16 rows of sizes
     the matrix-core kernel takes go there (prompt tiles and single tokens from the step's work
@@ -565,14 +598,16 @@ def attention_latent(q: torch.Tensor, rows: torch.Tensor, group, ctx, scale: flo
     mfma = latent_mfma_ok(q.dtype, rank, dr, window_kind) and (ctx.n_decode or ctx.n_prefill_tiles) and group.max_context > 0
     _need(kernel in (None, "generic", "mfma") and (kernel != "mfma" or mfma), "attention_latent: this step cannot take the kernel asked for")
     if mfma and kernel != "generic":
-        run = latent_run_keys(group.max_context, bool(ctx.n_prefill_tiles))
-        max_runs = (group.max_context + run - 1) // run
+        window = int(window) if window_kind == WINDOW_SLIDING else 0
+        span = min(group.max_context, window + LATENT_BLOCK_TOKENS) if window else group.max_context
+        run = latent_run_keys(span, bool(ctx.n_prefill_tiles))
+        max_runs, grid_runs = latent_runs(group.max_context, window, run)
         part_o = part_ml = None
         if max_runs > 1:
             part_o = torch.empty(T * nh * max_runs * rank, dtype=torch.float32, device=q.device)
             part_ml = torch.empty(T * nh * max_runs * 2, dtype=torch.float32, device=q.device)
         common = (_ptr(sink), _ptr(out), _ptr(part_o), _ptr(part_ml), float(scale), nh, rank, dr, run, max_runs,
-                  rows.shape[2], group.block_table.shape[1], rows.shape[0], _stream())
+                  rows.shape[2], group.block_table.shape[1], rows.shape[0], window, grid_runs, _stream())
         if ctx.n_prefill_tiles:
             _i32(ctx.prefill_tiles, "tiles")
             _need(ctx.prefill_tiles.dim() == 2 and ctx.prefill_tiles.shape[1] == 3, "attention_latent: tiles [n, 3]")
@@ -584,7 +619,7 @@ def attention_latent(q: torch.Tensor, rows: torch.Tensor, group, ctx, scale: flo
                  _ptr(ctx.positions), None, _ptr(ctx.decode_tokens), int(ctx.n_decode), 0, *common)
         if max_runs > 1:
             _run("sharpi_attention_latent_merge", _ptr(part_o), _ptr(part_ml), _ptr(ctx.positions), None, T, _ptr(sink),
-                 _ptr(out), nh, rank, run, max_runs, _stream())
+                 _ptr(out), nh, rank, run, max_runs, window, _stream())
         return out
     _run("sharpi_attention_latent", _ptr(q), _ptr(rows), _code(q.dtype), _ptr(group.block_table), _ptr(ctx.entry_of_token),
          _ptr(ctx.positions), _ptr(sink), _ptr(out), int(window_kind), int(window), float(scale), T, nh, rank, dr,
@@ -910,7 +945,7 @@ GATE_SIGMOID, GATE_SOFTMAX, GATE_SOFTMAX_PICKED = 0, 1, 2
 
 def router_topk(x: torch.Tensor, wr: torch.Tensor, k: int, gate: int = GATE_SIGMOID, renorm: bool = False,
                 want_gates: bool = False, correction: Optional[torch.Tensor] = None, n_groups: int = 1,
-                keep_groups: int = 1, bias: Optional[torch.Tensor] = None):
+                keep_groups: int = 1, bias: Optional[torch.Tensor] = None, weight_scale: float = 1.0):
     """Router logits in float (plus ``bias``, float32 [E], where given), gate, k picks (lowest index
     wins a tie).  Gates: sigmoid, softmax over all experts, or GATE_SOFTMAX_PICKED: the largest logits are
     picked and the weights are the softmax over the picked logits alone (the gate values handed
@@ -919,7 +954,7 @@ def router_topk(x: torch.Tensor, wr: torch.Tensor, k: int, gate: int = GATE_SIGM
     ``correction`` (float32 [E]) is added to the gate values for the choice only: the weights stay
     the gate values.  With ``n_groups`` > ``keep_groups`` the experts form n_groups equal groups of
     neighbours and only those of the keep_groups best groups can be picked (a group's rank: the sum
-    of its two largest choice scores)."""
+    of its two largest choice scores).  ``weight_scale`` multiplies the weights at the end."""
     _dev(x, wr, correction, bias)
     _need(x.dim() == 2 and wr.dim() == 2 and x.shape[1] == wr.shape[1], "router: x [T, H], wr [E, H]")
     T, H = x.shape
@@ -934,7 +969,7 @@ def router_topk(x: torch.Tensor, wr: torch.Tensor, k: int, gate: int = GATE_SIGM
     wts = torch.empty(T, k, dtype=torch.float32, device=x.device)
     gates = torch.empty(T, E, dtype=torch.float32, device=x.device) if want_gates else None
     _run("sharpi_router_topk", _ptr(x), _code(x.dtype), _ptr(wr), _code(wr.dtype), _ptr(ids), _ptr(wts), _ptr(gates),
-         T, H, E, k, gate, 1 if renorm else 0, _ptr(correction), int(n_groups), int(keep_groups), _ptr(bias), _stream())
+         T, H, E, k, gate, 1 if renorm else 0, _ptr(correction), int(n_groups), int(keep_groups), _ptr(bias), float(weight_scale), _stream())
     return (ids, wts, gates) if want_gates else (ids, wts)
 
 
@@ -1025,10 +1060,10 @@ def moe_permute(ids: torch.Tensor, wts: torch.Tensor, n_experts: int, shared_gro
 
 def route(x: torch.Tensor, wr: torch.Tensor, k: int, gate: int = GATE_SIGMOID, renorm: bool = False,
           shared_group: bool = False, correction: Optional[torch.Tensor] = None, n_groups: int = 1,
-          keep_groups: int = 1, bias: Optional[torch.Tensor] = None):
+          keep_groups: int = 1, bias: Optional[torch.Tensor] = None, weight_scale: float = 1.0):
     """router_topk then moe_permute: (ids, weights, Routing)."""
     ids, wts = router_topk(x, wr, k, gate, renorm, correction=correction, n_groups=n_groups, keep_groups=keep_groups,
-                           bias=bias)
+                           bias=bias, weight_scale=weight_scale)
     return ids, wts, moe_permute(ids, wts, wr.shape[0], shared_group)
 
 
@@ -1851,4 +1886,210 @@ def map_difference(a: torch.Tensor, n_heads: int, vd: int, lam: float, eps: floa
     out = torch.empty(T, n_heads * vd, dtype=a.dtype, device=a.device)
     _run("sharpi_map_difference", _ptr(a), _code(a.dtype), float(lam), float(eps), float(post), _ptr(gate_proj), stride,
          int(gate_off), _ptr(out), T, n_heads, vd, _stream())
+    return out
+
+
+# ---------------------------------------------------------------------------
+# layer norms behind branches, convolutions over the residual sum, an embedding of token pairs
+# ---------------------------------------------------------------------------
+RESIDUAL_CONV_MAX_TAPS = 8            # csrc/layer_norm.hip kLnMaxTaps
+LAYER_NORM_MAX_WIDTH = 15 * 1024      # floats of a row that the kernel keeps in LDS
+LN_COPY, LN_NORM, LN_CONV = 0, 1, 2
+
+
+def _step_arrays_ok(ctx, T: int) -> bool:
+    return (ctx.positions.shape == (T,) and ctx.entry_of_token.shape == (T,) and ctx.state_slots.shape == (ctx.n_entries,)
+            and ctx.cu_tokens.shape == (ctx.n_entries + 1,))
+
+
+def _ring_ok(ring: Optional[torch.Tensor], taps: int, channels: int) -> bool:
+    return taps == 1 or (ring is not None and ring.dtype == torch.float32 and ring.dim() == 3 and tuple(ring.shape[1:]) == (taps, channels))
+
+
+def layer_norm(h: torch.Tensor, delta=None, weight: Optional[torch.Tensor] = None, bias: Optional[torch.Tensor] = None,
+               eps: float = 1e-5, rows: Optional[torch.Tensor] = None, out_dtype: Optional[torch.dtype] = None,
+               norm: Optional[Tuple[torch.Tensor, torch.Tensor, float]] = None,
+               conv: Optional[Tuple[torch.Tensor, Optional[torch.Tensor], object]] = None) -> Optional[torch.Tensor]:
+    """x = h + ((delta - mean) / sqrt(variance + eps) * weight + bias), back into h (float32 [T, N], all statistics and sums
+    in float); delta None: x = h.  delta: a tensor or an ExpertSum (formed on the fly, not rounded).  With ``rows``
+    (int32) only those rows are taken and h is left as it is.  With ``out_dtype`` also returns, in that storage type:
+    ``norm`` = (weight, bias, eps): the layer norm of x; ``conv`` = (w float32 [N, taps], ring float32 [slots, taps,
+    N], ctx), steps of single tokens only: x + sum_j w[:, j] x_(p - taps + 1 + j), earlier inputs from the request's
+    ring (position p at p mod taps), into which x goes; neither: x itself."""
+    lazy = delta if isinstance(delta, ExpertSum) else None
+    base = lazy.y if lazy is not None else delta
+    shared = lazy.shared if lazy is not None else None
+    wts = lazy.weights if lazy is not None else None
+    cw, ring, ctx = conv if conv is not None else (None, None, None)
+    nw, nb, neps = norm if norm is not None else (None, None, 0.0)
+    _dev(h, base, weight, bias, rows, shared, wts, cw, ring, nw, nb)
+    _i32(rows, "rows")
+    _need(h.dim() == 2 and h.dtype == torch.float32, "layer_norm: h must be float32 [T, N]")
+    T, N = h.shape
+    _need(N <= LAYER_NORM_MAX_WIDTH, f"layer_norm: rows of at most {LAYER_NORM_MAX_WIDTH} elements")
+    f32 = lambda x: x is not None and x.dtype == torch.float32 and x.shape == (N,)
+    if delta is not None:
+        _need(tuple(delta.shape) == (T, N) and base.shape[1] == N, f"layer_norm: delta {tuple(delta.shape)} vs h {tuple(h.shape)}")
+        _need(f32(weight) and f32(bias), "layer_norm: weight and bias must be float32 [N]")
+    _need(norm is None or (f32(nw) and f32(nb) and conv is None), "layer_norm: the second norm's weight and bias must be float32 [N]")
+    n = T if rows is None else rows.shape[0]
+    taps = 0
+    if conv is not None:
+        taps = cw.shape[1]
+        _need(rows is None and cw.dtype == torch.float32 and cw.shape == (N, taps) and 1 <= taps <= RESIDUAL_CONV_MAX_TAPS
+              and _ring_ok(ring, taps, N), f"layer_norm: conv w float32 [N, 1..{RESIDUAL_CONV_MAX_TAPS}], ring float32 [slots, taps, N]")
+        _need(_step_arrays_ok(ctx, T) and ctx.n_entries == T, "layer_norm: a convolution inside the norm takes steps of single tokens")
+    out = torch.empty(n, N, dtype=out_dtype, device=h.device) if out_dtype is not None else None
+    mode = LN_NORM if norm is not None else LN_CONV if conv is not None else LN_COPY
+    _need(mode == LN_COPY or out is not None, "layer_norm: an out_dtype is wanted with norm or conv")
+    _run("sharpi_layer_norm", _ptr(h), _ptr(base), _code(base.dtype) if base is not None else 0, _ptr(lazy.inv_pos) if lazy is not None else None,
+         _ptr(wts), lazy.k if lazy is not None else 0, _ptr(shared), _ptr(weight), _ptr(bias), float(eps), _ptr(rows), n, N, _ptr(out),
+         _code(out_dtype) if out is not None else 0, mode, _ptr(nw), _ptr(nb), float(neps), _ptr(cw), _ptr(ring) if taps > 1 else None, taps,
+         _ptr(ctx.positions) if conv is not None else None, _ptr(ctx.state_slots) if conv is not None else None,
+         _ptr(ctx.entry_of_token) if conv is not None else None, _stream())
+    return out
+
+
+def residual_conv(h: torch.Tensor, weight: torch.Tensor, ring: Optional[torch.Tensor], ctx, out_dtype: torch.dtype) -> torch.Tensor:
+    """h + sum_j weight[:, j] h_(t - taps + 1 + j) per token of every entry (h float32 [T, N], weight float32 [N, taps]); the
+    inputs before an entry's first token come from its request's ring (float32 [slots, taps, N], position p at p mod
+    taps), which is brought up to date; zeros before position 0."""
+    _dev(h, weight, ring)
+    T, N = h.shape
+    taps = weight.shape[1]
+    _need(h.dtype == torch.float32 and weight.dtype == torch.float32 and weight.shape == (N, taps) and 1 <= taps <= RESIDUAL_CONV_MAX_TAPS
+          and _ring_ok(ring, taps, N), f"residual_conv: h float32 [T, N], weight float32 [N, 1..{RESIDUAL_CONV_MAX_TAPS}], ring float32 [slots, taps, N]")
+    _need(_step_arrays_ok(ctx, T), "residual_conv: the step's arrays do not fit")
+    out = torch.empty(T, N, dtype=out_dtype, device=h.device)
+    _run("sharpi_residual_conv", _ptr(h), _ptr(weight), taps, _ptr(ring) if taps > 1 else None, _ptr(ctx.positions), _ptr(ctx.state_slots),
+         _ptr(ctx.entry_of_token), _ptr(ctx.cu_tokens), _ptr(out), _code(out_dtype), T, N, _stream())
+    return out
+
+
+def embed_bigram(ctx, table: torch.Tensor, pairs: torch.Tensor, mul_prev: int, mul_cur: int, before: torch.Tensor,
+                 scale: float = 1.0) -> torch.Tensor:
+    """table[id] * scale + pairs[row] per token as float32, row = (previous id * mul_prev + id * mul_cur) mod buckets
+    (buckets = rows of `pairs` - 1), or the last row at position 0.  ``before`` int32 [slots, 2] carries each request's
+    last id from step to step."""
+    _dev(ctx.token_ids, table, pairs, before)
+    _i32(ctx.token_ids, "ids")
+    _i32(before, "before")
+    T, H = ctx.n_tokens, table.shape[1]
+    _need(ctx.token_ids.shape == (T,) and _step_arrays_ok(ctx, T), "embed_bigram: the step's arrays do not fit")
+    _need(pairs.dim() == 2 and pairs.shape[1] == H and pairs.shape[0] >= 2 and before.dim() == 2 and before.shape[1] == 2,
+          "embed_bigram: pairs [buckets + 1, H], before [slots, 2]")
+    out = torch.empty(T, H, dtype=torch.float32, device=table.device)
+    _run("sharpi_embed_bigram", _ptr(ctx.token_ids), _ptr(table), _code(table.dtype), float(scale), _ptr(pairs), _code(pairs.dtype),
+         int(mul_prev), int(mul_cur), pairs.shape[0] - 1, _ptr(before), _ptr(ctx.positions), _ptr(ctx.state_slots), _ptr(ctx.entry_of_token),
+         _ptr(ctx.cu_tokens), _ptr(out), T, H, _stream())
+    return out
+
+
+# ---------------------------------------------------------------------------
+# the gated delta rule
+# ---------------------------------------------------------------------------
+DELTA_MAX_KEY_DIM, DELTA_MAX_VALUE_DIM, DELTA_MAX_TAPS = 256, 1024, 8      # csrc/delta_rule.hip
+DELTA_CHUNK_TOKENS = _lib.DELTA_CHUNK_TOKENS
+
+
+def delta_state_shape(nh: int, dk: int, dv: int) -> tuple:
+    """A request's states: [heads, ceil(dv / 16), ceil(dk / 16), 256], tile by tile; in a tile lane 16 g + j keeps rows
+    4 g .. 4 g + 3 of column j, side by side."""
+    return (nh, (dv + 15) // 16, (dk + 15) // 16, 256)
+
+
+def delta_state_matrices(state: torch.Tensor, dk: int, dv: int) -> torch.Tensor:
+    """The states as kept -> the matrices [.., heads, dk, dv] (a copy; for tests and tools)."""
+    *lead, nh, ns, nt, _ = state.shape
+    n = len(lead)
+    m = state.reshape(*lead, nh, ns, nt, 4, 16, 4)                       # [.., h, strip, tile, g, j, i]: row 16 tile + 4 g + i
+    m = m.permute(*range(n), n, n + 2, n + 3, n + 5, n + 1, n + 4)        # [.., h, tile, g, i, strip, j]
+    return m.reshape(*lead, nh, nt * 16, ns * 16)[..., :dk, :dv].contiguous()
+
+
+def lowrank(x: torch.Tensor, decay: Tuple[int, torch.Tensor, torch.Tensor, torch.Tensor],
+            plain: Optional[Tuple[int, torch.Tensor]] = None):
+    """Two products through narrow middles, columns of x (float32 [T, M]), on the float matrix instruction.  decay = (column, w
+    [N, rank], bias float32 [N], A_log float32 [heads]): -exp(A_log) softplus(x w^T + bias), float32 [T, N], N a multiple of the
+    heads.  plain = (column, w [N', rank']): x w^T in w's type.  Returns (log decays, plain or None)."""
+    off, w, bias, a_log = decay
+    off1, w1 = plain if plain is not None else (0, None)
+    _dev(x, w, bias, a_log, w1)
+    T, M = x.shape
+    N, rank = w.shape
+    _need(x.dtype == torch.float32 and 0 <= off and off + rank <= M and bias.dtype == torch.float32 and bias.shape == (N,)
+          and a_log.dtype == torch.float32 and N % a_log.shape[0] == 0, "lowrank: x float32, the middle's columns inside it, bias [N], A_log [heads]")
+    _need(w1 is None or (w1.dtype == w.dtype and 0 <= off1 and off1 + w1.shape[1] <= M), "lowrank: the second middle's columns inside x, one weight type")
+    out = torch.empty(T, N, dtype=torch.float32, device=x.device)
+    out1 = torch.empty(T, w1.shape[0], dtype=w.dtype, device=x.device) if w1 is not None else None
+    _run("sharpi_lowrank", _ptr(x), M, _code(w.dtype), T, int(off), rank, _ptr(w), N, _ptr(bias), _ptr(a_log), N // a_log.shape[0], _ptr(out),
+         int(off1), w1.shape[1] if w1 is not None else 0, _ptr(w1), w1.shape[0] if w1 is not None else 0, _ptr(out1), _stream())
+    return out, out1
+
+
+def delta_chunks_of(lens, cu_tokens):
+    """The work lists of the chunked form: (chunks int32 [n, 4] = (entry, first row, tokens, 0), ent_chunks int32
+    [entries, 2] = (first chunk, chunks)), as numpy arrays."""
+    import numpy as np
+
+    C = DELTA_CHUNK_TOKENS
+    chunks, ents = [], []
+    for e, n in enumerate(lens):
+        ents.append((len(chunks), (n + C - 1) // C))
+        chunks += [(e, int(cu_tokens[e]) + o, min(C, n - o), 0) for o in range(0, n, C)]
+    return np.asarray(chunks, dtype=np.int32).reshape(-1, 4), np.asarray(ents, dtype=np.int32).reshape(-1, 2)
+
+
+def _delta_args(proj, c_off, conv_w, ring, log_decay, beta, beta_off, state, ctx, nh, nkv, dk, dv):
+    T, N = proj.shape
+    C = 2 * nkv * dk + nh * dv
+    taps = conv_w.shape[1]
+    _dev(proj, conv_w, ring, log_decay, beta, state)
+    _need(1 <= dk <= DELTA_MAX_KEY_DIM and 1 <= dv <= DELTA_MAX_VALUE_DIM and nkv >= 1 and nh % nkv == 0,
+          f"delta rule: key channels 1..{DELTA_MAX_KEY_DIM}, value channels 1..{DELTA_MAX_VALUE_DIM}, heads a multiple of the key heads")
+    _need(0 <= c_off and c_off + C <= N, "delta rule: q, k and v must lie inside proj")
+    _need(conv_w.dtype == torch.float32 and conv_w.shape == (C, taps) and 1 <= taps <= DELTA_MAX_TAPS and _ring_ok(ring, taps, C),
+          f"delta rule: conv_w float32 [channels, 1..{DELTA_MAX_TAPS}], ring float32 [slots, taps, channels]")
+    _need(log_decay.dtype == torch.float32 and log_decay.shape == (T, nh * dk), "delta rule: log_decay float32 [T, nh * dk]")
+    _need(beta.dtype == torch.float32 and beta.dim() == 2 and beta.shape[0] == T and 0 <= beta_off and beta_off + nh <= beta.shape[1],
+          "delta rule: beta float32 [T, ..] with a column per head")
+    _need(state.dtype == torch.float32 and tuple(state.shape[1:]) == delta_state_shape(nh, dk, dv), "delta rule: state float32 [slots, *delta_state_shape]")
+    _need(_step_arrays_ok(ctx, T) and ctx.n_tokens == T, "delta rule: the step's arrays do not fit")
+    return (_ptr(proj), _code(proj.dtype), N, int(c_off), _ptr(conv_w), taps, _ptr(ring) if taps > 1 else None, _ptr(log_decay), _ptr(beta),
+            beta.shape[1], int(beta_off), _ptr(ctx.positions), _ptr(ctx.state_slots), _ptr(ctx.cu_tokens), _ptr(state), ctx.n_entries, nh, nkv,
+            dk, dv, float(dk) ** -0.5)
+
+
+def delta_step(proj: torch.Tensor, c_off: int, conv_w: torch.Tensor, ring: Optional[torch.Tensor], log_decay: torch.Tensor,
+               beta: torch.Tensor, beta_off: int, state: torch.Tensor, ctx, nh: int, nkv: int, dk: int, dv: int,
+               norm_w: torch.Tensor, eps: float, gate: Optional[torch.Tensor]) -> torch.Tensor:
+    """The gated delta rule for a step of single tokens, from the projected channels (q | k | v from column c_off of proj) to
+    the heads' normed and gated outputs [T, nh * dv] of proj's dtype: convolution + SiLU (ring: the requests' last
+    inputs), unit q and k (q times dk^-1/2), S <- exp(log_decay) S, u = sigmoid(beta) (v - S^T k), S <- S + k u^T, o = S^T q,
+    o / rms(o) * norm_w * sigmoid(gate).  Head h reads key head h // (nh / nkv)."""
+    args = _delta_args(proj, c_off, conv_w, ring, log_decay, beta, beta_off, state, ctx, nh, nkv, dk, dv)
+    _dev(norm_w, gate)
+    T = proj.shape[0]
+    _need(ctx.n_entries == T, "delta_step: every entry brings one token")
+    _need(norm_w.dtype == torch.float32 and norm_w.shape == (dv,) and (gate is None or (gate.dtype == proj.dtype and gate.shape == (T, nh * dv))),
+          "delta_step: norm_w float32 [dv], gate [T, nh * dv] of proj's dtype")
+    out = torch.empty(T, nh * dv, dtype=proj.dtype, device=proj.device)
+    _run("sharpi_delta_step", *args, _ptr(norm_w), float(eps), _ptr(gate), _ptr(out), _stream())
+    return out
+
+
+def delta_chunks(proj: torch.Tensor, c_off: int, conv_w: torch.Tensor, ring: Optional[torch.Tensor], log_decay: torch.Tensor,
+                 beta: torch.Tensor, beta_off: int, state: torch.Tensor, ctx, nh: int, nkv: int, dk: int, dv: int, lists) -> torch.Tensor:
+    """The same recurrence for entries of any length, 16 tokens at a time (lists: ``delta_chunks_of`` on the device): o
+    float32 [T, nh * dv], neither normed nor gated."""
+    args = _delta_args(proj, c_off, conv_w, ring, log_decay, beta, beta_off, state, ctx, nh, nkv, dk, dv)
+    chunks, ents = lists
+    _dev(chunks, ents)
+    _i32(chunks, "chunks")
+    _i32(ents, "ent_chunks")
+    n = chunks.numel() // 4
+    _need(chunks.numel() == 4 * n and ents.numel() == 2 * ctx.n_entries and n >= ctx.n_entries, "delta_chunks: chunks [n, 4], ent_chunks [entries, 2]")
+    work = torch.empty(_lib.delta_chunk_floats(n, nh, dk, dv), dtype=torch.float32, device=proj.device)
+    out = torch.empty(proj.shape[0], nh * dv, dtype=torch.float32, device=proj.device)
+    _run("sharpi_delta_chunks", *args, _ptr(chunks), _ptr(ents), n, _ptr(work), _ptr(out), _stream())
     return out

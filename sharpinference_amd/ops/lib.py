@@ -36,13 +36,13 @@ _SIGNATURES = {
     "sharpi_gemm_skinny_swiglu": [P, P, P, I, I, I, P, P, I, P, I, I, I, I, I, F, P],
     "sharpi_gemm_skinny_picked": [P, P, P, I, I, I, P, P, I, I, I, I, I, I, F, I, I, I, P],
     "sharpi_add_rmsnorm_router": [P, P, P, I, P, I, I, F, P, I, P, P, I, I, I, I, P],
-    "sharpi_router_topk": [P, I, P, I, P, P, P, I, I, I, I, I, I, P, I, I, P, P],
+    "sharpi_router_topk": [P, I, P, I, P, P, P, I, I, I, I, I, I, P, I, I, P, F, P],
     "sharpi_norm_add": [P, P, I, P, P, I, I, I, F, P, P, I, P],
-    "sharpi_latent_prep": [P, I, I, I, I, P, P, P, P, P, I, P, F, I, I, I, I, I, P],
+    "sharpi_latent_prep": [P, I, I, P, I, I, P, I, I, I, I, P, P, P, P, P, P, I, F, P, P, F, I, I, I, I, I, P],
     "sharpi_head_gemm": [P, I, I, I, P, P, I, I, P, I, I, I, I, I, P],
     "sharpi_attention_latent": [P, P, I, P, P, P, P, P, I, I, F, I, I, I, I, I, I, I, P],
-    "sharpi_attention_latent_mfma": [P, P, P, P, P, P, P, I, I, P, P, P, P, F, I, I, I, I, I, I, I, I, P],
-    "sharpi_attention_latent_merge": [P, P, P, P, I, P, P, I, I, I, I, P],
+    "sharpi_attention_latent_mfma": [P, P, P, P, P, P, P, I, I, P, P, P, P, F, I, I, I, I, I, I, I, I, I, I, P],
+    "sharpi_attention_latent_merge": [P, P, P, P, I, P, P, I, I, I, I, I, P],
     "sharpi_moe_permute": [P, P, P, P, P, P, P, I, I, I, I, I, P],
     "sharpi_gemm_grouped": [P, I, P, P, I, I, I, I, P, P, P, I, I, I, P],
     "sharpi_gemm_grouped_swiglu": [P, I, P, P, I, I, I, P, P, P, I, P, I, I, F, I, P],
@@ -66,6 +66,12 @@ _SIGNATURES = {
     "sharpi_stream_add": [P, P, P, I, I, P, I, c_longlong, P],
     "sharpi_side_gate": [P, I, P, P, I, I, I, P, I, I, P],
     "sharpi_hyper_step": [P, c_longlong, c_longlong, P, P, I, P, P, P, I, P, P, P, P, I, F, P, I, P, I, I, I, P],
+    "sharpi_layer_norm": [P, P, I, P, P, I, P, P, P, F, P, I, I, P, I, I, P, P, F, P, P, I, P, P, P, P],
+    "sharpi_residual_conv": [P, P, I, P, P, P, P, P, P, I, I, I, P],
+    "sharpi_embed_bigram": [P, P, I, F, P, I, c_longlong, c_longlong, I, P, P, P, P, P, P, I, I, P],
+    "sharpi_lowrank": [P, I, I, I, I, I, P, I, P, P, I, P, I, I, P, I, P, P],
+    "sharpi_delta_step": [P, I, I, I, P, I, P, P, P, I, I, P, P, P, P, I, I, I, I, I, F, P, F, P, P, P],
+    "sharpi_delta_chunks": [P, I, I, I, P, I, P, P, P, I, I, P, P, P, P, I, I, I, I, I, F, P, P, I, P, P, P],
     "sharpi_map_difference": [P, I, F, F, F, P, I, I, P, I, I, I, P],
 }
 
@@ -81,6 +87,7 @@ FUSED_NORM_ROUTER_MAX_HIDDEN = 8192   # widest row of the norm + router kernel
 ROUTER_MAX_EXPERTS = 1024   # experts the routing kernels hold scores for
 GLA_STATE_COLS = 8          # value columns of a linear-attention state that lie together in memory
 WALK_STATE_COLS = 8         # value columns of a slice of a scalar-decay recurrent state (csrc/state_walk.hip)
+DELTA_CHUNK_TOKENS = 16     # tokens of a chunk of the gated delta rule (csrc/delta_rule.hip)
 _BUILT_WITH = {
     "sharpi_attention_decode_split_keys": DECODE_RUN_KEYS,
     "sharpi_attention_prefill_tile_tokens": PREFILL_TILE_TOKENS,
@@ -89,6 +96,7 @@ _BUILT_WITH = {
     "sharpi_add_rmsnorm_router_max_hidden": FUSED_NORM_ROUTER_MAX_HIDDEN,
     "sharpi_gla_state_cols": GLA_STATE_COLS,
     "sharpi_state_walk_cols": WALK_STATE_COLS,
+    "sharpi_delta_chunk_tokens": DELTA_CHUNK_TOKENS,
 }
 
 
@@ -159,6 +167,13 @@ def latent_attention_takes(rank: int, dr: int) -> bool:
         fn.argtypes, fn.restype = [c_int, c_int], c_int
         _takes[key] = bool(fn(int(rank), int(dr)))
     return _takes[key]
+
+
+def delta_chunk_floats(n_chunks: int, nh: int, dk: int, dv: int) -> int:
+    """Scratch floats of the gated delta rule's chunked form."""
+    fn = load().sharpi_delta_chunk_floats
+    fn.argtypes, fn.restype = [c_int] * 4, c_longlong
+    return int(fn(int(n_chunks), int(nh), int(dk), int(dv)))
 
 
 def grouped_tile_rows() -> int:

@@ -6,6 +6,7 @@ from typing import Dict
 import torch
 
 from .. import ops
+from ..cache.spec import combine_specs, states_of
 from ..ops.profile import section
 from .base import LayerCache, ParamSpec, Part, ResidualStream, StepContext, TensorSource
 
@@ -61,8 +62,6 @@ class PreNormBlock(Part):
     def decode_graph_safe(self) -> bool:
         """Can a decode step through this block be captured into a graph?  Paged attention can; a
         mixer with state of its own says so itself (``graph_safe``)."""
-        from ..cache.spec import states_of
-
         return not states_of(self.cache_spec()) or bool(getattr(self.mixer, "graph_safe", False))
 
     def forward(self, stream: ResidualStream, ctx: StepContext, cache: LayerCache) -> None:
@@ -110,6 +109,51 @@ class PostNormBlock(PreNormBlock):
         if self.ffn is not None:
             y = self.ffn.forward(stream.act, ctx)
             self.norm2.add_normed(stream, y, ctx.act_dtype)
+
+
+class ConvPostNormBlock(PreNormBlock):
+    """h += norm1(mixer(c1(h))); h += norm2(ffn(c2(h))): norms on the branches' outputs, and a short convolution over the
+    residual sum in front of each branch (parts/conv.py).  ``ffn`` None: a layer of a mixer alone.  A branch's output is
+    left waiting behind its norm (``stream.pending_norm``) for the next branch's convolution, for the model's last norm, or
+    for whoever settles the stream.  The convolutions' rings follow the mixer's own states in the layer's memory; a layer whose
+    pages are another layer's (``Run.kv_from``) still keeps them itself."""
+
+    def __init__(self, conv1: Part, mixer: Part, norm1: Part, conv2: Part = None, ffn: Part = None, norm2: Part = None, names=None):
+        if not ((conv2 is None) == (ffn is None) == (norm2 is None)):
+            raise ValueError("a feed-forward, its convolution and its norm come together")
+        super().__init__(norm1, mixer, norm2, ffn, names or {"conv1": "conv1.", "mixer": "mixer.", "norm1": "norm1.", "conv2": "conv2.",
+                                                             "ffn": "ffn.", "norm2": "norm2."})
+        self.conv1, self.conv2 = conv1, conv2
+
+    def _children(self):
+        kids = list(super()._children()) + [(self.names["conv1"], self.conv1)]
+        if self.conv2 is not None:
+            kids.append((self.names["conv2"], self.conv2))
+        return tuple(kids)
+
+    def _mixer_spec(self):
+        spec = getattr(self.mixer, "cache_spec", None)
+        return spec() if spec else None
+
+    def cache_spec(self):
+        return combine_specs([s for s in (self._mixer_spec(), self.conv1.cache_spec(), self.conv2.cache_spec() if self.conv2 else None)
+                              if s is not None])
+
+    def decode_graph_safe(self) -> bool:
+        return not states_of(self._mixer_spec()) or bool(getattr(self.mixer, "graph_safe", False))
+
+    def forward(self, stream: ResidualStream, ctx: StepContext, cache: LayerCache) -> None:
+        n = len(states_of(self._mixer_spec()))
+        mine, rings = list(cache.states[:n]), list(cache.states[n:])
+        ring1 = rings.pop(0) if self.conv1.cache_spec() is not None else None
+        ring2 = rings.pop(0) if self.conv2 is not None and self.conv2.cache_spec() is not None else None
+        sub = LayerCache(group=cache.group, k=cache.k, v=cache.v, state=mine[0] if mine else None, write=cache.write, states=mine)
+        stream.act = None
+        x = self.conv1.forward(stream, ctx, ring1)
+        stream.pending, stream.pending_norm = self.mixer.forward(x, ctx, sub), self.norm1
+        if self.ffn is not None:
+            x = self.conv2.forward(stream, ctx, ring2)
+            stream.pending, stream.pending_norm = self.ffn.forward(x, ctx), self.norm2
 
 
 class SandwichBlock(PreNormBlock):

@@ -134,7 +134,8 @@ class MoESwiGLU(Part):
     experts' gate function ("silu", the reference's, "gelu_tanh", or "swish_clamp" with ``limit``; the
     shared expert may have a limit and a width of its own, ``shared_limit``).  ``gate`` "softmax_picked":
     the largest logits are picked and their weights are the softmax over the picked logits alone.
-    ``router_bias``: a stored vector [E] is added to the router's logits."""
+    ``router_bias``: a stored vector [E] is added to the router's logits.  ``weight_scale`` multiplies the picks' weights
+    (after any division by their sum)."""
 
     MERGE_MAX_TOKENS = 16   # one row block of the few-rows kernel for the shared group (measured: up to 64 tokens
                             # the merged launches and the library's product for the shared expert are as fast)
@@ -150,7 +151,8 @@ class MoESwiGLU(Part):
                  shared_intermediate: Optional[int] = None, gate: str = "sigmoid", renormalise: bool = False,
                  score_on_input: bool = True, activation: str = "silu", correction: bool = False,
                  n_groups: int = 1, keep_groups: int = 1, names: Optional[Dict[str, str]] = None,
-                 limit: Optional[float] = None, shared_limit: Optional[float] = None, router_bias: bool = False):
+                 limit: Optional[float] = None, shared_limit: Optional[float] = None, router_bias: bool = False,
+                 weight_scale: float = 1.0):
         """``correction``: a stored vector [E] is added to the gate values where experts are chosen
         (the weights stay the gate values).  ``n_groups`` / ``keep_groups``: the experts form
         n_groups equal groups of neighbours and are chosen from the keep_groups best of them only
@@ -178,6 +180,7 @@ class MoESwiGLU(Part):
                                   names={k[len("shared_"):]: v for k, v in shared_names.items()} or None) if shared_intermediate else None
         self.gate = {"sigmoid": ops.GATE_SIGMOID, "softmax": ops.GATE_SOFTMAX, "softmax_picked": ops.GATE_SOFTMAX_PICKED}[gate]
         self.router_bias = bool(router_bias)
+        self.weight_scale = float(weight_scale)
         self.b_router: Optional[torch.Tensor] = None      # float32 [E]
         self.renormalise = bool(renormalise)
         self.score_on_input = bool(score_on_input)
@@ -216,7 +219,8 @@ class MoESwiGLU(Part):
         return out
 
     def _route_args(self) -> dict:
-        return dict(correction=self.w_correction, n_groups=self.n_groups, keep_groups=self.keep_groups, bias=self.b_router)
+        return dict(correction=self.w_correction, n_groups=self.n_groups, keep_groups=self.keep_groups, bias=self.b_router,
+                    weight_scale=self.weight_scale)
 
     def load(self, prefix: str, source: TensorSource) -> None:
         self.w_router = source.get(prefix + self.names["router"])
@@ -306,7 +310,7 @@ class MoESwiGLU(Part):
         few decode tokens the norm and the router are one launch (the bits of the two)."""
         T = stream.h.shape[0]
         plain_choice = (self.w_correction is None and self.keep_groups == self.n_groups and self.b_router is None
-                        and self.gate != ops.GATE_SOFTMAX_PICKED)   # what the fused kernel picks by
+                        and self.gate != ops.GATE_SOFTMAX_PICKED and self.weight_scale == 1.0)   # what the fused kernel picks by
         if (self._few_tokens(T, ctx) and isinstance(norm, RMSNorm) and plain_choice
                 and ops.norm_router_ok(stream.h, stream.pending, ctx.act_dtype)):
             with section("norm + router", nbytes=T * self.hidden * 10 + 2 * self.E * self.hidden):

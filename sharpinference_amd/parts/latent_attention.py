@@ -1,7 +1,7 @@
 """The latent attention mixer: keys and values of all heads kept as one low-rank row per token."""
 from __future__ import annotations
 
-from typing import Dict, Optional
+from typing import Dict, Optional, Tuple
 
 import torch
 
@@ -26,16 +26,23 @@ class LatentAttention(Part):
     float, with ``sink``: one learned term exp(sink_h) more in the denominator, without key or
     value.  With ``gate`` the heads' outputs are multiplied by sigmoid(W_g h) before W_o.
 
+    ``q_rank``: queries come through a latent of their own, q = W_uq rms_norm(W_dq h) (weight
+    ``dq.norm``), instead of W_q h.
+
     ``own_latent=False``: the layer has no W_dkv and attends over the rows another layer stored
-    (the schedule hands it that layer's cache with ``write=False``).  ``rotary``: any object with
-    ``table(device)`` (float32 frequencies of the rotated pairs (2i, 2i + 1), at most dr / 2).
+    (the schedule hands it that layer's cache with ``write=False``).  ``window_kind`` / ``window``: which
+    keys this layer sees; ``kept`` (kind, window): which the shared rows have to be kept for, where layers
+    with different windows read them (default: this layer's own).  ``rotary``: any object with
+    ``table(device)`` (float32 frequencies of the rotated pairs (2i, 2i + 1), at most dr / 2) and a
+    ``magnitude`` (of cos and sin).
     """
 
-    NAMES = {"q": "q", "dkv": "dkv", "dkv_norm": "dkv.norm", "uk": "uk", "uv": "uv", "sink": "sink", "g": "g", "o": "o"}
+    NAMES = {"q": "q", "dq": "dq", "dq_norm": "dq.norm", "uq": "uq", "dkv": "dkv", "dkv_norm": "dkv.norm", "uk": "uk", "uv": "uv", "sink": "sink", "g": "g", "o": "o"}
 
     def __init__(self, hidden: int, num_heads: int, nope_dim: int, rope_dim: int, v_dim: int, rank: int, rotary,
                  norm_eps: float, scale: float, sink: bool = True, gate: bool = True, own_latent: bool = True,
-                 window_kind: int = WINDOW_NONE, window: int = 0, names: Optional[Dict[str, str]] = None):
+                 window_kind: int = WINDOW_NONE, window: int = 0, names: Optional[Dict[str, str]] = None,
+                 q_rank: Optional[int] = None, kept: Optional[Tuple[int, int]] = None):
         if rank < 1 or rank > ops.LATENT_MAX_RANK:
             raise ValueError(f"a latent of {rank} elements is not taken: 1 to {ops.LATENT_MAX_RANK}")
         if min(num_heads, nope_dim, rope_dim, v_dim) < 1:
@@ -47,8 +54,14 @@ class LatentAttention(Part):
         self.rotary, self.eps, self.scale = rotary, float(norm_eps), float(scale)
         self.has_sink, self.has_gate, self.own_latent = bool(sink), bool(gate), bool(own_latent)
         self.window_kind, self.window = int(window_kind), int(window)
+        self.kept = (self.window_kind, self.window) if kept is None else (int(kept[0]), int(kept[1]))
+        self.q_rank = int(q_rank) if q_rank else 0
+        if self.q_rank < 0:
+            raise ValueError("the query latent's width must be positive")
+        self.w_uq = None
+        self.w_q_norm: Optional[torch.Tensor] = None       # float32 [q_rank]
         self.names = {**self.NAMES, **(names or {})}
-        self.w_in = None                                   # [q | g | dkv] rows: one product of the input
+        self.w_in = None                                   # [q (or dq) | g | dkv] rows: one product of the input
         self.w_uk_t: Optional[torch.Tensor] = None         # [heads, rank, dn]: W_uk per head, transposed
         self.w_uv: Optional[torch.Tensor] = None           # [heads, dv, rank]
         self.w_o = None
@@ -60,7 +73,7 @@ class LatentAttention(Part):
         return (_WORK_LISTS,)
 
     def cache_spec(self) -> KVSpec:
-        return KVSpec(1, self.rank + self.dr, self.window_kind, self.window, self.rank, values_in_keys=True)
+        return KVSpec(1, self.rank + self.dr, *self.kept, self.rank, values_in_keys=True)
 
     @property
     def q_dim(self) -> int:
@@ -73,11 +86,16 @@ class LatentAttention(Part):
     def param_specs(self, prefix: str) -> Dict[str, ParamSpec]:
         n = self.names
         specs = {
-            prefix + n["q"]: ParamSpec((self.q_dim, self.hidden)),
             prefix + n["uk"]: ParamSpec((self.nh * self.dn, self.rank)),
             prefix + n["uv"]: ParamSpec((self.o_dim, self.rank)),
             prefix + n["o"]: ParamSpec((self.hidden, self.o_dim)),
         }
+        if self.q_rank:
+            specs[prefix + n["dq"]] = ParamSpec((self.q_rank, self.hidden))
+            specs[prefix + n["dq_norm"]] = ParamSpec((self.q_rank,), "norm_weight")
+            specs[prefix + n["uq"]] = ParamSpec((self.q_dim, self.q_rank))
+        else:
+            specs[prefix + n["q"]] = ParamSpec((self.q_dim, self.hidden))
         if self.own_latent:
             specs[prefix + n["dkv"]] = ParamSpec((self.rank + self.dr, self.hidden))
             specs[prefix + n["dkv_norm"]] = ParamSpec((self.rank,), "norm_weight")
@@ -89,7 +107,10 @@ class LatentAttention(Part):
 
     def load(self, prefix: str, source: TensorSource) -> None:
         n = self.names
-        parts = [source.get(prefix + n["q"])]
+        parts = [source.get(prefix + n["dq" if self.q_rank else "q"])]
+        if self.q_rank:
+            self.w_q_norm = source.get(prefix + n["dq_norm"]).float().contiguous()
+            self.w_uq = ops.pack_weight(source.get(prefix + n["uq"]))
         if self.has_gate:
             parts.append(source.get(prefix + n["g"]))
         if self.own_latent:
@@ -116,8 +137,8 @@ class LatentAttention(Part):
         D = self.rank + self.dr
         width = 2 if ctx.act_dtype == torch.bfloat16 else 4
         n_in = self.w_in.shape[0]
-        g_off = self.q_dim
-        kv_off = self.q_dim + (self.o_dim if self.has_gate else 0)
+        g_off = self.q_rank or self.q_dim
+        kv_off = g_off + (self.o_dim if self.has_gate else 0)
         with section("q|g|dkv", nbytes=width * n_in * (self.hidden + T) + width * T * self.hidden, flops=2.0 * T * self.hidden * n_in):
             proj = ops.linear(x, self.w_in, ctx.act_dtype)
         store = self.own_latent and cache.write
@@ -125,12 +146,24 @@ class LatentAttention(Part):
             raise ValueError("a latent layer with a down projection of its own must own its cache")
         q_full = torch.empty(T, self.nh * D, dtype=ctx.act_dtype, device=x.device)
         inv_freq = self.rotary.table(x.device) if self.rotary is not None else None
-        with section("latent + rotary + cache write", nbytes=width * T * (2 * self.nh * self.dr + 2 * D)):
-            ops.latent_prep(proj, 0, kv_off if store else None, q_full, cache.k, g.slot_mapping if store else None,
-                            ctx.positions, inv_freq, self.w_norm, self.eps, self.nh, self.dn, self.dr, self.rank)
+        rows = (cache.k, g.slot_mapping) if store else (None, None)
+        common = (ctx.positions, inv_freq, self.w_norm, self.eps, self.nh, self.dn, self.dr, self.rank)
+        magnitude = getattr(self.rotary, "magnitude", 1.0)
+        if self.q_rank:
+            with section("latents + cache write", nbytes=width * T * (2 * self.q_rank + 2 * D)):
+                cq = ops.latent_prep(None, 0, kv_off if store else None, None, *rows, *common, magnitude=magnitude, kv=proj,
+                                     q_latent=(proj, 0, self.w_q_norm))
+            with section("uq", nbytes=width * (self.q_dim * self.q_rank + T * (self.q_rank + self.q_dim)), flops=2.0 * T * self.q_dim * self.q_rank):
+                q = ops.linear(cq, self.w_uq, ctx.act_dtype)
+            with section("rotary", nbytes=width * T * 2 * self.nh * self.dr):
+                ops.latent_prep(q, 0, None, q_full, None, None, *common, magnitude=magnitude)
+        else:
+            q = proj
+            with section("latent + rotary + cache write", nbytes=width * T * (2 * self.nh * self.dr + 2 * D)):
+                ops.latent_prep(q, 0, kv_off if store else None, q_full, *rows, *common, magnitude=magnitude)
         with section("q through uk", nbytes=width * (self.nh * self.dn * self.rank + T * self.nh * (self.dn + self.rank)),
                      flops=2.0 * T * self.nh * self.dn * self.rank):
-            ops.head_gemm(proj, 0, self.dn + self.dr, self.w_uk_t, q_full, 0, D)
+            ops.head_gemm(q, 0, self.dn + self.dr, self.w_uk_t, q_full, 0, D)
         with section("attention", nbytes=lambda: self._keys_held(ctx) * D * width + T * self.nh * (D + self.rank) * width,
                      flops=lambda: 2.0 * self._keys_read(ctx) * self.nh * (D + self.rank)):
             o_lat = ops.attention_latent(q_full, cache.k, g, ctx, self.scale, self.nh, self.rank, self.dr, sink=self.w_sink,
@@ -143,9 +176,9 @@ class LatentAttention(Part):
             return ops.linear(o, self.w_o, ctx.act_dtype)
 
     def _keys_read(self, ctx: StepContext) -> int:
-        spec = self.cache_spec()
+        spec = KVSpec(1, 1, self.window_kind, self.window)
         return sum(p - spec.first_visible(p) + 1 for s, n in zip(ctx.entry_starts, ctx.entry_lens) for p in range(s, s + n))
 
     def _keys_held(self, ctx: StepContext) -> int:
-        spec = self.cache_spec()
+        spec = KVSpec(1, 1, self.window_kind, self.window)
         return sum(s + n - spec.first_visible(s) for s, n in zip(ctx.entry_starts, ctx.entry_lens))

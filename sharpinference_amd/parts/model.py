@@ -7,6 +7,7 @@ from typing import Dict, List, Optional, Sequence, Tuple
 import torch
 
 from .. import ops
+from ..cache.spec import MixedSpec, kv_of, states_of
 from ..ops.profile import section
 from .base import LayerCache, ParamSpec, Part, ResidualStream, StepContext, TensorSource
 from .norm import RMSNorm
@@ -21,12 +22,15 @@ class Run:
     values that the slot's owner stored earlier in the same step and store nothing.
     ``add_row`` = (table, r): before the layer runs, row r of the model's tensor `table` (one of its
     ``row_tables``, [rows, hidden]) is added to every token's residual sum, in float: a learned
-    vector that marks, say, which pass of a repeated stretch of layers begins here."""
+    vector that marks, say, which pass of a repeated stretch of layers begins here.
+    ``kv_from``: the entry has a cache slot of its own for the fixed-size states its layer keeps, but
+    reads the pages of slot `kv_from` (which an earlier entry has written) and stores none."""
 
     layer: int
     cache: int
     write: bool = True
     add_row: Optional[Tuple[str, int]] = None
+    kv_from: Optional[int] = None
 
 
 class DecoderModel(Part):
@@ -42,7 +46,10 @@ class DecoderModel(Part):
                  layer_prefix: str = "model.layers.", embed_name: str = "model.embed_tokens.weight",
                  norm_prefix: str = "model.norm.", head_name: str = "lm_head.weight", embedding_scale: float = 1.0,
                  logit_scale: float = 1.0, logit_softcap: Optional[float] = None,
-                 row_tables: Optional[Dict[str, int]] = None, shared: Sequence[Part] = ()):
+                 row_tables: Optional[Dict[str, int]] = None, shared: Sequence[Part] = (), embedding: Optional[Part] = None):
+        # a part that makes the first residual sum from the step's tokens and the table (parts/embedding.py); what it
+        # keeps per request lies in a cache slot behind the layers' (None: the token's row times embedding_scale)
+        self.embedding = embedding
         self.shared = list(shared)       # tensors that several parts read (parts/token_side.py:SharedTensor), loaded once
         self.row_tables: Dict[str, int] = dict(row_tables or {})      # name -> rows of a [rows, hidden] tensor
         self._row_table_f32: Dict[str, torch.Tensor] = {}
@@ -78,6 +85,11 @@ class DecoderModel(Part):
                 if r.cache in owner:
                     raise ValueError(f"cache slot {r.cache} is written by two entries of the schedule")
                 owner[r.cache] = r.layer
+                if r.kv_from is not None:
+                    if r.kv_from not in owner or r.kv_from == r.cache:
+                        raise ValueError(f"cache slot {r.kv_from} is read before any entry has written it")
+                    if kv_of(self.blocks[owner[r.kv_from]].cache_spec()) != kv_of(spec):
+                        raise ValueError(f"layer {r.layer} reads the pages of layer {owner[r.kv_from]}, whose shape differs")
             else:
                 if r.cache not in owner:
                     raise ValueError(f"cache slot {r.cache} is read before any entry has written it")
@@ -86,6 +98,7 @@ class DecoderModel(Part):
 
     # -- cache ------------------------------------------------------------------
     def num_cache_slots(self) -> int:
+        """The layers' cache slots (an embedding with a memory of its own has one more behind them)."""
         return 1 + max((r.cache for r in self.schedule), default=-1)
 
     def cache_specs(self) -> list:
@@ -93,7 +106,13 @@ class DecoderModel(Part):
         specs = [None] * self.num_cache_slots()
         for r in self.schedule:
             if r.write:
-                specs[r.cache] = self.blocks[r.layer].cache_spec()
+                spec = self.blocks[r.layer].cache_spec()
+                if r.kv_from is not None:          # the pages are another slot's: the states alone
+                    own = states_of(spec)
+                    spec = MixedSpec(None, own) if own else None
+                specs[r.cache] = spec
+        if self.embedding is not None:
+            specs.append(self.embedding.cache_spec())
         return specs
 
     def decode_graph_safe(self) -> bool:
@@ -115,6 +134,8 @@ class DecoderModel(Part):
         for i, b in enumerate(self.blocks):
             out.update(b.param_specs(f"{self.layer_prefix}{i}."))
         out.update(self.final_norm.param_specs(self.norm_prefix))
+        if self.embedding is not None:
+            out.update(self.embedding.param_specs(""))
         for part in self.shared:
             out.update(part.param_specs(""))
         for name, rows in self.row_tables.items():
@@ -125,6 +146,8 @@ class DecoderModel(Part):
 
     def load_weights(self, source: TensorSource) -> None:
         self.embed = source.get(self.embed_name)
+        if self.embedding is not None:
+            self.embedding.load("", source)
         for part in self.shared:
             part.load("", source)
         for i, b in enumerate(self.blocks):
@@ -145,7 +168,11 @@ class DecoderModel(Part):
         (the reference keeps such a path for all-greedy batches,
         src/SharpInference.Engine/CudaForwardPass.cs:1574-1583)."""
         with section("embed", nbytes=ctx.n_tokens * self.hidden * 6):
-            stream = ResidualStream(ops.embed_gather(ctx.token_ids, self.embed, scale=self.embedding_scale))
+            if self.embedding is not None:
+                h = self.embedding.forward(ctx, self.embed, self.embedding_scale, caches[-1])
+            else:
+                h = ops.embed_gather(ctx.token_ids, self.embed, scale=self.embedding_scale)
+            stream = ResidualStream(h)
         for r in self.schedule:
             c = caches[r.cache]
             if r.add_row is not None:
@@ -156,6 +183,9 @@ class DecoderModel(Part):
                     ops.add_bias(stream.h, self._row_table_f32[r.add_row[0]][r.add_row[1]])
             if not r.write:
                 c = LayerCache(c.group, c.k, c.v, c.state, write=False, states=c.states)
+            elif r.kv_from is not None:
+                src = caches[r.kv_from]
+                c = LayerCache(src.group, src.k, src.v, c.state, write=False, states=c.states)
             self.blocks[r.layer].forward(stream, ctx, c)
         if logit_rows is None or logit_rows.numel() == 0:
             return None

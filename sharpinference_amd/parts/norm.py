@@ -10,6 +10,54 @@ from ..ops.profile import section
 from .base import INIT_NORM_WEIGHT, ParamSpec, Part, ResidualStream, TensorSource
 
 
+class LayerNorm(Part):
+    """(x - mean) / sqrt(variance + eps) * w + b over the last axis, the variance the mean of the squared deviations;
+    statistics and sums in float.  ``name``: the weight's name behind the part's prefix (the bias adds
+    ``bias_suffix``).  As the norm on a branch's output (``add_normed``) or as a norm of the stream itself."""
+
+    def __init__(self, dim: int, eps: float, name: str = "weight", bias_suffix: str = ".b"):
+        self.dim, self.eps, self.name, self.bias_suffix = int(dim), float(eps), name, bias_suffix
+        self.weight: Optional[torch.Tensor] = None     # float32 [dim]
+        self.bias: Optional[torch.Tensor] = None       # float32 [dim]
+
+    def param_specs(self, prefix: str) -> Dict[str, ParamSpec]:
+        return {prefix + self.name: ParamSpec((self.dim,), INIT_NORM_WEIGHT), prefix + self.name + self.bias_suffix: ParamSpec((self.dim,))}
+
+    def load(self, prefix: str, source: TensorSource) -> None:
+        self.weight = source.get(prefix + self.name).float().contiguous()
+        self.bias = source.get(prefix + self.name + self.bias_suffix).float().contiguous()
+
+    @staticmethod
+    def foldable(delta):
+        """`delta` as the layer norm kernel reads it (a tensor, or experts' outputs still to be summed)."""
+        return delta if delta is None or isinstance(delta, (torch.Tensor, ops.ExpertSum)) else delta.tensor()
+
+    def add_normed(self, stream: ResidualStream, delta, out_dtype: Optional[torch.dtype]) -> None:
+        """h += this norm of delta, in float, and ``stream.act`` = the new h in ``out_dtype`` (h itself in float32)."""
+        copy = out_dtype is not None and out_dtype != torch.float32
+        with section("norm", nbytes=stream.h.shape[0] * self.dim * 12):
+            out = ops.layer_norm(stream.h, self.foldable(delta), self.weight, self.bias, self.eps, out_dtype=out_dtype if copy else None)
+        stream.act = out if copy else stream.h
+
+    def forward(self, stream: ResidualStream, out_dtype: torch.dtype, rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """This norm of the stream; a branch output that waits behind a layer norm is added in the same launch.  With
+        ``rows`` only those rows are produced and the stream is left as it is."""
+        post, delta = stream.pending_norm, stream.pending
+        if post is not None and not isinstance(post, LayerNorm):
+            stream.settle()
+            post = delta = None
+        if post is None and delta is not None:
+            ops.stream_add(stream.h, delta if isinstance(delta, (torch.Tensor, ops.BranchSum)) else delta.tensor())
+            stream.pending = delta = None
+        n = stream.h.shape[0] if rows is None else rows.shape[0]
+        with section("norm", nbytes=n * self.dim * 12):
+            out = ops.layer_norm(stream.h, self.foldable(delta), post.weight if post else None, post.bias if post else None,
+                                 post.eps if post else self.eps, rows=rows, out_dtype=out_dtype, norm=(self.weight, self.bias, self.eps))
+        if rows is None:
+            stream.pending = stream.pending_norm = None
+        return out
+
+
 class RMSNorm(Part):
     """x * rsqrt(mean(x^2) + eps) * w, statistics in float
     (reference: src/SharpInference.Cpu/SimdKernels.cs:4209-4246; CUDA twin
