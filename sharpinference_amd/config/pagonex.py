@@ -39,22 +39,22 @@ class DeltaMixerConfig:
     dim: int
     vdim: int
     conv: int                   # taps of the convolutions behind q, k and v
-    decay_rank: int = DEFAULT_RANK
-    gate_rank: int = DEFAULT_RANK
+    decay_rank: Optional[int] = None
+    gate_rank: Optional[int] = None
 
     @classmethod
     def from_dict(cls, d: Dict[str, Any], where: str) -> "DeltaMixerConfig":
         _only(d, ("heads", "kv_heads", "dim", "vdim", "conv", "decay_rank", "gate_rank"), where)
         heads, dim = _num(d, "heads", where), _num(d, "dim", where)
         return cls(heads=heads, kv_heads=_num(d, "kv_heads", where, int, heads), dim=dim, vdim=_num(d, "vdim", where, int, dim),
-                   conv=_num(d, "conv", where), decay_rank=_num(d, "decay_rank", where, int, DEFAULT_RANK),
-                   gate_rank=_num(d, "gate_rank", where, int, DEFAULT_RANK))
+                   conv=_num(d, "conv", where), decay_rank=None if d.get("decay_rank") is None else _num(d, "decay_rank", where),
+                   gate_rank=None if d.get("gate_rank") is None else _num(d, "gate_rank", where))
 
     def to_dict(self) -> Dict[str, Any]:
         out: Dict[str, Any] = {"heads": self.heads, "kv_heads": self.kv_heads, "dim": self.dim, "vdim": self.vdim, "conv": self.conv}
-        if self.decay_rank != DEFAULT_RANK:
+        if self.decay_rank is not None:
             out["decay_rank"] = self.decay_rank
-        if self.gate_rank != DEFAULT_RANK:
+        if self.gate_rank is not None:
             out["gate_rank"] = self.gate_rank
         return out
 
@@ -234,7 +234,7 @@ class PagonexConfig(ModelConfig):
         for i, layer in enumerate(self.layers):
             where, m = f"layers[{i}].mixer", layer.mixer
             if layer.type == "channel_delta":
-                if min(m.heads, m.kv_heads, m.dim, m.vdim, m.conv, m.decay_rank, m.gate_rank) < 1 or m.heads % m.kv_heads:
+                if min(m.heads, m.kv_heads, m.dim, m.vdim, m.conv) < 1 or min(m.decay_rank or 1, m.gate_rank or 1) < 1 or m.heads % m.kv_heads:
                     raise ConfigError(f"{where}: heads, kv_heads, dim, vdim and conv must be positive and kv_heads divide heads")
             else:
                 if min(m.heads, m.dim, m.rot_dim, m.vdim, m.q_rank, m.kv_rank) < 1:

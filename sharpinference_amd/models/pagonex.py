@@ -24,7 +24,7 @@ from __future__ import annotations
 from typing import Dict, Tuple
 
 from ..cache.spec import WINDOW_NONE, WINDOW_SLIDING
-from ..config.pagonex import PagonexConfig
+from ..config.pagonex import DEFAULT_RANK, PagonexConfig
 from ..parts.block import ConvPostNormBlock
 from ..parts.conv import ResidualConv
 from ..parts.delta_rule import GatedDeltaRule
@@ -60,7 +60,8 @@ def build_pagonex(cfg: PagonexConfig) -> DecoderModel:
         m, f = layer.mixer, layer.mlp
         run = Run(i, i)
         if layer.type == "channel_delta":
-            mixer = GatedDeltaRule(W, m.heads, m.kv_heads, m.dim, m.vdim, m.conv, m.decay_rank, m.gate_rank, eps)
+            mixer = GatedDeltaRule(W, m.heads, m.kv_heads, m.dim, m.vdim, m.conv, m.decay_rank or DEFAULT_RANK,
+                                   m.gate_rank or DEFAULT_RANK, eps)
         else:
             rotary = None
             if m.rot is not None and m.rot.scaling is not None:
