@@ -18,7 +18,9 @@ attention beside it, dense feed-forwards) beside Llama 4 layers with dense feed-
 ``--shape nosedra`` runs Nosedra layers (attention with a learned sink beside a matrix memory with exponential
 gates, state-space layers) beside Pazatar layers of the same sizes;
 ``--shape fovosun`` runs Fovosun layers (differential attention, retention, clamped routed experts, four
-residual streams) beside Llama 4 layers of the same width, heads and experts.
+residual streams) beside Llama 4 layers of the same width, heads and experts;
+``--shape pagonex`` runs Pagonex layers (the gated delta rule, latent attention behind a window, routed experts)
+beside Kuvonex layers of the same width, heads and experts and Pazatar layers with the same recurrent heads.
 """
 from __future__ import annotations
 
@@ -713,6 +715,58 @@ def run_fovosun(args) -> int:
     return 0
 
 
+# ---------------------------------------------------------------------------
+# Pagonex beside Kuvonex and Pazatar at equal sizes
+# ---------------------------------------------------------------------------
+# width, layers (delta rule, latent attention, latent attention over its neighbour's rows, delta rule), heads (of the
+# latent layers: 128 + 64 wide over a latent of 512, queries through a latent of a quarter or half of the width), delta heads of
+# 128 key and 128 value channels over half as many key heads, routed experts, picks, expert width (and a shared expert of
+# that width with a limit of its own), vocabulary.  Kuvonex has the latent layers' like, Pazatar (one parallel layer in
+# two, dense feed-forwards as wide as the picks together) the recurrence's
+PAGONEX_SIZES = {
+    "w2048": dict(width=2048, layers=4, heads=16, q_rank=768, delta_heads=16, experts=64, top=6, ff=1408, groups=(8, 4), vocab=32000,
+                  window=1024, rank=128, kv_heads=4, chunk=1024, decay_rank=128),
+    "w4096": dict(width=4096, layers=4, heads=64, q_rank=1536, delta_heads=32, experts=32, top=4, ff=2048, groups=(4, 2), vocab=32000,
+                  window=1024, rank=128, kv_heads=8, chunk=1024, decay_rank=128),
+}
+PAGONEX_KINDS = ["channel_delta", "latent_attention", "latent_attention", "channel_delta"]
+
+
+def pagonex_config(z: dict) -> dict:
+    delta = {"heads": z["delta_heads"], "kv_heads": z["delta_heads"] // 2, "dim": 128, "vdim": 128, "conv": 4, "decay_rank": z["rank"],
+             "gate_rank": z["rank"]}
+    latent = {"heads": z["heads"], "dim": 128, "rot_dim": 64, "vdim": 128, "q_rank": z["q_rank"], "kv_rank": 512, "scale": 192 ** -0.5,
+              "mask": {"size": z["window"]},
+              "rot": {"base": 10000.0, "dims": 64, "scaling": {"factor": 8.0, "original": 1024, "fast": 32.0, "slow": 1.0}}}
+    mlp = {"kind": "moe", "expert": {"ff": z["ff"], "limit": 7.0}, "router": {"experts": z["experts"], "top": z["top"], "scale": 2.5},
+           "shared": {"ff": z["ff"], "limit": 3.0}}
+    layers = [{"type": kind, "mixer": dict(delta if kind == "channel_delta" else latent), "mlp": mlp} for kind in PAGONEX_KINDS[:z["layers"]]]
+    layers[2]["mixer"]["kv_from"] = 1
+    return {"architecture": "Pagonex", "vocab": z["vocab"], "width": z["width"], "norm": {"eps": 1e-5}, "canon": {"taps": 4},
+            "embedding": {"bigram": {"buckets": 100003, "mul_prev": 31, "mul_cur": 7}}, "logit_scale": 1.0, "layers": layers}
+
+
+def pazatar_like_pagonex(z: dict) -> dict:
+    return pazatar_config(dict(z, heads=z["delta_heads"], ff=z["ff"] * z["top"]))
+
+
+def run_pagonex(args) -> int:
+    """Prefill of one 2,048-token prompt and decode at batch 8 and 64 for the Pagonex design at two sizes (random
+    weights), each beside Kuvonex layers of the same width, heads, experts and expert width and Pazatar layers with the
+    same recurrent heads, with the per-kernel-class tables of one prefill and one decode step of all."""
+    pairs = (("pagonex", pagonex_config), ("kuvonex", kuvonex_config), ("pazatar", pazatar_like_pagonex))
+    rows, P, steps, warm = _beside(args, PAGONEX_SIZES, pairs[:1] if args.alone else pairs)
+    k0 = rows[0]
+    out = {"metric": "decode tok/s at batch 8 (Pagonex, width 2048, 4 layers, 2,048-token prompts)", "value": k0["decode_b8_tok_s"],
+           "unit": "tok/s", "n_gpus": 1, "steps": steps, "warmup": warm, "ms_per_step": k0["decode_b8_ms_per_step"],
+           "higher_is_better": True, "scaling": "weak", "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
+           "config": {"model": "pagonex-random beside kuvonex-random and pazatar-random at equal sizes", "global_batch": 8,
+                      "seq_len": CONTEXT, "parallelism": "single-gpu", "prompt_len": P, "sizes": PAGONEX_SIZES},
+           "rows": rows}
+    print(json.dumps(out), flush=True)
+    return 0
+
+
 def main() -> int:
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -726,10 +780,12 @@ def main() -> int:
     ap.add_argument("--no-graphs", action="store_true", help="launch decode steps kernel by kernel instead of replaying a HIP graph")
     ap.add_argument("--no-peaks", action="store_true", help="skip the two measuring kernels (pure read, matrix-core loop)")
     ap.add_argument("--profile", action="store_true", help="also print ms / bytes / GB/s per kernel class of one prefill and one decode step")
-    ap.add_argument("--shape", default="scout", choices=["scout", "maverick8", "long16", "kuvonex", "pazatar", "nosedra", "fovosun"],
+    ap.add_argument("--shape", default="scout", choices=["scout", "maverick8", "long16", "kuvonex", "pazatar", "nosedra", "fovosun", "pagonex"],
                     help="scout: the headline run; maverick8 / long16: two other workloads; kuvonex / pazatar: that design beside "
                          "Llama 4 layers of equal size; nosedra: that design beside Pazatar layers of equal size; fovosun: that design beside "
-                         "Llama 4 layers of equal size; each prints a JSON line of its own")
+                         "Llama 4 layers of equal size; pagonex: that design beside Kuvonex and Pazatar layers of equal size; each prints a JSON "
+                         "line of its own")
+    ap.add_argument("--alone", action="store_true", help="--shape pagonex without the models it is measured beside")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py measures one GPU: this engine has no multi-GPU path (N=1 only)")
@@ -746,6 +802,8 @@ def main() -> int:
         return run_nosedra(args)
     if args.shape == "fovosun":
         return run_fovosun(args)
+    if args.shape == "pagonex":
+        return run_pagonex(args)
 
     import torch  # noqa: F401
 

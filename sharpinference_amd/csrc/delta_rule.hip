@@ -59,50 +59,86 @@ struct LowRankJob {
 };
 struct LowRankJobs { LowRankJob j[2]; };
 
-template <typename T>
-__device__ __forceinline__ void load4(const T* p, int n, float* v) {       // n of four elements, the rest zero
+// n of four elements as floats, the rest zero (VEC: all four there, 8 or 16 bytes at once)
+template <typename T, bool VEC>
+__device__ __forceinline__ void load4(const T* p, int n, float* v) {
+  if constexpr (VEC && sizeof(T) == 4) {
+    const float4 x = *reinterpret_cast<const float4*>(p);
+    v[0] = x.x; v[1] = x.y; v[2] = x.z; v[3] = x.w;
+  } else if constexpr (VEC) {
+    const uint2 x = *reinterpret_cast<const uint2*>(p);
+    v[0] = bf16_bits_to_f32(x.x & 0xffffu); v[1] = bf16_bits_to_f32(x.x >> 16);
+    v[2] = bf16_bits_to_f32(x.y & 0xffffu); v[3] = bf16_bits_to_f32(x.y >> 16);
+  } else {
 #pragma unroll
-  for (int i = 0; i < 4; ++i) v[i] = i < n ? to_f32<T>(p[i]) : 0.f;
+    for (int i = 0; i < 4; ++i) v[i] = i < n ? to_f32<T>(p[i]) : 0.f;
+  }
 }
 
-template <typename T>
+template <typename T, bool VEC, int TT>      // VEC: ranks multiples of 16, rows and columns of x and w on 16-byte borders
 __global__ __launch_bounds__(256) void lowrank_kernel(const float* __restrict__ x, int stride, LowRankJobs jobs, int n_tokens) {
   const LowRankJob& jb = (int)blockIdx.y < jobs.j[0].blocks ? jobs.j[0] : jobs.j[1];
   const int nb = (int)blockIdx.y < jobs.j[0].blocks ? blockIdx.y : blockIdx.y - jobs.j[0].blocks;
   const int lane = threadIdx.x & 63, m = lane & 15, g = lane >> 4;
   const int n0 = (nb * 4 + (threadIdx.x >> 6)) * 16;
-  if (n0 >= jb.N) return;
-  const T* wr = (const T*)jb.w + (size_t)min(n0 + m, jb.N - 1) * jb.rank;
-  const float* xr[kLrTiles];
+  const int rank = jb.rank, N = jb.N;
+  if (n0 >= N) return;
+  const T* wr = (const T*)jb.w + (size_t)min(n0 + m, N - 1) * rank;
+  const float* xr[TT];
 #pragma unroll
-  for (int a = 0; a < kLrTiles; ++a)
-    xr[a] = x + (size_t)min((int)(blockIdx.x * kLrTiles + a) * 16 + m, n_tokens - 1) * stride + jb.x_off;
-  f32x4 acc[kLrTiles];
+  for (int a = 0; a < TT; ++a)
+    xr[a] = x + (size_t)min((int)(blockIdx.x * TT + a) * 16 + m, n_tokens - 1) * stride + jb.x_off;
+  f32x4 acc[TT];
 #pragma unroll
-  for (int a = 0; a < kLrTiles; ++a) acc[a] = f32x4{0.f, 0.f, 0.f, 0.f};
-  for (int k0 = 0; k0 < jb.rank; k0 += 16) {
-    const int k = k0 + 4 * g, left = jb.rank - k;
-    float wv[4], xv[kLrTiles][4];
-    load4<T>(wr + k, left, wv);
+  for (int a = 0; a < TT; ++a) acc[a] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 2
+  for (int k0 = 0; k0 < rank; k0 += 16) {
+    const int k = k0 + 4 * g, left = rank - k;
+    float wv[4], xv[TT][4];
+    load4<T, VEC>(wr + k, left, wv);
 #pragma unroll
-    for (int a = 0; a < kLrTiles; ++a) load4<float>(xr[a] + k, left, xv[a]);
+    for (int a = 0; a < TT; ++a) load4<float, VEC>(xr[a] + k, left, xv[a]);
 #pragma unroll
     for (int i = 0; i < 4; ++i)
 #pragma unroll
-      for (int a = 0; a < kLrTiles; ++a) acc[a] = mfma4(wv[i], xv[a][i], acc[a]);
+      for (int a = 0; a < TT; ++a) acc[a] = mfma4(wv[i], xv[a][i], acc[a]);
   }
-#pragma unroll
-  for (int a = 0; a < kLrTiles; ++a) {
-    const int t = (blockIdx.x * kLrTiles + a) * 16 + m;
-    if (t >= n_tokens) continue;
+  const bool decay = jb.mode == LOWRANK_LOG_DECAY;
+  float neg_a[4], bias[4];
+  if (decay) {
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      const int n = n0 + 4 * g + i;
-      if (n >= jb.N) continue;
-      if (jb.mode == LOWRANK_LOG_DECAY)
-        ((float*)jb.out)[(size_t)t * jb.N + n] = -expf(jb.a_log[n / jb.per]) * softplus_f32(acc[a][i] + jb.bias[n]);
-      else
-        ((T*)jb.out)[(size_t)t * jb.N + n] = from_f32<T>(acc[a][i]);
+      const int n = min(n0 + 4 * g + i, N - 1);
+      neg_a[i] = -expf(jb.a_log[n / jb.per]);
+      bias[i] = jb.bias[n];
+    }
+  }
+#pragma unroll
+  for (int a = 0; a < TT; ++a) {
+    const int t = (blockIdx.x * TT + a) * 16 + m;
+    if (t >= n_tokens) continue;
+    if (decay) {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) acc[a][i] = neg_a[i] * softplus_f32(acc[a][i] + bias[i]);
+    }
+    const size_t at = (size_t)t * N + n0 + 4 * g;
+    if (VEC && N % 4 == 0) {
+      if (n0 + 4 * g >= N) continue;
+      if (decay || sizeof(T) == 4) {
+        *reinterpret_cast<f32x4*>((float*)jb.out + at) = acc[a];
+      } else {
+        uint2 o;
+        o.x = (uint32_t)f32_to_bf16(acc[a][0]).bits | ((uint32_t)f32_to_bf16(acc[a][1]).bits << 16);
+        o.y = (uint32_t)f32_to_bf16(acc[a][2]).bits | ((uint32_t)f32_to_bf16(acc[a][3]).bits << 16);
+        *reinterpret_cast<uint2*>((T*)jb.out + at) = o;
+      }
+      continue;
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      if (n0 + 4 * g + i >= N) continue;
+      if (decay) ((float*)jb.out)[at + i] = acc[a][i];
+      else ((T*)jb.out)[at + i] = from_f32<T>(acc[a][i]);
     }
   }
 }
@@ -119,11 +155,27 @@ SHARPI_EXPORT int sharpi_lowrank(const float* x, int stride, int dtype, int n_to
   LowRankJobs jobs;
   jobs.j[0] = LowRankJob{x_off0, rank0, N0, LOWRANK_LOG_DECAY, per > 0 ? per : 1, w0, bias, a_log, out0, ceil_div(N0, 64)};
   jobs.j[1] = LowRankJob{x_off1, rank1, N1, LOWRANK_PLAIN, 1, w1, nullptr, nullptr, out1, ceil_div(N1, 64)};
-  dim3 grid(ceil_div(n_tokens, 16 * kLrTiles), jobs.j[0].blocks + jobs.j[1].blocks);
+  const int tt = n_tokens > 16 ? kLrTiles : 1;
+  dim3 grid(ceil_div(n_tokens, 16 * tt), jobs.j[0].blocks + jobs.j[1].blocks);
   if (grid.y > 65535) return SHARPI_ERR_ARG;
-  if (dtype == DT_F32) lowrank_kernel<float><<<grid, 256, 0, stream>>>(x, stride, jobs, n_tokens);
-  else if (dtype == DT_BF16) lowrank_kernel<bf16_t><<<grid, 256, 0, stream>>>(x, stride, jobs, n_tokens);
-  else return SHARPI_ERR_ARG;
+  auto on16 = [](const void* p) { return ((uintptr_t)p & 15) == 0; };
+  const bool vec = stride % 4 == 0 && on16(x) && (N0 == 0 || (rank0 % 16 == 0 && x_off0 % 4 == 0 && on16(w0) && on16(out0))) &&
+                   (N1 == 0 || (rank1 % 16 == 0 && x_off1 % 4 == 0 && on16(w1) && on16(out1)));
+#define LR(T, V)                                                                                   \
+  do {                                                                                             \
+    if (tt == 1) lowrank_kernel<T, V, 1><<<grid, 256, 0, stream>>>(x, stride, jobs, n_tokens);     \
+    else lowrank_kernel<T, V, kLrTiles><<<grid, 256, 0, stream>>>(x, stride, jobs, n_tokens);      \
+  } while (0)
+  if (dtype == DT_F32) {
+    if (vec) LR(float, true);
+    else LR(float, false);
+  } else if (dtype == DT_BF16) {
+    if (vec) LR(bf16_t, true);
+    else LR(bf16_t, false);
+  } else {
+    return SHARPI_ERR_ARG;
+  }
+#undef LR
   SHARPI_CHECK_LAUNCH();
   return SHARPI_OK;
 }
@@ -158,7 +210,7 @@ __device__ __forceinline__ float conv_one(const DeltaIn& a, const T* row, const 
 }
 
 template <typename T, int NT>       // NT: 16-row tiles a lane holds of a strip (rows beyond dk stay zero)
-__global__ __launch_bounds__(512) void delta_step_kernel(DeltaIn a, const float* __restrict__ norm_w, float eps,
+__global__ __launch_bounds__(512, NT <= 8 ? 4 : 2) void delta_step_kernel(DeltaIn a, const float* __restrict__ norm_w, float eps,
                                                          const T* __restrict__ gate, T* __restrict__ out) {
   __shared__ __attribute__((aligned(16))) float q_s[NT * 16], k_s[NT * 16], d_s[NT * 16];
   __shared__ float red[3][8];
@@ -238,6 +290,7 @@ __global__ __launch_bounds__(512) void delta_step_kernel(DeltaIn a, const float*
         dotk = fmaf(S[n][i], k4[i], dotk);
         dotq = fmaf(S[n][i], q4[i], dotq);
       }
+      if (n % 2) __builtin_amdgcn_sched_barrier(0);      // (all tiles' operands read ahead would not fit the registers)
     }
     dotk += __shfl_xor(dotk, 16, kWave);
     dotq += __shfl_xor(dotq, 16, kWave);
@@ -283,8 +336,10 @@ struct ChunkBuf {
   float *W, *Qd, *KT, *D, *U0, *A;
 };
 
-template <typename T>
-__global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaIn a, const int* __restrict__ chunks, ChunkBuf b, int ldk) {
+// (TAPS: the convolution's taps, or more: the weights beyond are zero; DKP: room for dk key channels)
+template <typename T, int TAPS, int DKP>
+__global__ __launch_bounds__(256, DKP <= 128 ? 4 : 2) void delta_chunk_prep_kernel(DeltaIn a, const int* __restrict__ chunks, ChunkBuf b) {
+  constexpr int ldk = DKP + 4;             // rows of LDS four banks apart
   extern __shared__ __attribute__((aligned(16))) float smem[];
   constexpr int C = kDcTokens;
   float* q_s = smem;                       // [C][ldk]
@@ -324,11 +379,11 @@ __global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaIn a, const 
       for (int t = 0; t < C; ++t) dst[t * ld] = 0.f;
       continue;
     }
-    float u[C], wt[kDrMaxTaps], past[kDrMaxTaps];
+    float u[C], wt[TAPS], past[TAPS];
 #pragma unroll
-    for (int t = 0; t < C; ++t) u[t] = t < n ? to_f32<T>(rows[(size_t)t * a.stride + chan]) : 0.f;
+    for (int t = 0; t < C; ++t) u[t] = to_f32<T>(rows[(size_t)min(t, n - 1) * a.stride + chan]);   // (no load behind a branch)
 #pragma unroll
-    for (int back = 0; back < kDrMaxTaps; ++back) {
+    for (int back = 0; back < TAPS; ++back) {
       wt[back] = back < a.taps ? a.conv_w[(size_t)chan * a.taps + a.taps - 1 - back] : 0.f;
       past[back] = 0.f;                    // the input `back` tokens before the chunk's first
       if (back > 0 && back < a.taps) {
@@ -340,15 +395,18 @@ __global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaIn a, const 
     for (int t = 0; t < C; ++t) {
       float acc = 0.f;
 #pragma unroll
-      for (int back = kDrMaxTaps - 1; back >= 0; --back) acc = fmaf(wt[back], t >= back ? u[t - back < 0 ? 0 : t - back] : past[back - t < 0 ? 0 : back - t], acc);
+      for (int back = TAPS - 1; back >= 0; --back) acc = fmaf(wt[back], t >= back ? u[t - back < 0 ? 0 : t - back] : past[back - t < 0 ? 0 : back - t], acc);
       dst[t * ld] = t < n ? acc * sigmoid_f32(acc) : 0.f;
     }
   }
   for (int c = tid; c < ldk; c += blockDim.x) {
-    float run = 0.f;
+    float l[C], run = 0.f;
+    const float* src = a.log_decay + (size_t)first * a.nh * a.dk + h * a.dk + min(c, a.dk - 1);
+#pragma unroll
+    for (int t = 0; t < C; ++t) l[t] = src[(size_t)min(t, n - 1) * a.nh * a.dk];
 #pragma unroll
     for (int t = 0; t < C; ++t) {
-      if (c < a.dk && t < n) run += a.log_decay[(size_t)(first + t) * a.nh * a.dk + h * a.dk + c] * kLog2e;
+      if (c < a.dk && t < n) run += l[t] * kLog2e;
       b_s[t * ldk + c] = run;
     }
   }
@@ -393,35 +451,50 @@ __global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaIn a, const 
   for (int idx = tid; idx < dkp + dvp; idx += blockDim.x) {
     const bool key = idx < dkp;
     const int c = key ? idx : idx - dkp;
+    const float* k_c = k_s + c;
+    const float* b_c = b_s + c;
     float x[C];
+    float* w_out = b.W + ch * C * dkp + c;
+    float* q_out = b.Qd + ch * C * dkp + c;
 #pragma unroll
     for (int t = 0; t < C; ++t) {
       float r;
-      if (key) r = k_s[t * ldk + c] * exp2_f32(b_s[t * ldk + c]);
-      else r = c < a.dv ? v_s[t * a.dv + c] : 0.f;
+      if (key) {
+        const float decayed = exp2_f32(b_c[t * ldk]);
+        r = k_c[t * ldk] * decayed;
+        *q_out = q_s[t * ldk + c] * decayed;
+        q_out += dkp;
+      } else {
+        r = c < a.dv ? v_s[t * a.dv + c] : 0.f;
+      }
+      f32x4 L[C / 4];                      // row t (its elements from the diagonal on are zero)
+#pragma unroll
+      for (int s = 0; s < t; s += 4) L[s / 4] = *reinterpret_cast<const f32x4*>(L_s + t * C + s);
 #pragma unroll
       for (int s = 0; s < C; ++s)
-        if (s < t) r = fmaf(-L_s[t * C + s], x[s], r);
+        if (s < t) r = fmaf(-L[s / 4][s % 4], x[s], r);
       x[t] = beta_s[t] * r;
+      if (key) {
+        *w_out = x[t];
+        w_out += dkp;
+      }
+      if (t % 2) __builtin_amdgcn_sched_barrier(0);      // (all rows read ahead would not fit the registers)
     }
     if (key) {
-      const float total = b_s[(C - 1) * ldk + c];
-#pragma unroll
-      for (int t = 0; t < C; ++t) {
-        b.W[(ch * C + t) * dkp + c] = x[t];
-        b.Qd[(ch * C + t) * dkp + c] = q_s[t * ldk + c] * exp2_f32(b_s[t * ldk + c]);
-      }
+      const float total = b_c[(C - 1) * ldk];
+      float* kt = b.KT + (ch * dkp + c) * C;
 #pragma unroll
       for (int t = 0; t < C; t += 4) {
         f32x4 v;
 #pragma unroll
-        for (int i = 0; i < 4; ++i) v[i] = k_s[(t + i) * ldk + c] * exp2_f32(total - b_s[(t + i) * ldk + c]);
-        *reinterpret_cast<f32x4*>(b.KT + (ch * dkp + c) * C + t) = v;
+        for (int i = 0; i < 4; ++i) v[i] = k_c[(t + i) * ldk] * exp2_f32(total - b_c[(t + i) * ldk]);
+        *reinterpret_cast<f32x4*>(kt + t) = v;
       }
       b.D[ch * dkp + c] = exp2_f32(total);
     } else {
+      float* u0 = b.U0 + (ch * dvp + c) * C;
 #pragma unroll
-      for (int t = 0; t < C; t += 4) *reinterpret_cast<f32x4*>(b.U0 + (ch * dvp + c) * C + t) = f32x4{x[t], x[t + 1], x[t + 2], x[t + 3]};
+      for (int t = 0; t < C; t += 4) *reinterpret_cast<f32x4*>(u0 + t) = f32x4{x[t], x[t + 1], x[t + 2], x[t + 3]};
     }
   }
 }
@@ -430,93 +503,122 @@ __global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaIn a, const 
 // takes group L % 8 + 8 (L / (8 ns)) and strip (L / 8) % ns.
 constexpr int kDies = 8;
 
-template <typename T, int TPW>      // TPW: 16-row tiles a wave
-__global__ __launch_bounds__(512) void delta_chunk_walk_kernel(DeltaIn a, const int* __restrict__ chunks, const int* __restrict__ ent_chunks,
-                                                               ChunkBuf b, float* __restrict__ out, int n_groups) {
-  constexpr int C = kDcTokens, kBuf = 3;
-  __shared__ __attribute__((aligned(16))) f32x4 p_s[2][8][kWave], o_s[2][8][kWave];
+// Four waves hold the state (TPW 16-row tiles each), a fifth makes the outputs.  Per chunk: P = W S (a partial sum a wave, added
+// through LDS by everyone behind the chunk's one barrier), O = Qd S while those sums are on their way, U = U0 - P, S = D S + KT U.
+// The partial sums of O are read by the fifth wave behind the NEXT chunk's barrier, with the U it has kept.
+constexpr int kDwWaves = 4;
+
+template <typename T, int TPW>
+__global__ __launch_bounds__(kWave * (kDwWaves + 1)) void delta_chunk_walk_kernel(
+    DeltaIn a, const int* __restrict__ chunks, const int* __restrict__ ent_chunks, ChunkBuf b, float* __restrict__ out, int n_groups) {
+  constexpr int C = kDcTokens, NW = kDwWaves;
+  __shared__ __attribute__((aligned(16))) f32x4 p_s[2][NW][kWave], o_s[2][NW][kWave];
   const int ns = (a.dv + 15) >> 4, nt = (a.dk + 15) >> 4, dkp = nt * 16, dvp = ns * 16;
   const int group = blockIdx.x % kDies + kDies * (blockIdx.x / (kDies * ns)), strip = (blockIdx.x / kDies) % ns;
   if (group >= n_groups) return;
   const int e = group / a.nh, h = group % a.nh;
-  const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, nw = blockDim.x >> 6, g = lane >> 4, m = lane & 15;
+  const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, g = lane >> 4, m = lane & 15;
   const int c_first = ent_chunks[2 * e], c_n = ent_chunks[2 * e + 1];
   const int slot = a.state_slots[e];
-  float* st = a.state + (((size_t)slot * a.nh + h) * ns + strip) * nt * 256;
-  f32x4 S[TPW];
-  bool has[TPW];
-#pragma unroll
-  for (int n = 0; n < TPW; ++n) {
-    has[n] = w + n * nw < nt;
-    S[n] = has[n] ? *reinterpret_cast<const f32x4*>(st + (size_t)(w + n * nw) * 256 + lane * 4) : f32x4{0.f, 0.f, 0.f, 0.f};
-  }
-  struct Ops {
-    f32x4 W[TPW], Q[TPW], K[TPW], D[TPW], U, A;
-  } buf[kBuf];
-  auto fetch = [&](int c, Ops& o) {
-    const size_t ch = (size_t)(c_first + c) * a.nh + h;
+  const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+  if (w < NW) {
+    float* st = a.state + (((size_t)slot * a.nh + h) * ns + strip) * nt * 256;
+    f32x4 S[TPW];
+    bool has[TPW];
+    int tile[TPW];
 #pragma unroll
     for (int n = 0; n < TPW; ++n) {
-      const int tile = min(w + n * nw, nt - 1);      // (a tile beyond the last: read, not used)
-      o.W[n] = *reinterpret_cast<const f32x4*>(b.W + (ch * C + m) * dkp + 16 * tile + 4 * g);
-      o.Q[n] = *reinterpret_cast<const f32x4*>(b.Qd + (ch * C + m) * dkp + 16 * tile + 4 * g);
-      o.K[n] = *reinterpret_cast<const f32x4*>(b.KT + (ch * dkp + 16 * tile + m) * C + 4 * g);
-      o.D[n] = *reinterpret_cast<const f32x4*>(b.D + ch * dkp + 16 * tile + 4 * g);
+      has[n] = w + n * NW < nt;
+      tile[n] = min(w + n * NW, nt - 1);       // (a tile beyond the last: its operands are read, its state stays zero)
+      S[n] = has[n] ? *reinterpret_cast<const f32x4*>(st + (size_t)tile[n] * 256 + lane * 4) : zero;
     }
-    o.U = *reinterpret_cast<const f32x4*>(b.U0 + (ch * dvp + strip * 16 + m) * C + 4 * g);
-    o.A = *reinterpret_cast<const f32x4*>(b.A + ch * 256 + m * 16 + 4 * g);
-  };
-  fetch(0, buf[0]);
-  if (c_n > 1) fetch(1, buf[1]);
-  for (int c0 = 0; c0 < c_n; c0 += kBuf) {
+    struct Ops {
+      f32x4 W[TPW], Q[TPW], K[TPW], D[TPW], U;
+    } buf[3];
+    auto fetch = [&](int c, Ops& o) {          // (chunks beyond the last: the last once more, no load behind a branch)
+      const size_t ch = (size_t)(c_first + min(c, c_n - 1)) * a.nh + h;
 #pragma unroll
-    for (int x = 0; x < kBuf; ++x) {
-      const int c = c0 + x;
-      if (c < c_n) {
-        const Ops& o = buf[x];
-        if (c + 2 < c_n) fetch(c + 2, buf[(x + 2) % kBuf]);
-        f32x4 P = {0.f, 0.f, 0.f, 0.f}, O = {0.f, 0.f, 0.f, 0.f};
+      for (int n = 0; n < TPW; ++n) {
+        o.W[n] = *reinterpret_cast<const f32x4*>(b.W + (ch * C + m) * dkp + 16 * tile[n] + 4 * g);
+        o.Q[n] = *reinterpret_cast<const f32x4*>(b.Qd + (ch * C + m) * dkp + 16 * tile[n] + 4 * g);
+        o.K[n] = *reinterpret_cast<const f32x4*>(b.KT + (ch * dkp + 16 * tile[n] + m) * C + 4 * g);
+        o.D[n] = *reinterpret_cast<const f32x4*>(b.D + ch * dkp + 16 * tile[n] + 4 * g);
+      }
+      o.U = *reinterpret_cast<const f32x4*>(b.U0 + (ch * dvp + strip * 16 + m) * C + 4 * g);
+    };
+    auto one = [&](int c, const Ops& o, Ops& ahead) {
+      fetch(c + 2, ahead);
+      f32x4 P = zero, O = zero;
 #pragma unroll
-        for (int n = 0; n < TPW; ++n)
-          if (has[n]) {
+      for (int n = 0; n < TPW; ++n)
 #pragma unroll
-            for (int i = 0; i < 4; ++i) {
-              P = mfma4(o.W[n][i], S[n][i], P);
-              O = mfma4(o.Q[n][i], S[n][i], O);
-            }
-          }
-        p_s[c & 1][w][lane] = P;
-        o_s[c & 1][w][lane] = O;
+        for (int i = 0; i < 4; ++i) P = mfma4(o.W[n][i], S[n][i], P);
+      p_s[c & 1][w][lane] = P;
+      __syncthreads();
+      f32x4 part[NW];
 #pragma unroll
-        for (int n = 0; n < TPW; ++n) S[n] *= o.D[n];
-        __syncthreads();
-        f32x4 U = o.U;
-        for (int i = 0; i < nw; ++i) U -= p_s[c & 1][i][lane];
+      for (int i = 0; i < NW; ++i) part[i] = p_s[c & 1][i][lane];
 #pragma unroll
-        for (int n = 0; n < TPW; ++n)
-          if (has[n]) {
+      for (int n = 0; n < TPW; ++n)
 #pragma unroll
-            for (int i = 0; i < 4; ++i) S[n] = mfma4(o.K[n][i], U[i], S[n]);
-          }
-        if (w == c % nw) {                 // the waves take turns with the outputs
-          f32x4 y = {0.f, 0.f, 0.f, 0.f};
-          for (int i = 0; i < nw; ++i) y += o_s[c & 1][i][lane];
+        for (int i = 0; i < 4; ++i) O = mfma4(o.Q[n][i], S[n][i], O);
+      f32x4 U = o.U;
 #pragma unroll
-          for (int i = 0; i < 4; ++i) y = mfma4(o.A[i], U[i], y);
-          const int first = chunks[4 * (c_first + c) + 1], cnt = chunks[4 * (c_first + c) + 2];
-          const int col = strip * 16 + m;
-          if (col < a.dv) {
+      for (int i = 0; i < NW; ++i) U -= part[i];
 #pragma unroll
-            for (int i = 0; i < 4; ++i)
-              if (4 * g + i < cnt) out[(size_t)(first + 4 * g + i) * a.nh * a.dv + (size_t)h * a.dv + col] = y[i];
-          }
+      for (int n = 0; n < TPW; ++n) {
+        S[n] *= o.D[n];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) S[n] = mfma4(has[n] ? o.K[n][i] : 0.f, U[i], S[n]);
+      }
+      o_s[c & 1][w][lane] = O;
+    };
+    fetch(0, buf[0]);
+    fetch(1, buf[1]);
+    int c = 0;
+    for (; c + 3 <= c_n; c += 3) {
+      one(c, buf[0], buf[2]);
+      one(c + 1, buf[1], buf[0]);
+      one(c + 2, buf[2], buf[1]);
+    }
+    if (c < c_n) one(c, buf[0], buf[2]);
+    if (c + 1 < c_n) one(c + 1, buf[1], buf[0]);
+    __syncthreads();                           // (the last chunk's shares of the outputs are there)
+#pragma unroll
+    for (int n = 0; n < TPW; ++n)
+      if (has[n]) *reinterpret_cast<f32x4*>(st + (size_t)tile[n] * 256 + lane * 4) = S[n];
+  } else {
+    const int col = strip * 16 + m;
+    f32x4 U_before = zero, A_before = zero;
+    auto u_of = [&](int c) { return *reinterpret_cast<const f32x4*>(b.U0 + (((size_t)(c_first + c) * a.nh + h) * dvp + strip * 16 + m) * C + 4 * g); };
+    auto a_of = [&](int c) { return *reinterpret_cast<const f32x4*>(b.A + ((size_t)(c_first + c) * a.nh + h) * 256 + m * 16 + 4 * g); };
+    f32x4 U_next = u_of(0), A_next = a_of(0);
+    for (int c = 0; c <= c_n; ++c) {
+      f32x4 U = U_next, A = A_next;
+      U_next = u_of(min(c + 1, c_n - 1));
+      A_next = a_of(min(c + 1, c_n - 1));
+      __syncthreads();                         // chunk c's P, chunk c - 1's O (the last time: its O alone)
+      if (c > 0) {
+        f32x4 y = zero;
+#pragma unroll
+        for (int i = 0; i < NW; ++i) y += o_s[(c - 1) & 1][i][lane];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) y = mfma4(A_before[i], U_before[i], y);
+        const int first = chunks[4 * (c_first + c - 1) + 1], cnt = chunks[4 * (c_first + c - 1) + 2];
+        if (col < a.dv) {
+#pragma unroll
+          for (int i = 0; i < 4; ++i)
+            if (4 * g + i < cnt) out[(size_t)(first + 4 * g + i) * a.nh * a.dv + (size_t)h * a.dv + col] = y[i];
         }
+      }
+      if (c < c_n) {
+#pragma unroll
+        for (int i = 0; i < NW; ++i) U -= p_s[c & 1][i][lane];
+        U_before = U;
+        A_before = A;
       }
     }
   }
-#pragma unroll
-  for (int n = 0; n < TPW; ++n)
-    if (has[n]) *reinterpret_cast<f32x4*>(st + (size_t)(w + n * nw) * 256 + lane * 4) = S[n];
   // the convolution's last inputs (everybody who reads the ring has run: the kernel before this one)
   if (a.ring && strip == 0) {
     const int last = a.cu_tokens[e + 1] - 1, len = last + 1 - a.cu_tokens[e], p_last = a.positions[last];
@@ -606,35 +708,50 @@ SHARPI_EXPORT int sharpi_delta_chunks(const void* proj, int dtype, int stride, i
   b.D = b.KT + per * 16 * dkp;
   b.U0 = b.D + per * dkp;
   b.A = b.U0 + per * 16 * dvp;
-  const int ldk = dkp + 4;                 // rows of LDS four banks apart
+  const int dk_room = dk <= 32 ? 32 : dk <= 64 ? 64 : dk <= 128 ? 128 : 256, ldk = dk_room + 4;
   const size_t lds = (size_t)(3 * kDcTokens * ldk + kDcTokens * kDcTokens + kDcTokens + kDcTokens * dv) * sizeof(float);
   if (lds > 160 * 1024) return SHARPI_ERR_ARG;
-#define PREP(TV)                                                                                                    \
+#define PREP(TV, TAPS, ROOM)                                                                                        \
   do {                                                                                                              \
-    auto kern = delta_chunk_prep_kernel<TV>;                                                                        \
+    auto kern = delta_chunk_prep_kernel<TV, TAPS, ROOM>;                                                            \
     static size_t allowed = 48 * 1024;     /* dynamic LDS this instantiation may take (raised once per size) */     \
     if (lds > allowed) {                                                                                            \
       hipError_t e_ = hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds); \
       if (e_ != hipSuccess) return (int)e_;                                                                         \
       allowed = lds;                                                                                                \
     }                                                                                                               \
-    kern<<<dim3(n_chunks, nh), 256, lds, stream>>>(a, chunks, b, ldk);                                              \
+    kern<<<dim3(n_chunks, nh), 256, lds, stream>>>(a, chunks, b);                                                   \
   } while (0)
-  if (dtype == DT_F32) PREP(float);
-  else PREP(bf16_t);
+#define PREP_BY(TV, TAPS)                         \
+  do {                                            \
+    if (dk_room == 32) PREP(TV, TAPS, 32);        \
+    else if (dk_room == 64) PREP(TV, TAPS, 64);   \
+    else if (dk_room == 128) PREP(TV, TAPS, 128); \
+    else PREP(TV, TAPS, 256);                     \
+  } while (0)
+  if (dtype == DT_F32) {
+    if (taps <= 4) PREP_BY(float, 4);
+    else PREP_BY(float, kDrMaxTaps);
+  } else {
+    if (taps <= 4) PREP_BY(bf16_t, 4);
+    else PREP_BY(bf16_t, kDrMaxTaps);
+  }
+#undef PREP_BY
 #undef PREP
   SHARPI_CHECK_LAUNCH();
-  const int groups = n_entries * nh, nw = nt < 8 ? nt : 8;
+  const int groups = n_entries * nh;
   const long long blocks = (long long)ceil_div(groups, kDies) * kDies * ns;
   if (blocks > 0x7fffffff) return SHARPI_ERR_ARG;
-#define WALK(TV, TPW) delta_chunk_walk_kernel<TV, TPW><<<(unsigned)blocks, kWave * nw, 0, stream>>>(a, chunks, ent_chunks, b, out, groups)
-  if (dtype == DT_F32) {
-    if (nt <= 8) WALK(float, 1);
-    else WALK(float, 2);
-  } else {
-    if (nt <= 8) WALK(bf16_t, 1);
-    else WALK(bf16_t, 2);
-  }
+#define WALK(TV, TPW) delta_chunk_walk_kernel<TV, TPW><<<(unsigned)blocks, kWave * (kDwWaves + 1), 0, stream>>>(a, chunks, ent_chunks, b, out, groups)
+#define WALK_BY(TV)                  \
+  do {                               \
+    if (nt <= 4) WALK(TV, 1);        \
+    else if (nt <= 8) WALK(TV, 2);   \
+    else WALK(TV, 4);                \
+  } while (0)
+  if (dtype == DT_F32) WALK_BY(float);
+  else WALK_BY(bf16_t);
+#undef WALK_BY
 #undef WALK
   SHARPI_CHECK_LAUNCH();
   return SHARPI_OK;

@@ -350,6 +350,17 @@ __global__ __launch_bounds__(256) void embed_bigram_kernel(const int* __restrict
   const T* a = table + (size_t)ids[t] * hidden;
   const TP* b = pairs + (size_t)row_s * hidden;
   float* o = out + (size_t)t * hidden;
+  if (hidden % 8 == 0) {           // (the tables begin on 32-byte borders: whole tensors)
+    for (int i = threadIdx.x * 8; i < hidden; i += blockDim.x * 8) {
+      float x[8], y[8];
+      load8(a + i, x);
+      load8(b + i, y);
+#pragma unroll
+      for (int k = 0; k < 8; ++k) x[k] = fmaf(x[k], scale, y[k]);
+      store8(o + i, x);
+    }
+    return;
+  }
   for (int i = threadIdx.x; i < hidden; i += blockDim.x) o[i] = fmaf(to_f32<T>(a[i]), scale, to_f32<TP>(b[i]));
 }
 
@@ -359,6 +370,7 @@ SHARPI_EXPORT int sharpi_embed_bigram(const int* ids, const void* table, int t_d
                                       int hidden, hipStream_t stream) {
   if (n_tokens <= 0) return SHARPI_OK;
   if (hidden <= 0 || buckets <= 0 || !before || !pairs) return SHARPI_ERR_ARG;
+  if (((uintptr_t)table | (uintptr_t)pairs | (uintptr_t)out) & 31) return SHARPI_ERR_ARG;
 #define EB(T, TP)                                                                                                                  \
   embed_bigram_kernel<T, TP><<<n_tokens, 256, 0, stream>>>(ids, (const T*)table, scale, (const TP*)pairs, mul_prev, mul_cur, buckets, \
                                                            before, positions, state_slots, entry_of_token, cu_tokens, out, hidden)

@@ -118,6 +118,125 @@ __device__ void gate_and_pick(float* g, int n_experts, int k, int gate, int reno
     for (int j = 0; j < k; ++j) w[j] /= wsum;
 }
 
+// The same by one wave, for up to 64 picks: lanes gate and rank experts lane, lane + 64, ..., a pick is a wave-wide
+// maximum (the lowest index wins a tie), pick j's id and weight stay in lane j until they are written.  The
+// additions over picks are in the picks' order, as one thread makes them.
+__device__ __forceinline__ void wave_lds_sync() {
+  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+  __builtin_amdgcn_wave_barrier();
+  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+}
+
+// index of the largest v[i], i < n, that is not marked in the lanes' masks (bit i / 64 of lane i % 64); -1: none
+__device__ __forceinline__ int wave_argmax(const float* v, int n, int lane, uint32_t taken, float* best_v) {
+  int best = -1;
+  float bv = -INFINITY;
+  for (int i = lane, b = 0; i < n; i += kWave, ++b) {
+    const float x = v[i];
+    if (!(taken >> b & 1u) && (best < 0 || x > bv)) {
+      bv = x;
+      best = i;
+    }
+  }
+#pragma unroll
+  for (int off = 32; off > 0; off >>= 1) {
+    const int oi = __shfl_xor(best, off, kWave);
+    const float ov = __shfl_xor(bv, off, kWave);
+    if (oi >= 0 && (best < 0 || ov > bv || (ov == bv && oi < best))) {
+      bv = ov;
+      best = oi;
+    }
+  }
+  best = __shfl(best, 0, kWave);           // (one answer for all lanes, whatever the values were)
+  *best_v = __shfl(bv, 0, kWave);
+  return best;
+}
+
+__device__ void gate_and_pick_wave(float* g, int n_experts, int k, int gate, int renorm, int* ids, float* w, float* gate_out,
+                                   float* choice, const float* corr, int n_groups, int keep, float w_scale, int lane) {
+  if (gate == 0) {
+    for (int e = lane; e < n_experts; e += kWave) g[e] = 1.0f / (1.0f + expf(-g[e]));
+  } else if (gate == 1) {
+    float mx = -INFINITY, sum = 0.f;
+    for (int e = lane; e < n_experts; e += kWave) mx = fmaxf(mx, g[e]);
+    mx = wave_max(mx);
+    for (int e = lane; e < n_experts; e += kWave) {
+      g[e] = expf(g[e] - mx);
+      sum += g[e];
+    }
+    const float inv = 1.0f / wave_sum(sum);
+    for (int e = lane; e < n_experts; e += kWave) g[e] *= inv;
+  }
+  if (gate_out)
+    for (int e = lane; e < n_experts; e += kWave) gate_out[e] = g[e];
+  const float* by = g;
+  if (choice) {
+    for (int e = lane; e < n_experts; e += kWave) choice[e] = corr ? g[e] + corr[e] : g[e];
+    if (n_groups > 1 && keep < n_groups) {
+      const int per = n_experts / n_groups;
+      float* rank = choice + n_experts;
+      wave_lds_sync();
+      for (int q = lane; q < n_groups; q += kWave) {
+        float top[kGroupTop];
+        for (int i = 0; i < kGroupTop; ++i) top[i] = -INFINITY;
+        for (int e = q * per; e < (q + 1) * per; ++e) {
+          float v = choice[e];
+          for (int i = 0; i < kGroupTop; ++i)
+            if (v > top[i]) {
+              const float o = top[i];
+              top[i] = v;
+              v = o;
+            }
+        }
+        float r = 0.f;
+        for (int i = 0; i < kGroupTop && i < per; ++i) r += top[i];
+        rank[q] = r;
+      }
+      wave_lds_sync();
+      uint32_t kept = 0;                   // bit b: group lane + 64 b
+      for (int j = 0; j < keep; ++j) {
+        float bv;
+        const int best = wave_argmax(rank, n_groups, lane, kept, &bv);
+        if (best >= 0 && best % kWave == lane) kept |= 1u << (best / kWave);
+      }
+      for (int q = lane, b = 0; q < n_groups; q += kWave, ++b)
+        if (!(kept >> b & 1u))
+          for (int e = q * per; e < (q + 1) * per; ++e) choice[e] = -INFINITY;
+    }
+    by = choice;
+  }
+  wave_lds_sync();
+  uint32_t taken = 0;
+  int my_id = 0;
+  float my_w = 0.f;
+  for (int j = 0; j < k; ++j) {
+    float bv;
+    int best = wave_argmax(by, n_experts, lane, taken, &bv);
+    if (best < 0) best = 0;                // (cannot be: k <= n_experts)
+    if (best % kWave == lane) taken |= 1u << (best / kWave);
+    if (lane == j) {
+      my_id = best;
+      my_w = g[best];
+    }
+  }
+  if (gate == 2) {
+    float mx = __shfl(my_w, 0, kWave);
+    for (int j = 1; j < k; ++j) mx = fmaxf(mx, __shfl(my_w, j, kWave));
+    my_w = expf(my_w - mx);
+    float sum = 0.f;
+    for (int j = 0; j < k; ++j) sum += __shfl(my_w, j, kWave);
+    my_w *= 1.0f / sum;
+  } else if (renorm && k > 1) {
+    float sum = 0.f;
+    for (int j = 0; j < k; ++j) sum += __shfl(my_w, j, kWave);
+    if (sum > 0.f) my_w /= sum;
+  }
+  if (lane < k) {
+    ids[lane] = my_id;
+    w[lane] = w_scale != 1.0f ? my_w * w_scale : my_w;
+  }
+}
+
 // One wave: s[i] = wrow . xr[i] for TT rows, in float.  Lanes stride over the width in runs of 8
 // (one fused multiply-add chain per lane and row, in ascending order), then the lanes are summed:
 // the order of the additions depends on the width only, and each row has its own accumulator, so
@@ -197,7 +316,14 @@ __global__ __launch_bounds__(1024) void router_topk_kernel(const T* __restrict__
     }
   }
   __syncthreads();
-  if (threadIdx.x < TT && t0 + threadIdx.x < n_tokens) {
+  if (k <= kWave) {                          // a wave a token
+    if (w < TT && t0 + w < n_tokens) {
+      const int t = t0 + w;
+      gate_and_pick_wave(g[w], n_experts, k, gate, renorm, topk_ids + (size_t)t * k, topk_w + (size_t)t * k,
+                         gate_out ? gate_out + (size_t)t * n_experts : nullptr,
+                         split_choice ? choice_s + (size_t)w * (n_experts + n_groups) : nullptr, corr, n_groups, keep, w_scale, lane);
+    }
+  } else if (threadIdx.x < TT && t0 + threadIdx.x < n_tokens) {
     const int t = t0 + threadIdx.x;
     gate_and_pick(g[threadIdx.x], n_experts, k, gate, renorm, topk_ids + (size_t)t * k, topk_w + (size_t)t * k,
                   gate_out ? gate_out + (size_t)t * n_experts : nullptr,
@@ -260,8 +386,13 @@ __global__ __launch_bounds__(1024) void add_rmsnorm_router_kernel(
     if (lane == 0) g[0][e] = v[0];
   }
   __syncthreads();
-  if (threadIdx.x == 0)
+  if (k <= kWave) {
+    if (wv == 0)
+      gate_and_pick_wave(g[0], n_experts, k, gate, renorm, topk_ids + (size_t)t * k, topk_w + (size_t)t * k, nullptr, nullptr, nullptr,
+                         1, 1, 1.0f, lane);
+  } else if (threadIdx.x == 0) {
     gate_and_pick(g[0], n_experts, k, gate, renorm, topk_ids + (size_t)t * k, topk_w + (size_t)t * k, nullptr);
+  }
 }
 
 // h [T, hidden] float (updated), delta [T, hidden] bf16 or null, w the norm's weights (bf16 or float, or
