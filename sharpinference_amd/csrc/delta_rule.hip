@@ -35,6 +35,7 @@ typedef __attribute__((ext_vector_type(4))) float f32x4;
 
 constexpr int kDcTokens = 16;            // tokens of a chunk
 constexpr int kDrMaxTaps = 8;
+constexpr int kDies = 8;                 // dies that blocks are dealt to, round robin
 constexpr float kUnitFloor = 1e-6f;      // added to a sum of squares under the unit vectors' root
 constexpr float kLog2e = 1.4426950408889634f;
 
@@ -330,8 +331,9 @@ __global__ __launch_bounds__(512, NT <= 8 ? 4 : 2) void delta_step_kernel(DeltaI
 // ---------------------------------------------------------------------------
 // chunks of 16 tokens
 // ---------------------------------------------------------------------------
-// chunks int [n, 4] = (entry, first row, tokens, unused).  Per (chunk, head), in floats: W [16][dkp], Qd [16][dkp],
-// KT [dkp][16], D [dkp], U0 [dvp][16], A [16][16] (dkp, dvp: dk and dv rounded up to 16).
+// chunks int [n, 4] = (entry, first row, tokens, unused).  Per (chunk, head), in floats: W and Qd [dkp / 16][16
+// tokens][16 rows], KT [dkp][16], D [dkp], U0 [dvp][16], A [16][16] (dkp, dvp: dk and dv rounded up to 16): every operand of the
+// walk's matrix instructions is one contiguous kilobyte.
 struct ChunkBuf {
   float *W, *Qd, *KT, *D, *U0, *A;
 };
@@ -349,9 +351,15 @@ __global__ __launch_bounds__(256, DKP <= 128 ? 4 : 2) void delta_chunk_prep_kern
   float* beta_s = L_s + C * C;             // [C]
   float* v_s = beta_s + C;                 // [C][dv]
   const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
-  const int h = blockIdx.y;
-  const size_t ch = (size_t)blockIdx.x * a.nh + h;
-  const int e = chunks[4 * blockIdx.x], first = chunks[4 * blockIdx.x + 1], n = chunks[4 * blockIdx.x + 2];
+  // a head's chunks on the die that will walk them, where the heads divide so (blocks are dealt to the dies round robin)
+  int h = blockIdx.x % a.nh, chunk = blockIdx.x / a.nh;
+  if (a.nh % kDies == 0) {
+    const int per = a.nh / kDies, i = blockIdx.x / kDies;
+    h = blockIdx.x % kDies + kDies * (i % per);
+    chunk = i / per;
+  }
+  const size_t ch = (size_t)chunk * a.nh + h;
+  const int e = chunks[4 * chunk], first = chunks[4 * chunk + 1], n = chunks[4 * chunk + 2];
   const int local0 = first - a.cu_tokens[e], p0 = a.positions[first];
   const int kh = h / a.rep, dkp = (a.dk + 15) & ~15, dvp = (a.dv + 15) & ~15;
   const float* ring = a.ring ? a.ring + (size_t)a.state_slots[e] * a.taps * a.channels : nullptr;
@@ -454,8 +462,8 @@ __global__ __launch_bounds__(256, DKP <= 128 ? 4 : 2) void delta_chunk_prep_kern
     const float* k_c = k_s + c;
     const float* b_c = b_s + c;
     float x[C];
-    float* w_out = b.W + ch * C * dkp + c;
-    float* q_out = b.Qd + ch * C * dkp + c;
+    float* w_out = b.W + ch * C * dkp + (c >> 4) * 256 + (c & 15);
+    float* q_out = b.Qd + ch * C * dkp + (c >> 4) * 256 + (c & 15);
 #pragma unroll
     for (int t = 0; t < C; ++t) {
       float r;
@@ -463,7 +471,7 @@ __global__ __launch_bounds__(256, DKP <= 128 ? 4 : 2) void delta_chunk_prep_kern
         const float decayed = exp2_f32(b_c[t * ldk]);
         r = k_c[t * ldk] * decayed;
         *q_out = q_s[t * ldk + c] * decayed;
-        q_out += dkp;
+        q_out += 16;
       } else {
         r = c < a.dv ? v_s[t * a.dv + c] : 0.f;
       }
@@ -476,7 +484,7 @@ __global__ __launch_bounds__(256, DKP <= 128 ? 4 : 2) void delta_chunk_prep_kern
       x[t] = beta_s[t] * r;
       if (key) {
         *w_out = x[t];
-        w_out += dkp;
+        w_out += 16;
       }
       if (t % 2) __builtin_amdgcn_sched_barrier(0);      // (all rows read ahead would not fit the registers)
     }
@@ -501,16 +509,15 @@ __global__ __launch_bounds__(256, DKP <= 128 ? 4 : 2) void delta_chunk_prep_kern
 
 // Blocks of one (entry, head) go to one die (they read the same W, Qd and KT): with 8 dies dealt round robin, block L
 // takes group L % 8 + 8 (L / (8 ns)) and strip (L / 8) % ns.
-constexpr int kDies = 8;
 
 // Four waves hold the state (TPW 16-row tiles each), a fifth makes the outputs.  Per chunk: P = W S (a partial sum a wave, added
 // through LDS by everyone behind the chunk's one barrier), O = Qd S while those sums are on their way, U = U0 - P, S = D S + KT U.
 // The partial sums of O are read by the fifth wave behind the NEXT chunk's barrier, with the U it has kept.
 constexpr int kDwWaves = 4;
 
-template <typename T, int TPW>
-__global__ __launch_bounds__(kWave * (kDwWaves + 1)) void delta_chunk_walk_kernel(
-    DeltaIn a, const int* __restrict__ chunks, const int* __restrict__ ent_chunks, ChunkBuf b, float* __restrict__ out, int n_groups) {
+template <typename T, int TPW, int BUFS>      // BUFS - 1: chunks whose operands are requested ahead
+__global__ __launch_bounds__(kWave * (kDwWaves + 1), 1) void delta_chunk_walk_kernel(
+    DeltaIn a, const int* __restrict__ ent_chunks, ChunkBuf b, float* __restrict__ out, int n_groups) {
   constexpr int C = kDcTokens, NW = kDwWaves;
   __shared__ __attribute__((aligned(16))) f32x4 p_s[2][NW][kWave], o_s[2][NW][kWave];
   const int ns = (a.dv + 15) >> 4, nt = (a.dk + 15) >> 4, dkp = nt * 16, dvp = ns * 16;
@@ -521,6 +528,7 @@ __global__ __launch_bounds__(kWave * (kDwWaves + 1)) void delta_chunk_walk_kerne
   const int c_first = ent_chunks[2 * e], c_n = ent_chunks[2 * e + 1];
   const int slot = a.state_slots[e];
   const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+  const unsigned at_u = (strip * 16 + m) * C + 4 * g;
   if (w < NW) {
     float* st = a.state + (((size_t)slot * a.nh + h) * ns + strip) * nt * 256;
     f32x4 S[TPW];
@@ -534,20 +542,28 @@ __global__ __launch_bounds__(kWave * (kDwWaves + 1)) void delta_chunk_walk_kerne
     }
     struct Ops {
       f32x4 W[TPW], Q[TPW], K[TPW], D[TPW], U;
-    } buf[3];
+    } buf[BUFS];
+    unsigned at_row[TPW], at_kt[TPW], at_d[TPW];
+#pragma unroll
+    for (int n = 0; n < TPW; ++n) {
+      at_row[n] = tile[n] * 256 + m * 16 + 4 * g;
+      at_kt[n] = (16 * tile[n] + m) * C + 4 * g;
+      at_d[n] = 16 * tile[n] + 4 * g;
+    }
     auto fetch = [&](int c, Ops& o) {          // (chunks beyond the last: the last once more, no load behind a branch)
       const size_t ch = (size_t)(c_first + min(c, c_n - 1)) * a.nh + h;
+      const float *W = b.W + ch * C * dkp, *Qd = b.Qd + ch * C * dkp, *KT = b.KT + ch * C * dkp, *D = b.D + ch * dkp, *U0 = b.U0 + ch * C * dvp;
 #pragma unroll
       for (int n = 0; n < TPW; ++n) {
-        o.W[n] = *reinterpret_cast<const f32x4*>(b.W + (ch * C + m) * dkp + 16 * tile[n] + 4 * g);
-        o.Q[n] = *reinterpret_cast<const f32x4*>(b.Qd + (ch * C + m) * dkp + 16 * tile[n] + 4 * g);
-        o.K[n] = *reinterpret_cast<const f32x4*>(b.KT + (ch * dkp + 16 * tile[n] + m) * C + 4 * g);
-        o.D[n] = *reinterpret_cast<const f32x4*>(b.D + ch * dkp + 16 * tile[n] + 4 * g);
+        o.W[n] = *reinterpret_cast<const f32x4*>(W + at_row[n]);
+        o.Q[n] = *reinterpret_cast<const f32x4*>(Qd + at_row[n]);
+        o.K[n] = *reinterpret_cast<const f32x4*>(KT + at_kt[n]);
+        o.D[n] = *reinterpret_cast<const f32x4*>(D + at_d[n]);
       }
-      o.U = *reinterpret_cast<const f32x4*>(b.U0 + (ch * dvp + strip * 16 + m) * C + 4 * g);
+      o.U = *reinterpret_cast<const f32x4*>(U0 + at_u);
     };
     auto one = [&](int c, const Ops& o, Ops& ahead) {
-      fetch(c + 2, ahead);
+      fetch(c + BUFS - 1, ahead);
       f32x4 P = zero, O = zero;
 #pragma unroll
       for (int n = 0; n < TPW; ++n)
@@ -555,6 +571,7 @@ __global__ __launch_bounds__(kWave * (kDwWaves + 1)) void delta_chunk_walk_kerne
         for (int i = 0; i < 4; ++i) P = mfma4(o.W[n][i], S[n][i], P);
       p_s[c & 1][w][lane] = P;
       __syncthreads();
+      __builtin_amdgcn_sched_barrier(0);       // (O's products stay behind the barrier: they cover the reads of the shares)
       f32x4 part[NW];
 #pragma unroll
       for (int i = 0; i < NW; ++i) part[i] = p_s[c & 1][i][lane];
@@ -573,51 +590,65 @@ __global__ __launch_bounds__(kWave * (kDwWaves + 1)) void delta_chunk_walk_kerne
       }
       o_s[c & 1][w][lane] = O;
     };
-    fetch(0, buf[0]);
-    fetch(1, buf[1]);
+#pragma unroll
+    for (int i = 0; i + 1 < BUFS; ++i) fetch(i, buf[i]);
     int c = 0;
-    for (; c + 3 <= c_n; c += 3) {
-      one(c, buf[0], buf[2]);
-      one(c + 1, buf[1], buf[0]);
-      one(c + 2, buf[2], buf[1]);
+    for (; c + BUFS <= c_n; c += BUFS) {
+#pragma unroll
+      for (int i = 0; i < BUFS; ++i) one(c + i, buf[i], buf[(i + BUFS - 1) % BUFS]);
     }
-    if (c < c_n) one(c, buf[0], buf[2]);
-    if (c + 1 < c_n) one(c + 1, buf[1], buf[0]);
+#pragma unroll
+    for (int i = 0; i + 1 < BUFS; ++i)
+      if (c + i < c_n) one(c + i, buf[i], buf[(i + BUFS - 1) % BUFS]);
     __syncthreads();                           // (the last chunk's shares of the outputs are there)
 #pragma unroll
     for (int n = 0; n < TPW; ++n)
       if (has[n]) *reinterpret_cast<f32x4*>(st + (size_t)tile[n] * 256 + lane * 4) = S[n];
   } else {
-    const int col = strip * 16 + m;
-    f32x4 U_before = zero, A_before = zero;
-    auto u_of = [&](int c) { return *reinterpret_cast<const f32x4*>(b.U0 + (((size_t)(c_first + c) * a.nh + h) * dvp + strip * 16 + m) * C + 4 * g); };
-    auto a_of = [&](int c) { return *reinterpret_cast<const f32x4*>(b.A + ((size_t)(c_first + c) * a.nh + h) * 256 + m * 16 + 4 * g); };
-    f32x4 U_next = u_of(0), A_next = a_of(0);
-    for (int c = 0; c <= c_n; ++c) {
-      f32x4 U = U_next, A = A_next;
-      U_next = u_of(min(c + 1, c_n - 1));
-      A_next = a_of(min(c + 1, c_n - 1));
-      __syncthreads();                         // chunk c's P, chunk c - 1's O (the last time: its O alone)
-      if (c > 0) {
-        f32x4 y = zero;
+    const int col = strip * 16 + m, row0 = a.cu_tokens[e], len = a.cu_tokens[e + 1] - row0;
+    const unsigned at_a = m * 16 + 4 * g;
+    f32x4 u[BUFS], A[BUFS], U_before = zero, A_before = zero;
+    auto fetch = [&](int c, int i) {
+      const size_t ch = (size_t)(c_first + min(c, c_n - 1)) * a.nh + h;
+      u[i] = *reinterpret_cast<const f32x4*>(b.U0 + ch * C * dvp + at_u);
+      A[i] = *reinterpret_cast<const f32x4*>(b.A + ch * 256 + at_a);
+    };
+    auto emit = [&](int c) {                   // chunk c's outputs (its P, O and U are known)
+      f32x4 y = zero;
 #pragma unroll
-        for (int i = 0; i < NW; ++i) y += o_s[(c - 1) & 1][i][lane];
+      for (int i = 0; i < NW; ++i) y += o_s[c & 1][i][lane];
 #pragma unroll
-        for (int i = 0; i < 4; ++i) y = mfma4(A_before[i], U_before[i], y);
-        const int first = chunks[4 * (c_first + c - 1) + 1], cnt = chunks[4 * (c_first + c - 1) + 2];
-        if (col < a.dv) {
+      for (int i = 0; i < 4; ++i) y = mfma4(A_before[i], U_before[i], y);
+      const int t = c * C + 4 * g;
+      float* to = out + (size_t)(row0 + t) * a.nh * a.dv + (size_t)h * a.dv + col;
+      if (col < a.dv) {
 #pragma unroll
-          for (int i = 0; i < 4; ++i)
-            if (4 * g + i < cnt) out[(size_t)(first + 4 * g + i) * a.nh * a.dv + (size_t)h * a.dv + col] = y[i];
-        }
+        for (int i = 0; i < 4; ++i)
+          if (t + i < len) to[(size_t)i * a.nh * a.dv] = y[i];
       }
-      if (c < c_n) {
+    };
+    auto one = [&](int c, int i) {
+      fetch(c + BUFS - 1, (i + BUFS - 1) % BUFS);
+      __syncthreads();                         // chunk c's P, chunk c - 1's O
+      f32x4 U = u[i];
 #pragma unroll
-        for (int i = 0; i < NW; ++i) U -= p_s[c & 1][i][lane];
-        U_before = U;
-        A_before = A;
-      }
+      for (int j = 0; j < NW; ++j) U -= p_s[c & 1][j][lane];
+      if (c > 0) emit(c - 1);
+      U_before = U;
+      A_before = A[i];
+    };
+#pragma unroll
+    for (int i = 0; i + 1 < BUFS; ++i) fetch(i, i);
+    int c = 0;
+    for (; c + BUFS <= c_n; c += BUFS) {
+#pragma unroll
+      for (int i = 0; i < BUFS; ++i) one(c + i, i);
     }
+#pragma unroll
+    for (int i = 0; i + 1 < BUFS; ++i)
+      if (c + i < c_n) one(c + i, i);
+    __syncthreads();
+    emit(c_n - 1);
   }
   // the convolution's last inputs (everybody who reads the ring has run: the kernel before this one)
   if (a.ring && strip == 0) {
@@ -698,7 +729,7 @@ SHARPI_EXPORT int sharpi_delta_chunks(const void* proj, int dtype, int stride, i
   const DeltaIn a = delta_in(proj, stride, c_off, conv_w, taps, ring, log_decay, beta, beta_stride, beta_off, positions, state_slots,
                              cu_tokens, state, nh, nkv, dk, dv, q_scale);
   if (nkv <= 0 || !delta_args_ok(a, n_entries) || !chunks || !ent_chunks || !work || !out || n_chunks < n_entries) return SHARPI_ERR_ARG;
-  if (dtype != DT_F32 && dtype != DT_BF16) return SHARPI_ERR_ARG;
+  if ((dtype != DT_F32 && dtype != DT_BF16) || (long long)n_chunks * nh > 0x7fffffff) return SHARPI_ERR_ARG;
   const int dkp = (dk + 15) / 16 * 16, dvp = (dv + 15) / 16 * 16, nt = dkp / 16, ns = dvp / 16;
   const size_t per = (size_t)n_chunks * nh;
   ChunkBuf b;
@@ -720,7 +751,7 @@ SHARPI_EXPORT int sharpi_delta_chunks(const void* proj, int dtype, int stride, i
       if (e_ != hipSuccess) return (int)e_;                                                                         \
       allowed = lds;                                                                                                \
     }                                                                                                               \
-    kern<<<dim3(n_chunks, nh), 256, lds, stream>>>(a, chunks, b);                                                   \
+    kern<<<n_chunks * nh, 256, lds, stream>>>(a, chunks, b);                                                        \
   } while (0)
 #define PREP_BY(TV, TAPS)                         \
   do {                                            \
@@ -742,12 +773,12 @@ SHARPI_EXPORT int sharpi_delta_chunks(const void* proj, int dtype, int stride, i
   const int groups = n_entries * nh;
   const long long blocks = (long long)ceil_div(groups, kDies) * kDies * ns;
   if (blocks > 0x7fffffff) return SHARPI_ERR_ARG;
-#define WALK(TV, TPW) delta_chunk_walk_kernel<TV, TPW><<<(unsigned)blocks, kWave * (kDwWaves + 1), 0, stream>>>(a, chunks, ent_chunks, b, out, groups)
+#define WALK(TV, TPW, BUFS) delta_chunk_walk_kernel<TV, TPW, BUFS><<<(unsigned)blocks, kWave * (kDwWaves + 1), 0, stream>>>(a, ent_chunks, b, out, groups)
 #define WALK_BY(TV)                  \
   do {                               \
-    if (nt <= 4) WALK(TV, 1);        \
-    else if (nt <= 8) WALK(TV, 2);   \
-    else WALK(TV, 4);                \
+    if (nt <= 4) WALK(TV, 1, 6);     \
+    else if (nt <= 8) WALK(TV, 2, 5);\
+    else WALK(TV, 4, 2);             \
   } while (0)
   if (dtype == DT_F32) WALK_BY(float);
   else WALK_BY(bf16_t);
