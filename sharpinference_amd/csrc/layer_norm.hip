@@ -40,12 +40,20 @@ __device__ __forceinline__ void ln_delta(const LnDelta& d, size_t r, int hidden,
   }
 #pragma unroll
   for (int i = 0; i < V; ++i) v[i] = 0.f;
-  for (int q = 0; q < d.k; ++q) {
-    float x[V];
-    ln_load<TD, V>((const TD*)d.y + (size_t)d.pos[r * d.k + q] * hidden + c, x);
-    const float wq = d.w ? d.w[r * d.k + q] : 1.0f;
+  for (int q0 = 0; q0 < d.k; q0 += 4) {    // (four rows are requested before the first is added)
+    float x[4][V], wq[4];
 #pragma unroll
-    for (int i = 0; i < V; ++i) v[i] = fmaf(wq, x[i], v[i]);
+    for (int j = 0; j < 4; ++j) {
+      const int q = min(q0 + j, d.k - 1);
+      ln_load<TD, V>((const TD*)d.y + (size_t)d.pos[r * d.k + q] * hidden + c, x[j]);
+      wq[j] = d.w ? d.w[r * d.k + q] : 1.0f;
+    }
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      if (q0 + j < d.k) {
+#pragma unroll
+        for (int i = 0; i < V; ++i) v[i] = fmaf(wq[j], x[j][i], v[i]);
+      }
   }
   if (d.shared) {
     float x[V];
@@ -160,6 +168,102 @@ __global__ __launch_bounds__(1024) void layer_norm_kernel(float* __restrict__ h,
   }
 }
 
+// The same where a thread has one run of eight elements of the row (hidden a multiple of 8 up to 8,192): everything stays in
+// registers, and what is needed behind the two reductions (h, weights, the earlier inputs of the convolution) is
+// requested before them: with a handful of rows (decode) the kernel is nothing but the latency of its loads.
+template <typename TD, typename TO, int TAPS>      // TAPS: the convolution's (LN_CONV), else 0
+__global__ __launch_bounds__(1024) void layer_norm_run_kernel(float* __restrict__ h, LnDelta delta, const float* __restrict__ w,
+                                                              const float* __restrict__ b, float eps, const int* __restrict__ rows,
+                                                              int write_back, TO* __restrict__ out, int mode,
+                                                              const float* __restrict__ w2, const float* __restrict__ b2, float eps2,
+                                                              LnConv cv, int hidden) {
+  __shared__ float red[16];
+  constexpr int N = TAPS > 1 ? TAPS : 1;
+  const size_t i = blockIdx.x, r = rows ? rows[i] : i;
+  const int c = threadIdx.x * 8;
+  const bool in = c < hidden;
+  float* hr = h + r * hidden;
+  float x[8], y[8], wv[8], bv[8], past[N][8], cw[N * 8];
+  float* ring = nullptr;
+  int p = 0;
+  if (in) {
+    load8(hr + c, x);
+    if (delta.y) {
+      ln_delta<TD, 8>(delta, r, hidden, c, y);
+      load8(w + c, wv);
+      load8(b + c, bv);
+    }
+    if constexpr (TAPS > 0) {
+      p = cv.positions[r];
+#pragma unroll
+      for (int k = 0; k < TAPS; ++k) load8(cv.w + (size_t)c * TAPS + k * 8, cw + k * 8);      // channel c + k's taps at k TAPS
+      if constexpr (TAPS > 1) {
+        ring = cv.ring + (size_t)cv.state_slots[cv.entry_of_token[r]] * TAPS * hidden + c;
+#pragma unroll
+        for (int back = 1; back < TAPS; ++back)          // (before position 0: some row of the ring, not used)
+          load8(ring + (size_t)((p + TAPS - back) % TAPS) * hidden, past[back]);
+      }
+    }
+  }
+  if (delta.y) {
+    float s = 0.f;
+    if (in) {
+#pragma unroll
+      for (int k = 0; k < 8; ++k) s += y[k];
+    }
+    const float mean = block_sum(s, red) / (float)hidden;
+    s = 0.f;
+    if (in) {
+#pragma unroll
+      for (int k = 0; k < 8; ++k) s = fmaf(y[k] - mean, y[k] - mean, s);
+    }
+    const float inv = 1.0f / sqrtf(block_sum(s, red) / (float)hidden + eps);
+    if (in) {
+#pragma unroll
+      for (int k = 0; k < 8; ++k) x[k] += fmaf((y[k] - mean) * inv, wv[k], bv[k]);
+      if (write_back) store8(hr + c, x);
+    }
+  }
+  if (!out) return;
+  TO* o = out + i * hidden + c;
+  if (mode == LN_COPY) {
+    if (in) store8(o, x);
+  } else if (mode == LN_NORM) {
+    float s = 0.f;
+    if (in) {
+      load8(w2 + c, wv);
+      load8(b2 + c, bv);
+#pragma unroll
+      for (int k = 0; k < 8; ++k) s += x[k];
+    }
+    const float mean = block_sum(s, red) / (float)hidden;
+    s = 0.f;
+    if (in) {
+#pragma unroll
+      for (int k = 0; k < 8; ++k) s = fmaf(x[k] - mean, x[k] - mean, s);
+    }
+    const float inv = 1.0f / sqrtf(block_sum(s, red) / (float)hidden + eps2);
+    if (in) {
+#pragma unroll
+      for (int k = 0; k < 8; ++k) x[k] = fmaf((x[k] - mean) * inv, wv[k], bv[k]);
+      store8(o, x);
+    }
+  } else if constexpr (TAPS > 0) {
+    if (in) {
+#pragma unroll
+      for (int k = 0; k < 8; ++k) y[k] = 0.f;
+#pragma unroll
+      for (int back = TAPS - 1; back > 0; --back)
+#pragma unroll
+        for (int k = 0; k < 8; ++k) y[k] = p >= back ? fmaf(cw[k * TAPS + TAPS - 1 - back], past[back][k], y[k]) : y[k];
+      if constexpr (TAPS > 1) store8(ring + (size_t)(p % TAPS) * hidden, x);
+#pragma unroll
+      for (int k = 0; k < 8; ++k) x[k] += fmaf(cw[k * TAPS + TAPS - 1], x[k], y[k]);
+      store8(o, x);
+    }
+  }
+}
+
 // h [T, hidden] float.  With delta (y of d_dtype; pos/sum_w/k/shared describe an expert sum): x = h + LN(delta) w + b,
 // back into h unless `rows` (int32 [n_rows]: only those rows, h unchanged) is given.  out (o_dtype, or null), mode 0:
 // x; 1: LN(x) w2 + b2; 2: x + conv(x) with conv_w float [hidden, taps] and the entries' rings (every entry of
@@ -187,6 +291,31 @@ SHARPI_EXPORT int sharpi_layer_norm(float* h, const void* delta, int d_dtype, co
   if (threads > (wide ? 1024 : 256)) threads = wide ? 1024 : 256;
   const size_t lds = (size_t)hidden * sizeof(float);
   const int wb = rows ? 0 : 1;
+  // (with more taps the registers do not reach)
+  if (wide && hidden <= 8192 && (mode != LN_CONV || !out || (aligned(conv_w) && taps <= 5))) {
+    const int t = mode == LN_CONV && out ? taps : 0;
+#define LNR(TD, TO, TAPS)                                                                                                             \
+  case TAPS:                                                                                                                          \
+    layer_norm_run_kernel<TD, TO, TAPS><<<n_rows, threads, 0, stream>>>(h, d, w, b, eps, rows, wb, (TO*)out, mode, w2, b2, eps2, cv, hidden); \
+    break
+#define LNR_BY(TD, TO)                                                                                                                \
+  switch (t) {                                                                                                                        \
+    LNR(TD, TO, 0); LNR(TD, TO, 1); LNR(TD, TO, 2); LNR(TD, TO, 3); LNR(TD, TO, 4); LNR(TD, TO, 5); \
+    default: return SHARPI_ERR_ARG;                                                                                                   \
+  }
+    const bool to_f = !out || o_dtype == DT_F32;
+    if (d_dtype == DT_F32) {
+      if (to_f) { LNR_BY(float, float) }
+      else { LNR_BY(float, bf16_t) }
+    } else {
+      if (to_f) { LNR_BY(bf16_t, float) }
+      else { LNR_BY(bf16_t, bf16_t) }
+    }
+#undef LNR_BY
+#undef LNR
+    SHARPI_CHECK_LAUNCH();
+    return SHARPI_OK;
+  }
 #define LN(TD, TO)                                                                                                                    \
   do {                                                                                                                                \
     if (wide) layer_norm_kernel<TD, TO, 8><<<n_rows, threads, lds, stream>>>(h, d, w, b, eps, rows, wb, (TO*)out, mode, w2, b2, eps2, cv, hidden); \
