@@ -743,7 +743,7 @@ def pagonex_config(z: dict) -> dict:
     layers = [{"type": kind, "mixer": dict(delta if kind == "channel_delta" else latent), "mlp": mlp} for kind in PAGONEX_KINDS[:z["layers"]]]
     layers[2]["mixer"]["kv_from"] = 1
     return {"architecture": "Pagonex", "vocab": z["vocab"], "width": z["width"], "norm": {"eps": 1e-5}, "canon": {"taps": 4},
-            "embedding": {"bigram": {"buckets": 100003, "mul_prev": 31, "mul_cur": 7}}, "logit_scale": 1.0, "layers": layers}
+            "embedding": {"bigram": {"buckets": 100003, "mul_prev": 10007, "mul_cur": 257}}, "logit_scale": 1.0, "layers": layers}
 
 
 def pazatar_like_pagonex(z: dict) -> dict:
