@@ -6,7 +6,8 @@ entry b names the page that holds positions [b * page_size, (b + 1) * page_size)
 layer of a group uses the same page ids in its own tensor, as the reference shares one slot
 index across layers (reference: src/SharpInference.Engine/PagedKvCache.cs:34-44, 144-148); unlike the
 reference, the pools are shared by all requests.  Pages return to the pool when a request ends
-and, in a windowed group, as soon as no later query can see them; nothing is cleared on
+and, in a windowed group, as soon as no later query can see them (pages that hold first keys
+which the window keeps in sight stay with the request); nothing is cleared on
 release (lengths and block tables mask stale contents).  Requests also hold one *state slot*
 each: an index into per-layer tensors of fixed size, zeroed at admission
 (reference: src/SharpInference.Engine/GdnStateCache.cs:7-33).
@@ -32,13 +33,13 @@ class CacheError(RuntimeError):
 def pages_to_hold(spec: KVSpec, page_size: int, total_tokens: int, max_step_tokens: int) -> int:
     """Upper bound of the pages a request of `total_tokens` holds at once under `spec` when no step
     brings more than `max_step_tokens` of it: all of them without a window; with one, the window,
-    the step that is being appended before the pages behind the window are given back, and one
-    page for the edges."""
+    the step that is being appended before the pages behind the window are given back, one
+    page for the edges, and the pages of the first keys that the window keeps."""
     full = (total_tokens + page_size - 1) // page_size
     if spec.window_kind == 0:
         return full
     span = spec.window + max(1, max_step_tokens)
-    return min(full, (span + page_size - 1) // page_size + 1)
+    return min(full, (span + page_size - 1) // page_size + 1 + spec.kept_blocks(page_size))
 
 
 def pool_sizes(slot_specs, page_size: int, max_requests: int, total_tokens: int, max_step_tokens: int,
@@ -135,7 +136,7 @@ class CacheManager:
                 if key not in by_key:
                     n = num_pages[key] if isinstance(num_pages, dict) else int(num_pages)
                     by_key[key] = len(self.groups)
-                    self.groups.append(CacheGroup(key, KVSpec(0, 0, spec.window_kind, spec.window), PagePool(n)))
+                    self.groups.append(CacheGroup(key, KVSpec(0, 0, spec.window_kind, spec.window, keep_first=spec.keep_first), PagePool(n)))
                 g = by_key[key]
                 self.groups[g].slots.append(i)
                 self.group_of_slot.append(g)
@@ -299,7 +300,8 @@ class CacheManager:
             first_needed = grp.spec.first_visible(rc.length)   # the next query sits at position `length`
             tbl = rc.tables[g]
             upto = min(first_needed // self.page_size, len(tbl))
-            for b in range(rc.passed[g], upto):                # (blocks below `passed` went back in earlier steps)
+            # (blocks below `passed` went back in earlier steps; those of kept first keys never do)
+            for b in range(max(rc.passed[g], grp.spec.kept_blocks(self.page_size)), upto):
                 if tbl[b] >= 0:
                     grp.pool.release(tbl[b])
                     tbl[b] = -1

@@ -32,6 +32,7 @@ class KVSpec:
     window: int = 0
     v_head_dim: int = 0
     values_in_keys: bool = False     # the values are a leading part of the key rows: no value tensor is kept
+    keep_first: int = 0              # beside its window a query sees the sequence's first `keep_first` keys
 
     @property
     def value_dim(self) -> int:
@@ -43,16 +44,25 @@ class KVSpec:
         return self.num_kv_heads * (self.head_dim + (0 if self.values_in_keys else self.value_dim))
 
     def first_visible(self, pos: int) -> int:
-        """The earliest key position a query at `pos` can see."""
+        """The earliest key position a query at `pos` can see in its window (kept first keys lie before it)."""
         if self.window_kind == WINDOW_CHUNK:
             return (pos // self.window) * self.window
         if self.window_kind == WINDOW_SLIDING:
             return max(0, pos - self.window + 1)
         return 0
 
+    def keys_seen(self, pos: int) -> int:
+        """How many keys a query at `pos` sees: its window's, and the kept ones before it."""
+        first = self.first_visible(pos)
+        return pos - first + 1 + min(self.keep_first, first)
+
+    def kept_blocks(self, page_size: int) -> int:
+        """Pages at a sequence's start that are never given back while the request lives."""
+        return (self.keep_first + page_size - 1) // page_size if self.window_kind != WINDOW_NONE else 0
+
     def group_key(self):
         # layers whose pages live and die together share a block table
-        return ("kv", self.window_kind, self.window)
+        return ("kv", self.window_kind, self.window) + ((self.keep_first,) if self.keep_first else ())
 
 
 @dataclass(frozen=True)

@@ -110,6 +110,21 @@ __device__ __forceinline__ float gated_f32(GatedAct actp, float g, float u, floa
   return (g / (1.0f + expf(-g))) * u;
 }
 
+// An activation without a gate, one element (feed-forwards down(f(up x))).  Codes shared with the Python side: the
+// square of relu; GELU in its tanh form; SiLU; GELU as x times the normal distribution function (erf).
+// One definition for the activation kernel and for the products that apply it in their epilogue.
+enum : int { UACT_NONE = 0, UACT_RELU2 = 1, UACT_GELU_TANH = 2, UACT_SILU = 3, UACT_GELU = 4 };
+static inline __host__ __device__ bool uact_known(int f) { return f >= UACT_RELU2 && f <= UACT_GELU; }
+__device__ __forceinline__ float ungated_f32(int f, float v) {
+  if (f == UACT_RELU2) {
+    const float r = fmaxf(v, 0.f);
+    return r * r;
+  }
+  if (f == UACT_GELU_TANH) return 0.5f * v * (1.0f + tanhf(0.7978845608028654f * (v + 0.044715f * v * v * v)));
+  if (f == UACT_GELU) return 0.5f * v * (1.0f + erff(v * 0.7071067811865476f));
+  return v / (1.0f + expf(-v));
+}
+
 // dtype codes shared with the Python side
 enum : int { DT_F32 = 0, DT_BF16 = 1 };
 

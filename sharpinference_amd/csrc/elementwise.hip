@@ -332,13 +332,15 @@ SHARPI_EXPORT int sharpi_silu_mul(const void* gu, const float* scale, void* out,
 template <typename T>
 __global__ void moe_combine_kernel(const T* __restrict__ y, const int* __restrict__ inv_pos,
                                    const T* __restrict__ shared, const float* __restrict__ w,
-                                   T* __restrict__ out, int hidden, int k) {
+                                   T* __restrict__ out, int hidden, int k, const int* __restrict__ ids, int n_experts,
+                                   const T* __restrict__ ident) {
   const int t = blockIdx.x;
   const int c = blockIdx.y * blockDim.x + threadIdx.x;
   if (c >= hidden) return;
   float acc = 0.f;
   for (int j = 0; j < k; ++j) {
-    const float v = to_f32<T>(y[(size_t)inv_pos[t * k + j] * hidden + c]);
+    const bool self = ids && ids[t * k + j] >= n_experts;      // an identity expert returns the token's own row
+    const float v = to_f32<T>(self ? ident[(size_t)t * hidden + c] : y[(size_t)inv_pos[t * k + j] * hidden + c]);
     acc += w ? w[t * k + j] * v : v;
   }
   if (shared) acc += to_f32<T>(shared[(size_t)t * hidden + c]);
@@ -348,14 +350,15 @@ __global__ void moe_combine_kernel(const T* __restrict__ y, const int* __restric
 template <typename T>
 __global__ void moe_combine_vec_kernel(const T* __restrict__ y, const int* __restrict__ inv_pos,
                                        const T* __restrict__ shared, const float* __restrict__ w,
-                                       T* __restrict__ out, int hidden, int k) {
+                                       T* __restrict__ out, int hidden, int k, const int* __restrict__ ids, int n_experts,
+                                       const T* __restrict__ ident) {
   const int t = blockIdx.x;
   const int c = (blockIdx.y * blockDim.x + threadIdx.x) * 8;
   if (c >= hidden) return;
   float acc[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
   for (int j = 0; j < k; ++j) {
     float v[8];
-    load8(y + (size_t)inv_pos[t * k + j] * hidden + c, v);
+    load8(ids && ids[t * k + j] >= n_experts ? ident + (size_t)t * hidden + c : y + (size_t)inv_pos[t * k + j] * hidden + c, v);
     const float wj = w ? w[t * k + j] : 1.0f;
 #pragma unroll
     for (int i = 0; i < 8; ++i) acc[i] += w ? wj * v[i] : v[i];
@@ -369,9 +372,12 @@ __global__ void moe_combine_vec_kernel(const T* __restrict__ y, const int* __res
   store8(out + (size_t)t * hidden + c, acc);
 }
 
+// ids (int32 [T, k], or null): picks of n_experts and above are identity experts, whose output is row t of ident [T, hidden].
 SHARPI_EXPORT int sharpi_moe_combine(const void* y, const int* inv_pos, const void* shared, const float* w, void* out, int dtype,
-                                     int n_tokens, int hidden, int k, hipStream_t stream) {
+                                     int n_tokens, int hidden, int k, const int* ids, int n_experts, const void* ident,
+                                     hipStream_t stream) {
   if (n_tokens <= 0) return SHARPI_OK;
+  if (ids && !ident) return SHARPI_ERR_ARG;
   if (hidden <= 0 || k <= 0 || ceil_div(hidden, 256) > 65535) return SHARPI_ERR_ARG;
   dim3 block(256), grid(n_tokens, ceil_div(hidden, 256));
   if (dtype != DT_F32 && dtype != DT_BF16) return SHARPI_ERR_ARG;
@@ -379,16 +385,16 @@ SHARPI_EXPORT int sharpi_moe_combine(const void* y, const int* inv_pos, const vo
     dim3 vblock(128), vgrid(n_tokens, ceil_div(hidden, 128 * 8));
     if (dtype == DT_F32)
       moe_combine_vec_kernel<float><<<vgrid, vblock, 0, stream>>>((const float*)y, inv_pos, (const float*)shared, w,
-                                                                 (float*)out, hidden, k);
+                                                                 (float*)out, hidden, k, ids, n_experts, (const float*)ident);
     else
       moe_combine_vec_kernel<bf16_t><<<vgrid, vblock, 0, stream>>>((const bf16_t*)y, inv_pos, (const bf16_t*)shared, w,
-                                                                  (bf16_t*)out, hidden, k);
+                                                                  (bf16_t*)out, hidden, k, ids, n_experts, (const bf16_t*)ident);
   } else if (dtype == DT_F32)
     moe_combine_kernel<float><<<grid, block, 0, stream>>>((const float*)y, inv_pos, (const float*)shared, w,
-                                                         (float*)out, hidden, k);
+                                                         (float*)out, hidden, k, ids, n_experts, (const float*)ident);
   else
     moe_combine_kernel<bf16_t><<<grid, block, 0, stream>>>((const bf16_t*)y, inv_pos, (const bf16_t*)shared, w,
-                                                          (bf16_t*)out, hidden, k);
+                                                          (bf16_t*)out, hidden, k, ids, n_experts, (const bf16_t*)ident);
   SHARPI_CHECK_LAUNCH();
   return SHARPI_OK;
 }
@@ -467,30 +473,38 @@ SHARPI_EXPORT int sharpi_scale_softcap(float* x, long long n, float scale, float
 }
 
 // ---------------------------------------------------------------------------
-// An ungated activation, element by element: out = f(x).  f: 1 the square of relu; 2 tanh-GELU;
-// 3 SiLU.  For feed-forwards without a gate (down(f(up x))).
+// An ungated activation, element by element: out = f(x), f a code of common.h (UACT_*).  For
+// feed-forwards without a gate (down(f(up x))).  Eight elements a thread where the array allows it.
 // ---------------------------------------------------------------------------
 template <typename T>
 __global__ void activation_kernel(const T* __restrict__ x, T* __restrict__ out, size_t n, int f) {
-  for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (size_t)gridDim.x * blockDim.x) {
-    const float v = to_f32<T>(x[i]);
-    float y;
-    if (f == 1) {
-      const float r = fmaxf(v, 0.f);
-      y = r * r;
-    } else if (f == 2) {
-      y = 0.5f * v * (1.0f + tanhf(0.7978845608028654f * (v + 0.044715f * v * v * v)));
-    } else {
-      y = v / (1.0f + expf(-v));
-    }
-    out[i] = from_f32<T>(y);
+  for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (size_t)gridDim.x * blockDim.x)
+    out[i] = from_f32<T>(ungated_f32(f, to_f32<T>(x[i])));
+}
+
+template <typename T>
+__global__ void activation8_kernel(const T* __restrict__ x, T* __restrict__ out, size_t n8, int f) {
+  for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < n8; i += (size_t)gridDim.x * blockDim.x) {
+    float v[8];
+    load8(x + i * 8, v);
+#pragma unroll
+    for (int k = 0; k < 8; ++k) v[k] = ungated_f32(f, v[k]);
+    store8(out + i * 8, v);
   }
 }
 
 SHARPI_EXPORT int sharpi_activation(const void* x, void* out, int dtype, long long n, int f, hipStream_t stream) {
   if (n <= 0) return SHARPI_OK;
-  if (f < 1 || f > 3) return SHARPI_ERR_ARG;
-  const dim3 block(256), grid((unsigned)min((long long)8192, (n + 255) / 256));
+  if (!uact_known(f)) return SHARPI_ERR_ARG;
+  const dim3 block(256);
+  if (n % 8 == 0 && ((uintptr_t)x & 31) == 0 && ((uintptr_t)out & 31) == 0 && (dtype == DT_F32 || dtype == DT_BF16)) {
+    const dim3 grid8((unsigned)min((long long)16384, (n / 8 + 255) / 256));
+    if (dtype == DT_F32) activation8_kernel<float><<<grid8, block, 0, stream>>>((const float*)x, (float*)out, (size_t)n / 8, f);
+    else activation8_kernel<bf16_t><<<grid8, block, 0, stream>>>((const bf16_t*)x, (bf16_t*)out, (size_t)n / 8, f);
+    SHARPI_CHECK_LAUNCH();
+    return SHARPI_OK;
+  }
+  const dim3 grid((unsigned)min((long long)8192, (n + 255) / 256));
   if (dtype == DT_F32) activation_kernel<float><<<grid, block, 0, stream>>>((const float*)x, (float*)out, (size_t)n, f);
   else if (dtype == DT_BF16) activation_kernel<bf16_t><<<grid, block, 0, stream>>>((const bf16_t*)x, (bf16_t*)out, (size_t)n, f);
   else return SHARPI_ERR_ARG;

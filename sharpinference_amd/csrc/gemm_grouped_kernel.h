@@ -33,6 +33,8 @@
 //    products of its outputs, rounds them to bfloat16 (what a separate activation kernel would have
 //    read) and stores act(s g) * (s u), s the row's score: out is [rows, N/2] and the gate|up
 //    rows never go to memory.
+//  * The plain form may square the relu of its results (relu2: feed-forwards without a gate), rounded to
+//    bfloat16 first (what a separate activation kernel would have read).
 // Limits: K % 64 == 0, N % 4 == 0 (N % 32 == 0 in the SwiGLU form).
 #pragma once
 #include <type_traits>
@@ -96,7 +98,7 @@ template <bool STREAM> __device__ __forceinline__ bf16x8 load_weights(const bf16
 template <typename TO, int MT, int NT, bool PACKED, bool ACT, bool STREAM>
 __device__ __forceinline__ void grouped_tile(const bf16_t* __restrict__ x, const bf16_t* __restrict__ We,
                                              TO* __restrict__ out, int N, int K, const int* __restrict__ a_rows,
-                                             const float* __restrict__ act_scale, GatedAct act, int row0, int row_end,
+                                             const float* __restrict__ act_scale, GatedAct act, int relu2, int row0, int row_end,
                                              int n_base, bf16_t (*xs)[GM][GPAD]) {
   static_assert(!ACT || NT % 2 == 0, "the SwiGLU form pairs gate tiles with up tiles");
   constexpr int HT = ACT ? NT / 2 : NT;         // tiles of distinct output columns per wave
@@ -270,7 +272,12 @@ __device__ __forceinline__ void grouped_tile(const bf16_t* __restrict__ x, const
       for (int t = 0; t < NT; ++t) {
         const int n = n_base + t * 16 + 4 * g;
         if (n >= N) continue;
-        store(out + (size_t)row * N + n, acc[t][mb]);
+        f32x4 v = acc[t][mb];
+        if (relu2) {
+#pragma unroll
+          for (int i = 0; i < 4; ++i) v[i] = ungated_f32(UACT_RELU2, bf16_to_f32(f32_to_bf16(v[i])));
+        }
+        store(out + (size_t)row * N + n, v);
       }
     }
   }
@@ -279,7 +286,7 @@ __device__ __forceinline__ void grouped_tile(const bf16_t* __restrict__ x, const
 template <typename TO, int NT, bool PACKED, bool ACT>
 __global__ __launch_bounds__(GW* kWave, 2) void grouped_gemm_kernel(
     const bf16_t* __restrict__ x, const bf16_t* __restrict__ W, TO* __restrict__ out, int N, int K,
-    const int* __restrict__ a_rows, const float* __restrict__ act_scale, GatedAct act,
+    const int* __restrict__ a_rows, const float* __restrict__ act_scale, GatedAct act, int relu2,
     const int* __restrict__ group_offsets, const int* __restrict__ plan, int n_groups, int nb) {
   __shared__ __attribute__((aligned(16))) bf16_t xs[2][GM][GPAD];
   __shared__ int s_slot;
@@ -353,7 +360,7 @@ __global__ __launch_bounds__(GW* kWave, 2) void grouped_gemm_kernel(
       const int n_base = col_base + (threadIdx.x >> 6) * wave_cols;
       const bf16_t* We = W + (size_t)e * N * K;
       static_assert(GM == 128, "tile heights are compiled in steps of 32 rows up to 128");
-#define GT1(MTV, NTV, ST) grouped_tile<TO, MTV, NTV, PACKED, ACT, ST>(x, We, out, N, K, a_rows, act_scale, act, row0, row_end, n_base, xs)
+#define GT1(MTV, NTV, ST) grouped_tile<TO, MTV, NTV, PACKED, ACT, ST>(x, We, out, N, K, a_rows, act_scale, act, relu2, row0, row_end, n_base, xs)
       // (the hint only for weights stored tile by tile, the order the served model keeps them in)
 #define GT2(MTV, NTV)                                \
   do {                                               \

@@ -19,10 +19,10 @@ SHARPI_EXPORT int sharpi_gemm_grouped_swiglu(const void* x, int x_rows, const vo
   const dim3 grid = grouped_grid(n_rows, n_groups, nb, max_blocks), block(GW * kWave);
   if (packed)
     grouped_gemm_kernel<bf16_t, kMaxNT, true, true><<<grid, block, 0, stream>>>(
-        (const bf16_t*)x, (const bf16_t*)W, (bf16_t*)out, N, K, a_rows, act_scale, act, group_offsets, plan, n_groups, nb);
+        (const bf16_t*)x, (const bf16_t*)W, (bf16_t*)out, N, K, a_rows, act_scale, act, 0, group_offsets, plan, n_groups, nb);
   else
     grouped_gemm_kernel<bf16_t, kMaxNT, false, true><<<grid, block, 0, stream>>>(
-        (const bf16_t*)x, (const bf16_t*)W, (bf16_t*)out, N, K, a_rows, act_scale, act, group_offsets, plan, n_groups, nb);
+        (const bf16_t*)x, (const bf16_t*)W, (bf16_t*)out, N, K, a_rows, act_scale, act, 0, group_offsets, plan, n_groups, nb);
   SHARPI_CHECK_LAUNCH();
   return SHARPI_OK;
 }

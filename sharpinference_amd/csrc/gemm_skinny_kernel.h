@@ -34,6 +34,8 @@
 //    rounds both to bfloat16 (what a separate activation kernel would have read) and stores
 //    act(s g) * (s u), s the row's score and act the activation the caller names (SiLU, GELU):
 //    out is [M, N/2] and the gate|up rows never go to memory.
+//  * An ungated activation (uact, common.h) may be applied to the plain form's results, rounded to
+//    bfloat16 first (what a separate activation kernel would have read).
 //
 // Limits (the caller falls back to other kernels otherwise): K % 128 == 0, N % 4 == 0, M <= 64 (plain form).
 #pragma once
@@ -63,6 +65,7 @@ struct Picks {
   int n_pairs, k, n_experts;
   int gather;          // x rows are tokens (pair i reads row i / k); otherwise x is in the output's row order
   int shared;          // the tensor holds one more expert (index n_experts) that every token goes through
+                       // (ids of n_experts and above are identity experts: their pairs have no product and no row)
 };
 
 // Forms whose registers hold two K units at once (the loop then requests a unit ahead).
@@ -72,7 +75,7 @@ template <int R, int MB, int NW, typename TO, bool ACT, bool PACKED>
 __global__ __launch_bounds__(NW* kWave) void skinny_gemm_kernel(
     const bf16_t* __restrict__ x, const bf16_t* __restrict__ W, TO* __restrict__ out, int M, int N, int K,
     const int* __restrict__ a_rows, const int* __restrict__ group_offsets, const float* __restrict__ act_scale,
-    GatedAct act, Picks pk) {
+    GatedAct act, Picks pk, int uact) {
   static_assert(!ACT || R % 2 == 0, "the SwiGLU form pairs gate and up tiles");
   constexpr int RT = ACT ? R : kRedTiles;   // tiles that meet in LDS per round
   constexpr int TG = ACT ? R / 2 : R;       // tiles of distinct output columns per block
@@ -98,14 +101,15 @@ __global__ __launch_bounds__(NW* kWave) void skinny_gemm_kernel(
       const int n_groups = gridDim.y;
       const bool always_on = pk.shared && blockIdx.y == 0;
       const int ordinal_wanted = (int)blockIdx.y - pk.shared;
-      const int mine_e = lane < pk.n_pairs ? pk.ids[lane] : -1;
+      const int picked_e = lane < pk.n_pairs ? pk.ids[lane] : -1;
+      const int mine_e = picked_e < pk.n_experts ? picked_e : -1;
       int expert = -1;                            // the block's expert; -1: there are fewer distinct experts than groups
       if (always_on) {
         expert = pk.n_experts;
       } else if (n_groups - pk.shared == pk.n_experts) {
         expert = ordinal_wanted;                  // as many groups as experts: group y is expert y
       } else {
-        bool first = lane < pk.n_pairs;           // no earlier pair picked this lane's expert
+        bool first = mine_e >= 0;                 // no earlier pair picked this lane's expert
         for (int j = 0; j < pk.n_pairs; ++j) {
           const int ej = __shfl(mine_e, j, kWave);
           if (j < lane && ej == mine_e) first = false;
@@ -312,7 +316,13 @@ __global__ __launch_bounds__(NW* kWave) void skinny_gemm_kernel(
         // lane holds out[row = ... + r][n = n_base + t*16 + g*4 + 0..3]
         const int row = row_begin + (rb0 + mb) * 16 + r;
         const int n = n_base + t * 16 + g * 4;
-        if (row < row_end && n < N) store4<TO>(out + (size_t)out_row(row) * N + n, v);
+        if (row < row_end && n < N) {
+          if (uact) {
+#pragma unroll
+            for (int i = 0; i < 4; ++i) v[i] = ungated_f32(uact, bf16_to_f32(f32_to_bf16(v[i])));
+          }
+          store4<TO>(out + (size_t)out_row(row) * N + n, v);
+        }
       }
     }
   }
@@ -321,15 +331,15 @@ __global__ __launch_bounds__(NW* kWave) void skinny_gemm_kernel(
 template <int R, int MB, int NW, bool ACT, bool PACKED>
 static inline int launch_skinny(const void* x, const void* W, void* out, int out_dtype, int M, int N, int K,
                          const int* a_rows, const int* group_offsets, int groups, const float* act_scale,
-                         hipStream_t stream, Picks pk = Picks{}, GatedAct act = GatedAct{ACT_SILU, 0.f}) {
+                         hipStream_t stream, Picks pk = Picks{}, GatedAct act = GatedAct{ACT_SILU, 0.f}, int uact = UACT_NONE) {
   dim3 grid(ceil_div(ACT ? N / 2 : N, 16 * (ACT ? R / 2 : R)), groups > 0 ? groups : 1), block(NW * kWave);
   const int* go = groups > 0 ? group_offsets : nullptr;
   if (out_dtype == DT_F32)
     skinny_gemm_kernel<R, MB, NW, float, ACT, PACKED><<<grid, block, 0, stream>>>(
-        (const bf16_t*)x, (const bf16_t*)W, (float*)out, M, N, K, a_rows, go, act_scale, act, pk);
+        (const bf16_t*)x, (const bf16_t*)W, (float*)out, M, N, K, a_rows, go, act_scale, act, pk, uact);
   else
     skinny_gemm_kernel<R, MB, NW, bf16_t, ACT, PACKED><<<grid, block, 0, stream>>>(
-        (const bf16_t*)x, (const bf16_t*)W, (bf16_t*)out, M, N, K, a_rows, go, act_scale, act, pk);
+        (const bf16_t*)x, (const bf16_t*)W, (bf16_t*)out, M, N, K, a_rows, go, act_scale, act, pk, uact);
   SHARPI_CHECK_LAUNCH();
   return SHARPI_OK;
 }

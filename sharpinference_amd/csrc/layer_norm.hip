@@ -1,10 +1,13 @@
-// Layers whose branches end in a layer norm and begin with a short convolution over the residual sum; the
-// embedding with a second table indexed by a pair of tokens.
+// Layers whose branches end in a layer norm and begin with a short convolution over the residual sum; layers with a
+// layer norm of the whole sum behind each branch; the embedding with a second table indexed by a pair of tokens, and
+// the embedding with a norm.
 //
 // layer_norm:      x = h[r] (+ LN(delta[r]) w + b); the new x back into h; and, by what is asked for, x itself, LN of
 //                  x (a model's last norm), or x + conv(x) (what the next branch reads; steps of single
 //                  tokens) in the activations' storage type.  delta is a tensor or an expert sum still to be formed.
 // residual_conv:   out[t] = h[t] + sum_j w[:, j] h[t - taps + 1 + j], for steps that bring longer entries.
+// sum_norm:        x = LN(alpha h + delta) w + b, the new x back into h, and x in the activations' storage type.
+// embed_norm:      out[t] = LN(table[id] * scale) w + b, likewise with a copy in the activations' storage type.
 // embed_bigram:    out[t] = table[id] * scale + pairs[(previous id * a + id * b) mod buckets].
 //
 // A convolution's last inputs lie in a ring [slots, taps, channels] of floats, position p at p mod taps; what lies
@@ -19,6 +22,9 @@ struct LnDelta {
   const float* w;                // [T, k] or null
   const void* shared;            // [T, hidden] or null (expert sums only)
   int k;
+  const int* ids = nullptr;      // [T, k]: picks of n_experts and above are identity experts (sum_norm)
+  int n_experts = 0;
+  const void* ident = nullptr;   // [T, hidden]: their outputs (null: the row of h itself, in float)
 };
 
 template <typename TD, int V>
@@ -330,6 +336,196 @@ SHARPI_EXPORT int sharpi_layer_norm(float* h, const void* delta, int d_dtype, co
     else LN(bf16_t, bf16_t);
   }
 #undef LN
+  SHARPI_CHECK_LAUNCH();
+  return SHARPI_OK;
+}
+
+// ---------------------------------------------------------------------------
+// The norm of the sum: x = LN(alpha h[t] + delta[t]) w + b back into h, and, with out, x in the activations' storage
+// type.  delta: a tensor or an expert sum still to be formed, whose identity picks add weight * (the layer's input row):
+// a row of `ident`, or h itself in float (then they only change the coefficient of h).
+// ---------------------------------------------------------------------------
+template <typename TD, int V>
+__device__ __forceinline__ void sum_of_row(const LnDelta& d, size_t r, int hidden, int c, float alpha, const float* x, float* v) {
+  if (!d.ids) {
+    ln_delta<TD, V>(d, r, hidden, c, v);
+  } else {
+#pragma unroll
+    for (int i = 0; i < V; ++i) v[i] = 0.f;
+    for (int q0 = 0; q0 < d.k; q0 += 4) {    // (four rows are requested before the first is added)
+      float y[4][V], wq[4];
+      bool own[4];
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const size_t q = r * d.k + min(q0 + j, d.k - 1);
+        own[j] = d.ids[q] >= d.n_experts;
+        const TD* row = own[j] ? (d.ident ? (const TD*)d.ident + r * hidden : nullptr) : (const TD*)d.y + (size_t)d.pos[q] * hidden;
+        if (row) ln_load<TD, V>(row + c, y[j]);
+        else {
+#pragma unroll
+          for (int i = 0; i < V; ++i) y[j][i] = x[i];
+        }
+        wq[j] = d.w ? d.w[q] : 1.0f;
+      }
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        if (q0 + j < d.k) {
+#pragma unroll
+          for (int i = 0; i < V; ++i) v[i] = fmaf(wq[j], y[j][i], v[i]);
+        }
+    }
+    if (d.shared) {
+      float y[V];
+      ln_load<TD, V>((const TD*)d.shared + r * hidden + c, y);
+#pragma unroll
+      for (int i = 0; i < V; ++i) v[i] += y[i];
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < V; ++i) v[i] = fmaf(alpha, x[i], v[i]);
+}
+
+// A thread has one run of eight elements (hidden a multiple of 8 up to 8,192): everything in registers, all loads ahead of the
+// reductions.
+template <typename TD, typename TO>
+__global__ __launch_bounds__(1024) void sum_norm_run_kernel(float* __restrict__ h, LnDelta delta, float alpha,
+                                                            const float* __restrict__ w, const float* __restrict__ b, float eps,
+                                                            TO* __restrict__ out, int hidden) {
+  __shared__ float red[16];
+  const size_t r = blockIdx.x;
+  const int c = threadIdx.x * 8;
+  const bool in = c < hidden;
+  float x[8], y[8], wv[8], bv[8];
+  float s = 0.f;
+  if (in) {
+    load8(h + r * hidden + c, x);
+    load8(w + c, wv);
+    load8(b + c, bv);
+    sum_of_row<TD, 8>(delta, r, hidden, c, alpha, x, y);
+#pragma unroll
+    for (int k = 0; k < 8; ++k) s += y[k];
+  }
+  const float mean = block_sum(s, red) / (float)hidden;
+  s = 0.f;
+  if (in) {
+#pragma unroll
+    for (int k = 0; k < 8; ++k) s = fmaf(y[k] - mean, y[k] - mean, s);
+  }
+  const float inv = 1.0f / sqrtf(block_sum(s, red) / (float)hidden + eps);
+  if (in) {
+#pragma unroll
+    for (int k = 0; k < 8; ++k) x[k] = fmaf((y[k] - mean) * inv, wv[k], bv[k]);
+    store8(h + r * hidden + c, x);
+    if (out) store8(out + r * hidden + c, x);
+  }
+}
+
+template <typename TD, typename TO>
+__global__ __launch_bounds__(256) void sum_norm_kernel(float* __restrict__ h, LnDelta delta, float alpha, const float* __restrict__ w,
+                                                       const float* __restrict__ b, float eps, TO* __restrict__ out, int hidden) {
+  extern __shared__ __attribute__((aligned(16))) float row[];
+  __shared__ float red[16];
+  const size_t r = blockIdx.x;
+  float* hr = h + r * hidden;
+  float s = 0.f;
+  for (int c = threadIdx.x; c < hidden; c += blockDim.x) {     // (a thread reads what it wrote)
+    float y;
+    sum_of_row<TD, 1>(delta, r, hidden, c, alpha, hr + c, &y);
+    row[c] = y;
+    s += y;
+  }
+  const float mean = block_sum(s, red) / (float)hidden;
+  s = 0.f;
+  for (int c = threadIdx.x; c < hidden; c += blockDim.x) s = fmaf(row[c] - mean, row[c] - mean, s);
+  const float inv = 1.0f / sqrtf(block_sum(s, red) / (float)hidden + eps);
+  for (int c = threadIdx.x; c < hidden; c += blockDim.x) {
+    const float x = fmaf((row[c] - mean) * inv, w[c], b[c]);
+    hr[c] = x;
+    if (out) out[r * hidden + c] = from_f32<TO>(x);
+  }
+}
+
+// h float [T, hidden]; delta [T, hidden] of d_dtype, or (pos) the experts' rows with pos int32 [T, k], sum_w float [T, k] or
+// null, shared [T, hidden] or null, and (ids int32 [T, k]) identity picks from n_experts on, whose output is row t of
+// ident [T, hidden] of d_dtype or, with ident null, of h.  out [T, hidden] of o_dtype, or null.
+SHARPI_EXPORT int sharpi_sum_norm(float* h, const void* delta, int d_dtype, const int* pos, const float* sum_w, int k, const void* shared,
+                                  const int* ids, int n_experts, const void* ident, float alpha, const float* w, const float* b,
+                                  float eps, int n_rows, int hidden, void* out, int o_dtype, hipStream_t stream) {
+  if (n_rows <= 0) return SHARPI_OK;
+  if (hidden <= 0 || (size_t)hidden * sizeof(float) > 60 * 1024 || !delta || !w || !b || !(eps > 0.f)) return SHARPI_ERR_ARG;
+  if ((pos && k <= 0) || (ids && !pos)) return SHARPI_ERR_ARG;
+  if ((d_dtype != DT_F32 && d_dtype != DT_BF16) || (out && o_dtype != DT_F32 && o_dtype != DT_BF16)) return SHARPI_ERR_ARG;
+  auto aligned = [](const void* p) { return ((uintptr_t)p & 31) == 0; };
+  const bool wide = hidden % 8 == 0 && hidden <= 8192 && aligned(h) && aligned(delta) && aligned(shared) && aligned(ident) && aligned(w) &&
+                    aligned(b) && aligned(out);
+  LnDelta d{delta, pos, sum_w, shared, k, ids, n_experts, ident};
+  const int runs = wide ? hidden / 8 : hidden;
+  int threads = ceil_div(runs, kWave) * kWave;
+  if (threads > (wide ? 1024 : 256)) threads = wide ? 1024 : 256;
+  const size_t lds = (size_t)hidden * sizeof(float);
+#define SN(TD, TO)                                                                                                \
+  do {                                                                                                            \
+    if (wide) sum_norm_run_kernel<TD, TO><<<n_rows, threads, 0, stream>>>(h, d, alpha, w, b, eps, (TO*)out, hidden); \
+    else sum_norm_kernel<TD, TO><<<n_rows, threads, lds, stream>>>(h, d, alpha, w, b, eps, (TO*)out, hidden);      \
+  } while (0)
+  const bool of = !out || o_dtype == DT_F32;
+  if (d_dtype == DT_F32) {
+    if (of) SN(float, float);
+    else SN(float, bf16_t);
+  } else {
+    if (of) SN(bf16_t, float);
+    else SN(bf16_t, bf16_t);
+  }
+#undef SN
+  SHARPI_CHECK_LAUNCH();
+  return SHARPI_OK;
+}
+
+// ---------------------------------------------------------------------------
+// The embedding with a norm: out[t] = LN(table[ids[t]] * scale) w + b in float, and a copy in the activations' storage
+// type (copy null: none).
+// ---------------------------------------------------------------------------
+template <typename T, typename TO>
+__global__ __launch_bounds__(256) void embed_norm_kernel(const int* __restrict__ ids, const T* __restrict__ table, float scale,
+                                                         const float* __restrict__ w, const float* __restrict__ b, float eps,
+                                                         float* __restrict__ out, TO* __restrict__ copy, int hidden) {
+  extern __shared__ __attribute__((aligned(16))) float row[];
+  __shared__ float red[16];
+  const size_t t = blockIdx.x;
+  const T* src = table + (size_t)ids[t] * hidden;
+  float s = 0.f;
+  for (int c = threadIdx.x; c < hidden; c += blockDim.x) {     // (a thread reads what it wrote)
+    const float v = to_f32<T>(src[c]) * scale;
+    row[c] = v;
+    s += v;
+  }
+  const float mean = block_sum(s, red) / (float)hidden;
+  s = 0.f;
+  for (int c = threadIdx.x; c < hidden; c += blockDim.x) s = fmaf(row[c] - mean, row[c] - mean, s);
+  const float inv = 1.0f / sqrtf(block_sum(s, red) / (float)hidden + eps);
+  for (int c = threadIdx.x; c < hidden; c += blockDim.x) {
+    const float x = fmaf((row[c] - mean) * inv, w[c], b[c]);
+    out[t * hidden + c] = x;
+    if (copy) copy[t * hidden + c] = from_f32<TO>(x);
+  }
+}
+
+SHARPI_EXPORT int sharpi_embed_norm(const int* ids, const void* table, int t_dtype, float scale, const float* w, const float* b,
+                                    float eps, float* out, void* copy, int c_dtype, int n_tokens, int hidden, hipStream_t stream) {
+  if (n_tokens <= 0) return SHARPI_OK;
+  if (hidden <= 0 || (size_t)hidden * sizeof(float) > 60 * 1024 || !w || !b || !(eps > 0.f)) return SHARPI_ERR_ARG;
+  if ((t_dtype != DT_F32 && t_dtype != DT_BF16) || (copy && c_dtype != DT_F32 && c_dtype != DT_BF16)) return SHARPI_ERR_ARG;
+  const size_t lds = (size_t)hidden * sizeof(float);
+#define EN(T, TO) embed_norm_kernel<T, TO><<<n_tokens, 256, lds, stream>>>(ids, (const T*)table, scale, w, b, eps, out, (TO*)copy, hidden)
+  const bool cf = !copy || c_dtype == DT_F32;
+  if (t_dtype == DT_F32) {
+    if (cf) EN(float, float);
+    else EN(float, bf16_t);
+  } else {
+    if (cf) EN(bf16_t, float);
+    else EN(bf16_t, bf16_t);
+  }
+#undef EN
   SHARPI_CHECK_LAUNCH();
   return SHARPI_OK;
 }

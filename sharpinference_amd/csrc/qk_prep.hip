@@ -10,7 +10,8 @@
 // several score maps side by side (`maps`): norm weights and cache rows stay per head, the rotation
 // works on each map's own leading elements, and the queries leave expanded, one row of the head's
 // width per (head, map) with that map's elements in their place and zeros elsewhere, so that an
-// attention kernel over keys of the head's width computes each map's scores on its own.
+// attention kernel over keys of the head's width computes each map's scores on its own; and values mixed with
+// those of another layer, (1 - c) v + c v_other, in float on their way into the cache.
 //
 // One block per token, or, in steps of few tokens, one per (token, kv head): the block then takes
 // that kv head's key and value and the query heads that read it, so that a decode step still fills
@@ -56,6 +57,9 @@ struct PrepArgs {
   int temp_on;             // query temperature
   float temp_floor, temp_scale;
   int maps;                // score maps a head (1: the plain layout of q_out; > 1: q_out [T, nh * maps * hd], expanded)
+  const void* v_other;     // another layer's projections of the same tokens (null: values as they are)
+  int v_other_stride, v_other_off;
+  float v_mix;             // c
   int by8;                 // every offset, stride and width a multiple of 8 (and split halves): eight channels a thread
 };
 
@@ -152,7 +156,9 @@ __global__ __launch_bounds__(kPrepThreads) void qk_prep_kernel(PrepArgs a) {
     const float* vsrc = own_v ? row + qn + kn : row + qn;
     for (int i = kh0 * a.vd + threadIdx.x; i < kh1 * a.vd; i += kPrepThreads) {
       const int g = i / a.vd, d = i % a.vd;
-      vc[(((size_t)page * a.nkv + g) * a.vd + d) * a.page_size + off] = from_f32<T>(vsrc[i]);
+      float v = vsrc[i];
+      if (a.v_other) v = (1.0f - a.v_mix) * v + a.v_mix * to_f32<T>(((const T*)a.v_other)[(size_t)t * a.v_other_stride + a.v_other_off + i]);
+      vc[(((size_t)page * a.nkv + g) * a.vd + d) * a.page_size + off] = from_f32<T>(v);
     }
   }
 
@@ -340,7 +346,9 @@ __global__ void conv_tail_kernel(const T* __restrict__ proj, int stride, int q_o
 // page_size, hd], V [pages, nkv, vd, page_size]; slot_mapping null or -1: nothing is stored.
 // bias float [q + k + v channels] or null (only without a convolution); temp_on: q times
 // 1 + temp_scale ln(floor((pos + 1) / temp_floor) + 1); maps > 1: hd is the width of a head's maps
-// together, rotary_dim <= hd / maps, and q_out is [T, nh * maps * hd].
+// together, rotary_dim <= hd / maps, and q_out is [T, nh * maps * hd].  v_other (of `dtype`, or null): rows of
+// v_other_stride elements whose columns v_other_off .. hold another layer's values: what is stored is
+// (1 - v_mix) v + v_mix v_other.
 SHARPI_EXPORT int sharpi_qk_prep(const void* proj, int dtype, int stride, int q_off, int k_off, int v_off, int n_tokens,
                                  int n_entries, int nh, int nkv, int hd, int vd, const float* conv_w, int taps, float* tail,
                                  const int* state_slots, const int* entry_of_token, const int* cu_tokens,
@@ -348,8 +356,10 @@ SHARPI_EXPORT int sharpi_qk_prep(const void* proj, int dtype, int stride, int q_
                                  float eps, const float* inv_freq, int rotary_dim, int half_split, float magnitude,
                                  void* q_out, void* k_cache, void* v_cache, const int* slot_mapping, int page_size,
                                  int update_tail, const float* bias, int temp_on, float temp_floor, float temp_scale,
-                                 int maps, hipStream_t stream) {
+                                 int maps, const void* v_other, int v_other_stride, int v_other_off, float v_mix,
+                                 hipStream_t stream) {
   if (n_tokens <= 0) return SHARPI_OK;
+  if (v_other && (v_other_off < 0 || v_other_off + nkv * vd > v_other_stride)) return SHARPI_ERR_ARG;
   if (maps < 1 || hd % (2 * maps) || rotary_dim > hd / maps) return SHARPI_ERR_ARG;
   if ((bias && taps > 0) || (temp_on && !(temp_floor > 0.f))) return SHARPI_ERR_ARG;
   if (nh <= 0 || nkv <= 0 || hd <= 0 || hd % 2 || vd <= 0 || nh + nkv > kPrepMaxHeads) return SHARPI_ERR_ARG;
@@ -372,7 +382,7 @@ SHARPI_EXPORT int sharpi_qk_prep(const void* proj, int dtype, int stride, int q_
   PrepArgs a{proj, stride, q_off, k_off, v_off, nh, nkv, hd, vd, conv_w, taps, tail, state_slots, entry_of_token,
              cu_tokens, positions, norm_mode, q_norm_w, k_norm_w, eps, rotary_dim > 0 ? inv_freq : nullptr, rotary_dim,
              half_split, magnitude, q_out, k_cache, v_cache, slot_mapping, page_size, parts, bias, temp_on, temp_floor,
-             temp_scale, maps, by8};
+             temp_scale, maps, v_other, v_other_stride, v_other_off, v_mix, by8};
   dim3 pgrid(n_tokens, parts);
   if (dtype == DT_F32) qk_prep_kernel<float><<<pgrid, kPrepThreads, lds, stream>>>(a);
   else if (dtype == DT_BF16) qk_prep_kernel<bf16_t><<<pgrid, kPrepThreads, lds, stream>>>(a);

@@ -13,6 +13,8 @@
 // walks (grouped_plan.h: units of sibling row tiles dealt to the XCDs).  With shared_group the list gets one
 // more group after the experts: every token once, weight 1 (an always-on expert that shares the
 // experts' weight tensor); offsets then has n_experts + 2 entries and the row arrays n_tokens more.
+// Picks of n_experts and above (identity experts: the token's own row is their output) get no row: the list
+// then ends at offsets[n_experts], before its room does.  The two do not come together.
 #include "common.h"
 #include "grouped_plan.h"
 
@@ -23,13 +25,13 @@ constexpr int kMaxExperts = 1024;
 // `choice` (or null) is scratch of n_experts + n_groups floats and turns the choice apart from the
 // weights: experts are then picked by g[e] + corr[e] (corr may be null), among the experts of the
 // `keep` best of n_groups equal groups of neighbours only (a group's rank: the sum of its
-// kGroupTop largest choice scores; the lowest index wins a tie; the others' choice scores count as
+// group_top largest choice scores; the lowest index wins a tie; the others' choice scores count as
 // minus infinity), and a pick's weight stays its gate value g[e].
-constexpr int kGroupTop = 2;
+constexpr int kMaxGroupTop = 2;
 
 __device__ void gate_and_pick(float* g, int n_experts, int k, int gate, int renorm, int* ids, float* w,
                               float* gate_out, float* choice = nullptr, const float* corr = nullptr,
-                              int n_groups = 1, int keep = 1) {
+                              int n_groups = 1, int keep = 1, int group_top = kMaxGroupTop) {
   if (gate == 2) {
     // the logits themselves rank the experts; the picks' weights are the softmax over the picked logits alone
   } else if (gate == 0) {
@@ -54,12 +56,12 @@ __device__ void gate_and_pick(float* g, int n_experts, int k, int gate, int reno
       const int per = n_experts / n_groups;
       float* rank = choice + n_experts;
       for (int q = 0; q < n_groups; ++q) {
-        // the sum of the group's kGroupTop largest choice scores (of all of them in a smaller group)
-        float top[kGroupTop];
-        for (int i = 0; i < kGroupTop; ++i) top[i] = -INFINITY;
+        // the sum of the group's group_top largest choice scores (of all of them in a smaller group)
+        float top[kMaxGroupTop];
+        for (int i = 0; i < kMaxGroupTop; ++i) top[i] = -INFINITY;
         for (int e = q * per; e < (q + 1) * per; ++e) {
           float v = choice[e];
-          for (int i = 0; i < kGroupTop; ++i)
+          for (int i = 0; i < kMaxGroupTop; ++i)
             if (v > top[i]) {
               const float o = top[i];
               top[i] = v;
@@ -67,7 +69,7 @@ __device__ void gate_and_pick(float* g, int n_experts, int k, int gate, int reno
             }
         }
         float r = 0.f;
-        for (int i = 0; i < kGroupTop && i < per; ++i) r += top[i];
+        for (int i = 0; i < group_top && i < per; ++i) r += top[i];
         rank[q] = r;
       }
       for (int j = 0; j < keep; ++j) {       // the kept groups are marked with +infinity
@@ -153,7 +155,7 @@ __device__ __forceinline__ int wave_argmax(const float* v, int n, int lane, uint
 }
 
 __device__ void gate_and_pick_wave(float* g, int n_experts, int k, int gate, int renorm, int* ids, float* w, float* gate_out,
-                                   float* choice, const float* corr, int n_groups, int keep, float w_scale, int lane) {
+                                   float* choice, const float* corr, int n_groups, int keep, float w_scale, int lane, int group_top = kMaxGroupTop) {
   if (gate == 0) {
     for (int e = lane; e < n_experts; e += kWave) g[e] = 1.0f / (1.0f + expf(-g[e]));
   } else if (gate == 1) {
@@ -177,11 +179,11 @@ __device__ void gate_and_pick_wave(float* g, int n_experts, int k, int gate, int
       float* rank = choice + n_experts;
       wave_lds_sync();
       for (int q = lane; q < n_groups; q += kWave) {
-        float top[kGroupTop];
-        for (int i = 0; i < kGroupTop; ++i) top[i] = -INFINITY;
+        float top[kMaxGroupTop];
+        for (int i = 0; i < kMaxGroupTop; ++i) top[i] = -INFINITY;
         for (int e = q * per; e < (q + 1) * per; ++e) {
           float v = choice[e];
-          for (int i = 0; i < kGroupTop; ++i)
+          for (int i = 0; i < kMaxGroupTop; ++i)
             if (v > top[i]) {
               const float o = top[i];
               top[i] = v;
@@ -189,7 +191,7 @@ __device__ void gate_and_pick_wave(float* g, int n_experts, int k, int gate, int
             }
         }
         float r = 0.f;
-        for (int i = 0; i < kGroupTop && i < per; ++i) r += top[i];
+        for (int i = 0; i < group_top && i < per; ++i) r += top[i];
         rank[q] = r;
       }
       wave_lds_sync();
@@ -296,7 +298,7 @@ __global__ __launch_bounds__(1024) void router_topk_kernel(const T* __restrict__
                                                            float* __restrict__ gate_out, int n_tokens, int hidden,
                                                            int n_experts, int k, int gate, int renorm,
                                                            const float* __restrict__ corr, int n_groups, int keep,
-                                                           int split_choice, const float* __restrict__ bias, float w_scale) {
+                                                           int split_choice, const float* __restrict__ bias, float w_scale, int group_top) {
   // TT tokens per block: a router row is fetched once for all of them.
   __shared__ float g[TT][kMaxExperts];
   extern __shared__ float choice_s[];        // [TT][n_experts + n_groups] when the choice has scores of its own
@@ -321,13 +323,13 @@ __global__ __launch_bounds__(1024) void router_topk_kernel(const T* __restrict__
       const int t = t0 + w;
       gate_and_pick_wave(g[w], n_experts, k, gate, renorm, topk_ids + (size_t)t * k, topk_w + (size_t)t * k,
                          gate_out ? gate_out + (size_t)t * n_experts : nullptr,
-                         split_choice ? choice_s + (size_t)w * (n_experts + n_groups) : nullptr, corr, n_groups, keep, w_scale, lane);
+                         split_choice ? choice_s + (size_t)w * (n_experts + n_groups) : nullptr, corr, n_groups, keep, w_scale, lane, group_top);
     }
   } else if (threadIdx.x < TT && t0 + threadIdx.x < n_tokens) {
     const int t = t0 + threadIdx.x;
     gate_and_pick(g[threadIdx.x], n_experts, k, gate, renorm, topk_ids + (size_t)t * k, topk_w + (size_t)t * k,
                   gate_out ? gate_out + (size_t)t * n_experts : nullptr,
-                  split_choice ? choice_s + (size_t)threadIdx.x * (n_experts + n_groups) : nullptr, corr, n_groups, keep);
+                  split_choice ? choice_s + (size_t)threadIdx.x * (n_experts + n_groups) : nullptr, corr, n_groups, keep, group_top);
     if (w_scale != 1.0f)
       for (int j = 0; j < k; ++j) topk_w[(size_t)t * k + j] *= w_scale;
   }
@@ -425,18 +427,20 @@ SHARPI_EXPORT int sharpi_add_rmsnorm_router(float* h, const void* delta, const v
 }
 
 // corr (float [n_experts] or null): added to the gate values for the choice only.  n_groups, keep:
-// picks come from the `keep` best of n_groups equal groups of neighbouring experts (1, 1: no groups).
+// picks come from the `keep` best of n_groups equal groups of neighbouring experts (1, 1: no groups), a group
+// ranked by the sum of its group_top (1 or 2) largest choice scores.
 // bias (float [n_experts] or null): added to the logits.  gate 0: sigmoid; 1: softmax over all experts;
 // 2: the largest logits are picked and their weights are the softmax over the picked logits alone.
 // w_scale multiplies the picks' weights at the end.
 SHARPI_EXPORT int sharpi_router_topk(const void* x, int x_dtype, const void* wr, int w_dtype, int* topk_ids,
                                      float* topk_w, float* gate_out, int n_tokens, int hidden, int n_experts,
                                      int k, int gate, int renorm, const float* corr, int n_groups, int keep,
-                                     const float* bias, float w_scale, hipStream_t stream) {
+                                     const float* bias, float w_scale, int group_top, hipStream_t stream) {
   if (n_tokens <= 0) return SHARPI_OK;
   if (hidden <= 0 || n_experts <= 0 || n_experts > kMaxExperts || k <= 0 || k > n_experts) return SHARPI_ERR_ARG;
   if (gate < 0 || gate > 2) return SHARPI_ERR_ARG;
   if (n_groups < 1 || keep < 1 || keep > n_groups || n_experts % n_groups != 0 || k > keep * (n_experts / n_groups)) return SHARPI_ERR_ARG;
+  if (group_top < 1 || group_top > kMaxGroupTop) return SHARPI_ERR_ARG;
   const int split_choice = corr != nullptr || keep < n_groups;
   // one wave per expert at a time: enough waves for the experts, at most 16; with many tokens four
   // share a block (and each fetch of a router row)
@@ -448,11 +452,11 @@ SHARPI_EXPORT int sharpi_router_topk(const void* x, int x_dtype, const void* wr,
     if (tt == 4)                                                                                                 \
       router_topk_kernel<TX, TWT, 4><<<grid, block, lds, stream>>>((const TX*)x, (const TWT*)wr, topk_ids, topk_w, \
                                                                  gate_out, n_tokens, hidden, n_experts, k, gate, \
-                                                                 renorm, corr, n_groups, keep, split_choice, bias, w_scale); \
+                                                                 renorm, corr, n_groups, keep, split_choice, bias, w_scale, group_top); \
     else                                                                                                         \
       router_topk_kernel<TX, TWT, 1><<<grid, block, lds, stream>>>((const TX*)x, (const TWT*)wr, topk_ids, topk_w, \
                                                                  gate_out, n_tokens, hidden, n_experts, k, gate, \
-                                                                 renorm, corr, n_groups, keep, split_choice, bias, w_scale); \
+                                                                 renorm, corr, n_groups, keep, split_choice, bias, w_scale, group_top); \
   } while (0)
   if (x_dtype == DT_F32 && w_dtype == DT_F32) ROUTER_LAUNCH(float, float);
   else if (x_dtype == DT_BF16 && w_dtype == DT_BF16) ROUTER_LAUNCH(bf16_t, bf16_t);
@@ -473,7 +477,8 @@ __device__ void permute_block(const int* __restrict__ topk_ids, const float* __r
                               int* plan_scratch) {
   for (int e = threadIdx.x; e < n_experts; e += blockDim.x) count[e] = 0;
   __syncthreads();
-  for (int i = threadIdx.x; i < n_pairs; i += blockDim.x) atomicAdd(&count[topk_ids[i]], 1);
+  for (int i = threadIdx.x; i < n_pairs; i += blockDim.x)
+    if (topk_ids[i] < n_experts) atomicAdd(&count[topk_ids[i]], 1);
   __syncthreads();
   if (threadIdx.x == 0) {
     int run = 0;
@@ -551,6 +556,10 @@ __device__ void permute_block(const int* __restrict__ topk_ids, const float* __r
   __syncthreads();
   for (int i = threadIdx.x; i < n_pairs; i += blockDim.x) {
     const int e = topk_ids[i];
+    if (e >= n_experts) {                // an identity expert: no product, no row (whoever sums the pairs asks the id)
+      inv_pos[i] = 0;
+      continue;
+    }
     const int r = atomicAdd(&cursor[e], 1);
     sorted_token[r] = i / k;
     sorted_w[r] = topk_w[i];
@@ -575,7 +584,8 @@ __global__ __launch_bounds__(1024) void moe_permute_kernel(const int* __restrict
 // plan: plan_ints(n_experts + shared_group) ints (grouped_plan.h) for the grouped product of many rows, or null.
 SHARPI_EXPORT int sharpi_moe_permute(const int* topk_ids, const float* topk_w, int* offsets, int* sorted_token,
                                      float* sorted_w, int* inv_pos, int* plan, int plan_len, int n_tokens, int k,
-                                     int n_experts, int shared_group, hipStream_t stream) {
+                                     int n_experts, int shared_group, int identity, hipStream_t stream) {
+  if (shared_group && identity) return SHARPI_ERR_ARG;
   if (n_experts <= 0 || n_experts > kMaxExperts || k <= 0) return SHARPI_ERR_ARG;
   if (n_tokens < 0) return SHARPI_ERR_ARG;
   if (plan && plan_len < plan_ints(n_experts + (shared_group ? 1 : 0))) return SHARPI_ERR_ARG;

@@ -116,12 +116,13 @@ class ExpertSum:
     """A branch output that is still a sum to be formed: row t = sum_j w[t, j] * y[inv_pos[t*k + j]]
     (+ shared[t]); ``weights`` None means ones (scores already applied to the experts' inputs).
     ``add_rmsnorm`` forms it on the fly; ``tensor()`` forms it with a kernel of its own.  Either
-    way the sum is rounded once to y's storage type."""
+    way the sum is rounded once to y's storage type.  ``identity`` = (ids int32 [T, k], n_experts, x [T, H] of y's
+    dtype): picks of n_experts and above are identity experts, which have no row in y and return row t of x."""
 
-    __slots__ = ("y", "inv_pos", "shared", "n_tokens", "k", "weights")
+    __slots__ = ("y", "inv_pos", "shared", "n_tokens", "k", "weights", "identity")
 
     def __init__(self, y: torch.Tensor, inv_pos: torch.Tensor, shared: Optional[torch.Tensor], n_tokens: int, k: int,
-                 weights: Optional[torch.Tensor] = None):
+                 weights: Optional[torch.Tensor] = None, identity=None):
         _need(y.dim() == 2 and inv_pos.numel() == n_tokens * k, "ExpertSum: y [rows, H], inv_pos [T*k]")
         if shared is not None:
             _need(shared.shape == (n_tokens, y.shape[1]) and shared.dtype == y.dtype and shared.is_contiguous(),
@@ -129,7 +130,13 @@ class ExpertSum:
         if weights is not None:
             _need(weights.numel() == n_tokens * k and weights.dtype == torch.float32 and weights.is_contiguous(),
                   "ExpertSum: weights must be contiguous float32 [T, k]")
+        if identity is not None:
+            ids, _, x = identity
+            _need(ids.dtype == torch.int32 and ids.numel() == n_tokens * k and ids.is_contiguous() and x.is_contiguous()
+                  and tuple(x.shape) == (n_tokens, y.shape[1]) and x.dtype == y.dtype,
+                  "ExpertSum: identity ids must be int32 [T, k], their outputs [T, H] of y's dtype")
         self.y, self.inv_pos, self.shared, self.n_tokens, self.k, self.weights = y, inv_pos, shared, n_tokens, k, weights
+        self.identity = identity
 
     @property
     def shape(self):
@@ -141,7 +148,12 @@ class ExpertSum:
 
     def tensor(self) -> torch.Tensor:
         return moe_combine(self.y[: self.n_tokens * self.k], self.inv_pos, self.shared, self.n_tokens, self.k,
-                           self.weights)
+                           self.weights, self.identity)
+
+
+def _foldable(delta):
+    """`delta` as the kernels that form expert sums on the fly take it: a sum with identity experts is formed first."""
+    return delta.tensor() if isinstance(delta, ExpertSum) and delta.identity is not None else delta
 
 
 def add_rmsnorm(h: torch.Tensor, delta, weight: Optional[torch.Tensor], eps: float,
@@ -149,6 +161,7 @@ def add_rmsnorm(h: torch.Tensor, delta, weight: Optional[torch.Tensor], eps: flo
                 out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """(h + delta) -> RMSNorm -> out; the sum goes back into h unless rows are gathered.
     delta: a tensor, an ExpertSum, or None."""
+    delta = _foldable(delta)
     lazy = delta if isinstance(delta, ExpertSum) else None
     if lazy is not None and h.shape[1] % 8 != 0:
         delta, lazy = lazy.tensor(), None          # the kernel folds a sum in only at widths that are multiples of 8
@@ -198,9 +211,11 @@ def silu_mul(gate_up: torch.Tensor, scale: Optional[torch.Tensor] = None) -> tor
 
 
 def moe_combine(y: torch.Tensor, inv_pos: torch.Tensor, shared: Optional[torch.Tensor], n_tokens: int,
-                k: int, weights: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """out[t] = sum_j w[t, j] * y[inv_pos[t*k+j]] (+ shared[t]); weights None: ones."""
-    _dev(y, inv_pos, shared, weights)
+                k: int, weights: Optional[torch.Tensor] = None, identity=None) -> torch.Tensor:
+    """out[t] = sum_j w[t, j] * y[inv_pos[t*k+j]] (+ shared[t]); weights None: ones.  ``identity`` = (ids, n_experts, x):
+    see :class:`ExpertSum`."""
+    ids, n_experts, ident = identity if identity is not None else (None, 0, None)
+    _dev(y, inv_pos, shared, weights, ids, ident)
     _i32(inv_pos, "inv_pos")
     _need(y.dim() == 2 and y.shape[0] == n_tokens * k and inv_pos.numel() == n_tokens * k,
           "moe_combine: y must be [T*k, H] and inv_pos [T*k]")
@@ -211,7 +226,7 @@ def moe_combine(y: torch.Tensor, inv_pos: torch.Tensor, shared: Optional[torch.T
         _need(weights.numel() == n_tokens * k and weights.dtype == torch.float32, "moe_combine: weights must be float32 [T, k]")
     out = torch.empty(n_tokens, H, dtype=y.dtype, device=y.device)
     _run("sharpi_moe_combine", _ptr(y), _ptr(inv_pos), _ptr(shared), _ptr(weights), _ptr(out), _code(y.dtype), n_tokens,
-         H, k, _stream())
+         H, k, _ptr(ids), int(n_experts), _ptr(ident), _stream())
     return out
 
 
@@ -315,11 +330,12 @@ def _sink_args(sink, nh: int):
 def attention_generic(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_table: torch.Tensor,
                       entry_of_token: torch.Tensor, positions: torch.Tensor, window_kind: int, window: int,
                       scale: float, nh: int, nkv: int, hd: int, vd: Optional[int] = None, softcap: float = 0.0,
-                      sink: bool = False) -> torch.Tensor:
+                      sink: bool = False, keep: int = 0, gate=None) -> torch.Tensor:
     """Attention of every token of the batch over its request's pages; float arithmetic.  Values
     (and so the output, [T, nh*vd]) may have another width than keys.  softcap > 0: scores become
     softcap * tanh(score / softcap); sink: one more term exp(0), without a value, in the softmax's
-    denominator."""
+    denominator.  keep: the sequence's first `keep` keys are seen beside the window's.  gate = (rows [T, N] of q's
+    dtype, column): head h's output is multiplied by sigmoid(rows[t, column + h])."""
     _dev(q, k_cache, v_cache, block_table, entry_of_token, positions)
     _i32(block_table, "block_table")
     _i32(entry_of_token, "entry_of_token")
@@ -334,8 +350,20 @@ def attention_generic(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Ten
     out = torch.empty(T, nh * vd, dtype=q.dtype, device=q.device)
     _run("sharpi_attention_generic", _ptr(q), _ptr(k_cache), _ptr(v_cache), _code(q.dtype), _ptr(block_table),
          _ptr(entry_of_token), _ptr(positions), _ptr(out), int(window_kind), int(window), float(scale), T, nh, nkv,
-         hd, vd, k_cache.shape[2], block_table.shape[1], k_cache.shape[0], float(softcap), *_sink_args(sink, nh), _stream())
+         hd, vd, k_cache.shape[2], block_table.shape[1], k_cache.shape[0], float(softcap), *_sink_args(sink, nh), int(keep),
+         *_gate_args(gate, q, nh), _stream())
     return out
+
+
+def _gate_args(gate, q: torch.Tensor, nh: int):
+    """(pointer, row stride) of a gate with one number per token and head: gate = (rows [T, N] of q's dtype, column) or None."""
+    if gate is None:
+        return None, 0
+    rows, col = gate
+    _dev(rows)
+    _need(rows.dim() == 2 and rows.shape[0] == q.shape[0] and rows.dtype == q.dtype and 0 <= col and col + nh <= rows.shape[1],
+          "attention: the gates' columns must lie inside [T, N] rows of q's dtype")
+    return rows.data_ptr() + col * rows.element_size(), rows.shape[1]
 
 
 DECODE_RUN_KEYS = _lib.DECODE_RUN_KEYS   # keys per block of the decode kernel (fixed: sums must not depend on the batch)
@@ -348,73 +376,89 @@ def decode_max_splits(max_context: int) -> int:
     return ((max(1, int(max_context)) - 1) >> 4) // (DECODE_RUN_KEYS // 16) + 1
 
 
-def decode_attention_ok(dtype: torch.dtype, hd: int) -> bool:
-    return dtype == torch.bfloat16 and _lib.attention_takes("decode", hd)
+def decode_runs(max_context: int, window_kind: int, window: int, keep: int = 0) -> int:
+    """The same for a layer whose window is known: a token walks the 16-key blocks that its window touches and
+    those that hold the kept first keys."""
+    every = decode_max_splits(max_context)
+    if window_kind == WINDOW_NONE:
+        return every
+    blocks = (int(window) + 14) // 16 + 1 + (int(keep) + 15) // 16
+    return min(every, (blocks * 16 + DECODE_RUN_KEYS - 1) // DECODE_RUN_KEYS)
+
+
+def decode_attention_ok(dtype: torch.dtype, hd: int, vd: Optional[int] = None) -> bool:
+    return dtype == torch.bfloat16 and _lib.attention_takes("decode", hd, vd)
 
 
 def attention_decode(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_table: torch.Tensor,
                      entry_of_token: torch.Tensor, positions: torch.Tensor, token_list: Optional[torch.Tensor],
                      max_context: int, window_kind: int, window: int, scale: float, nh: int, nkv: int, hd: int,
-                     out: Optional[torch.Tensor] = None, softcap: float = 0.0, sink: bool = False) -> torch.Tensor:
+                     out: Optional[torch.Tensor] = None, softcap: float = 0.0, sink: bool = False,
+                     vd: Optional[int] = None, keep: int = 0, gate=None) -> torch.Tensor:
     """Split-K flash-decode for the listed tokens (all tokens if token_list is None), each a
-    single query over its request's pages.  `max_context` bounds position + 1 of every token."""
+    single query over its request's pages.  `max_context` bounds position + 1 of every token.  vd, keep and gate:
+    see :func:`attention_generic`."""
     _dev(q, k_cache, v_cache, block_table, entry_of_token, positions, token_list, out)
     _i32(block_table, "block_table")
     _i32(entry_of_token, "entry_of_token")
     _i32(positions, "positions")
     _i32(token_list, "token_list")
     T = q.shape[0]
-    _need(q.shape == (T, nh * hd) and decode_attention_ok(q.dtype, hd), "attention_decode: q must be bfloat16 [T, nh*hd], hd a head size the kernel is compiled for")
-    _need(_cache_shapes_ok(k_cache, v_cache, nkv, hd) and k_cache.dtype == q.dtype and v_cache.dtype == q.dtype,
+    vd = int(vd or hd)
+    _need(q.shape == (T, nh * hd) and decode_attention_ok(q.dtype, hd, vd), "attention_decode: q must be bfloat16 [T, nh*hd], hd and vd head sizes the kernel is compiled for")
+    _need(_cache_shapes_ok(k_cache, v_cache, nkv, hd, vd) and k_cache.dtype == q.dtype and v_cache.dtype == q.dtype,
           "attention_decode: caches must be K [pages, nkv, page_size, hd], V [pages, nkv, hd, page_size] bfloat16")
     _need(block_table.dim() == 2 and entry_of_token.shape == (T,) and positions.shape == (T,),
           "attention_decode: block_table [entries, max_blocks], per-token arrays [T]")
     n_list = T if token_list is None else token_list.shape[0]
     if out is None:
-        out = torch.empty_like(q)
-    _need(out.shape == q.shape and out.dtype == q.dtype, "attention_decode: out must match q")
-    max_splits = decode_max_splits(max_context)
-    part_o = torch.empty(n_list * nh * max_splits * hd, dtype=torch.float32, device=q.device)
+        out = torch.empty(T, nh * vd, dtype=q.dtype, device=q.device)
+    _need(out.shape == (T, nh * vd) and out.dtype == q.dtype, "attention_decode: out must be [T, nh*vd] of q's dtype")
+    max_splits = decode_runs(max_context, window_kind, window, keep)
+    part_o = torch.empty(n_list * nh * max_splits * vd, dtype=torch.float32, device=q.device)
     part_ml = torch.empty(n_list * nh * max_splits * 2, dtype=torch.float32, device=q.device)
-    _run("sharpi_attention_decode", _ptr(q), _ptr(k_cache), _ptr(v_cache), _ptr(block_table), _ptr(entry_of_token),
+    _run("sharpi_attention_decode_values", _ptr(q), _ptr(k_cache), _ptr(v_cache), _ptr(block_table), _ptr(entry_of_token),
          _ptr(positions), _ptr(token_list), _ptr(part_o), _ptr(part_ml), _ptr(out), int(window_kind), int(window),
-         float(scale), n_list, nh, nkv, hd, k_cache.shape[2], block_table.shape[1], k_cache.shape[0], max_splits,
-         float(softcap), *_sink_args(sink, nh), _stream())
+         float(scale), n_list, nh, nkv, hd, vd, k_cache.shape[2], block_table.shape[1], k_cache.shape[0], max_splits,
+         float(softcap), *_sink_args(sink, nh), int(keep), *_gate_args(gate, q, nh), _stream())
     return out
 
 
 PREFILL_TILE_TOKENS = _lib.PREFILL_TILE_TOKENS   # tokens per block of the prefill kernel (32 per wave)
 
 
-def prefill_attention_ok(dtype: torch.dtype, hd: int) -> bool:
-    return dtype == torch.bfloat16 and _lib.attention_takes("prefill", hd)
+def prefill_attention_ok(dtype: torch.dtype, hd: int, vd: Optional[int] = None) -> bool:
+    return dtype == torch.bfloat16 and _lib.attention_takes("prefill", hd, vd)
 
 
 def attention_prefill(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_table: torch.Tensor,
                       positions: torch.Tensor, tiles: torch.Tensor, window_kind: int, window: int, scale: float,
                       nh: int, nkv: int, hd: int, out: Optional[torch.Tensor] = None,
-                      tile_tokens: int = PREFILL_TILE_TOKENS, softcap: float = 0.0, sink: bool = False) -> torch.Tensor:
+                      tile_tokens: int = PREFILL_TILE_TOKENS, softcap: float = 0.0, sink: bool = False,
+                      vd: Optional[int] = None, keep: int = 0, gate=None) -> torch.Tensor:
     """Flash attention for the listed tiles: tiles int32 [n, 3] = (entry, first token, rows <=
     tile_tokens), the tokens of a tile consecutive in one entry.  tile_tokens (128, or 64: blocks of
     half the rows, for short prompts) is what the caller cut the tiles to; a row's result does not
-    depend on it."""
+    depend on it.  vd, keep and gate: see :func:`attention_generic`."""
     _dev(q, k_cache, v_cache, block_table, positions, tiles, out)
     _i32(block_table, "block_table")
     _i32(positions, "positions")
     _i32(tiles, "tiles")
     T = q.shape[0]
-    _need(q.shape == (T, nh * hd) and prefill_attention_ok(q.dtype, hd),
-          "attention_prefill: q must be bfloat16 [T, nh*hd], hd a head size the kernel is compiled for")
-    _need(_cache_shapes_ok(k_cache, v_cache, nkv, hd) and k_cache.dtype == q.dtype and v_cache.dtype == q.dtype,
+    vd = int(vd or hd)
+    _need(q.shape == (T, nh * hd) and prefill_attention_ok(q.dtype, hd, vd),
+          "attention_prefill: q must be bfloat16 [T, nh*hd], hd and vd head sizes the kernel is compiled for")
+    _need(_cache_shapes_ok(k_cache, v_cache, nkv, hd, vd) and k_cache.dtype == q.dtype and v_cache.dtype == q.dtype,
           "attention_prefill: caches must be K [pages, nkv, page_size, hd], V [pages, nkv, hd, page_size] bfloat16")
     _need(block_table.dim() == 2 and positions.shape == (T,) and tiles.dim() == 2 and tiles.shape[1] == 3,
           "attention_prefill: block_table [entries, max_blocks], positions [T], tiles [n, 3]")
     if out is None:
-        out = torch.empty_like(q)
-    _need(out.shape == q.shape and out.dtype == q.dtype, "attention_prefill: out must match q")
+        out = torch.empty(T, nh * vd, dtype=q.dtype, device=q.device)
+    _need(out.shape == (T, nh * vd) and out.dtype == q.dtype, "attention_prefill: out must be [T, nh*vd] of q's dtype")
     _run("sharpi_attention_prefill", _ptr(q), _ptr(k_cache), _ptr(v_cache), _ptr(block_table), _ptr(positions),
          _ptr(tiles), _ptr(out), tiles.shape[0], int(tile_tokens), int(window_kind), int(window), float(scale), nh,
-         nkv, hd, k_cache.shape[2], block_table.shape[1], k_cache.shape[0], float(softcap), *_sink_args(sink, nh), _stream())
+         nkv, hd, vd, k_cache.shape[2], block_table.shape[1], k_cache.shape[0], float(softcap), *_sink_args(sink, nh), int(keep),
+         *_gate_args(gate, q, nh), _stream())
     return out
 
 
@@ -441,6 +485,7 @@ def norm_add(h: torch.Tensor, delta, weight: torch.Tensor, eps: float,
     """h += unit_rms(delta) * weight, in place in float; with ``out_dtype`` the new h is also
     returned in that storage type (what the next branch reads).  delta: a tensor [T, H] or an
     ExpertSum without a shared part (formed on the fly, rounded once to its storage type)."""
+    delta = _foldable(delta)
     lazy = delta if isinstance(delta, ExpertSum) else None
     if lazy is not None and lazy.shared is not None:
         delta, lazy = lazy.tensor(), None
@@ -757,12 +802,20 @@ def _row_blocks(group_rows: Optional[int]) -> int:
     return 2 if group_rows <= 32 else 4
 
 
+UNGATED_ACTIVATIONS = {"relu2": 1, "gelu_tanh": 2, "silu": 3, "gelu": 4}      # csrc/common.h UACT_*
+
+
+def _ungated_code(act: Optional[str]) -> int:
+    _need(act is None or act in UNGATED_ACTIVATIONS, f"activation {act!r} is not known ({', '.join(sorted(UNGATED_ACTIVATIONS))})")
+    return 0 if act is None else UNGATED_ACTIVATIONS[act]
+
+
 def gemm_skinny(x: torch.Tensor, w, out_dtype: torch.dtype, a_rows: Optional[torch.Tensor] = None,
                 offsets: Optional[torch.Tensor] = None, n_rows: Optional[int] = None, R: Optional[int] = None,
-                NW: Optional[int] = None, group_rows: Optional[int] = None) -> torch.Tensor:
+                NW: Optional[int] = None, group_rows: Optional[int] = None, act: Optional[str] = None) -> torch.Tensor:
     """x [M, K] @ w[N, K]^T for M <= 64, or per expert with w [E, N, K] over an expert-sorted row
     list (``group_rows``: a bound on the rows of one expert, if known), on the matrix cores;
-    w a tensor (row-major) or a PackedWeight."""
+    w a tensor (row-major) or a PackedWeight.  ``act``: an ungated activation on the results (rounded to bfloat16 first)."""
     w, packed = _unwrap(w)
     _dev(x, w, a_rows, offsets)
     _i32(a_rows, "a_rows")
@@ -788,7 +841,7 @@ def gemm_skinny(x: torch.Tensor, w, out_dtype: torch.dtype, a_rows: Optional[tor
     pr, pw = skinny_plan(N, K, _row_blocks(group_rows) if grouped else (M + 15) // 16, max(E, 1))
     out = torch.empty(M, N, dtype=out_dtype, device=x.device)
     _run("sharpi_gemm_skinny", _ptr(x), _ptr(w), _ptr(out), _code(out_dtype), M, N, K, _ptr(a_rows), _ptr(offsets), E,
-         R or pr, NW or pw, 1 if packed else 0, _row_blocks(group_rows) if grouped else 0, _stream())
+         R or pr, NW or pw, 1 if packed else 0, _row_blocks(group_rows) if grouped else 0, _ungated_code(act), _stream())
     return out
 
 
@@ -846,13 +899,14 @@ def picked_ok(n_tokens: int, k: int, N: int, K: int, act: bool, packed: bool) ->
 
 
 def gemm_skinny_picked(x: torch.Tensor, w, ids: torch.Tensor, wts: Optional[torch.Tensor], shared: bool, gather: bool,
-                       act, out_dtype: torch.dtype) -> torch.Tensor:
+                       act, out_dtype: torch.dtype, ungated: Optional[str] = None) -> torch.Tensor:
     """Per-expert products of a few decode tokens straight from the router's picks ids [T, k]:
     row i of the result is pair i = (token i // k, pick i % k), followed (shared) by one row per
     token through expert E of w [E + 1, N, K].  gather: x [T, K] is read by token, otherwise x is in
     the result's row order.  act (True: SiLU; or an activation's code; False: none): w holds gate
     rows then up rows and the result is act(s g) * (s u) [rows, N/2] with s the pair's weight (wts;
-    1 for the shared rows)."""
+    1 for the shared rows).  ``ungated``: an activation without a gate on the plain results instead.  Picks
+    of the experts' number and above (identity experts) have no product: their rows are left as they are."""
     act, act_limit = _act_pair(ACT_SILU if act is True else act)
     w, packed = _unwrap(w)
     _dev(x, w, ids, wts)
@@ -876,12 +930,12 @@ def gemm_skinny_picked(x: torch.Tensor, w, ids: torch.Tensor, wts: Optional[torc
     pr, pw = skinny_plan(N, K, 1 if T * k <= 16 else 2 if T * k <= 32 else 4, min(E, T * k) + (1 if shared else 0), bool(act))
     out = torch.empty(rows, N // 2 if act else N, dtype=out_dtype, device=x.device)
     _run("sharpi_gemm_skinny_picked", _ptr(x), _ptr(w), _ptr(out), _code(out_dtype), N, K, _ptr(ids), _ptr(wts), T * k, k, E,
-         1 if shared else 0, 1 if gather else 0, act, act_limit, pr, pw, 1 if packed else 0, _stream())
+         1 if shared else 0, 1 if gather else 0, act, act_limit, pr, pw, 1 if packed else 0, _ungated_code(ungated), _stream())
     return out
 
 
-def linear(x: torch.Tensor, w, out_dtype: Optional[torch.dtype] = None) -> torch.Tensor:
-    """y = x W^T.  float32 weights: the float FMA kernel (true 32-bit, whatever x was stored
+def linear(x: torch.Tensor, w, out_dtype: Optional[torch.dtype] = None, act: Optional[str] = None) -> torch.Tensor:
+    """y = x W^T, or f(x W^T) with ``act`` (an ungated activation: in the few-rows kernel's epilogue, else a kernel of its own).  float32 weights: the float FMA kernel (true 32-bit, whatever x was stored
     as).  bfloat16 weights stored tile by tile (a PackedWeight): the weight-streaming kernel for a
     few rows; beyond, the library's matrix product with float accumulation over the row-major
     copy, as the reference calls a library there (reference:
@@ -890,6 +944,11 @@ def linear(x: torch.Tensor, w, out_dtype: Optional[torch.dtype] = None) -> torch
     (the few-rows kernel up to 64 rows, the grouped kernel with the matrix as its one group
     beyond)."""
     out_dtype = out_dtype or x.dtype
+    if act is not None:
+        few = out_dtype == torch.bfloat16 and w.dtype == torch.bfloat16 and skinny_ok(x.shape[0], w.shape[0], w.shape[1])
+        if not few:
+            return activation(linear(x, w, out_dtype), act)
+        return gemm_skinny(x if x.dtype == torch.bfloat16 else cast(x, torch.bfloat16), w, out_dtype, act=act)
     if isinstance(w, PackedWeight):
         xb = x if x.dtype == torch.bfloat16 else cast(x, torch.bfloat16)
         _need(xb.dim() == 2 and xb.shape[1] == w.shape[1], f"linear: x {tuple(x.shape)} vs w {tuple(w.shape)}")
@@ -945,7 +1004,7 @@ GATE_SIGMOID, GATE_SOFTMAX, GATE_SOFTMAX_PICKED = 0, 1, 2
 
 def router_topk(x: torch.Tensor, wr: torch.Tensor, k: int, gate: int = GATE_SIGMOID, renorm: bool = False,
                 want_gates: bool = False, correction: Optional[torch.Tensor] = None, n_groups: int = 1,
-                keep_groups: int = 1, bias: Optional[torch.Tensor] = None, weight_scale: float = 1.0):
+                keep_groups: int = 1, bias: Optional[torch.Tensor] = None, weight_scale: float = 1.0, group_top: int = 2):
     """Router logits in float (plus ``bias``, float32 [E], where given), gate, k picks (lowest index
     wins a tie).  Gates: sigmoid, softmax over all experts, or GATE_SOFTMAX_PICKED: the largest logits are
     picked and the weights are the softmax over the picked logits alone (the gate values handed
@@ -954,7 +1013,7 @@ def router_topk(x: torch.Tensor, wr: torch.Tensor, k: int, gate: int = GATE_SIGM
     ``correction`` (float32 [E]) is added to the gate values for the choice only: the weights stay
     the gate values.  With ``n_groups`` > ``keep_groups`` the experts form n_groups equal groups of
     neighbours and only those of the keep_groups best groups can be picked (a group's rank: the sum
-    of its two largest choice scores).  ``weight_scale`` multiplies the weights at the end."""
+    of its ``group_top`` (1 or 2) largest choice scores).  ``weight_scale`` multiplies the weights at the end."""
     _dev(x, wr, correction, bias)
     _need(x.dim() == 2 and wr.dim() == 2 and x.shape[1] == wr.shape[1], "router: x [T, H], wr [E, H]")
     T, H = x.shape
@@ -969,7 +1028,8 @@ def router_topk(x: torch.Tensor, wr: torch.Tensor, k: int, gate: int = GATE_SIGM
     wts = torch.empty(T, k, dtype=torch.float32, device=x.device)
     gates = torch.empty(T, E, dtype=torch.float32, device=x.device) if want_gates else None
     _run("sharpi_router_topk", _ptr(x), _code(x.dtype), _ptr(wr), _code(wr.dtype), _ptr(ids), _ptr(wts), _ptr(gates),
-         T, H, E, k, gate, 1 if renorm else 0, _ptr(correction), int(n_groups), int(keep_groups), _ptr(bias), float(weight_scale), _stream())
+         T, H, E, k, gate, 1 if renorm else 0, _ptr(correction), int(n_groups), int(keep_groups), _ptr(bias), float(weight_scale),
+         int(group_top), _stream())
     return (ids, wts, gates) if want_gates else (ids, wts)
 
 
@@ -1042,11 +1102,12 @@ def _new_routing(T: int, k: int, n_experts: int, shared_group: bool, dev) -> Rou
     return rt
 
 
-def moe_permute(ids: torch.Tensor, wts: torch.Tensor, n_experts: int, shared_group: bool = False) -> Routing:
+def moe_permute(ids: torch.Tensor, wts: torch.Tensor, n_experts: int, shared_group: bool = False, identity: bool = False) -> Routing:
     """(token, pick) pairs sorted by expert: offsets [E+1], sorted_token, sorted_w, inv_pos, and
     the plan of the grouped product for many rows, which
     says how the experts' row tiles are dealt to the blocks (csrc/grouped_plan.h).  With
-    shared_group one more group follows the experts: every token once with weight 1."""
+    shared_group one more group follows the experts: every token once with weight 1.  With ``identity``
+    picks of n_experts and above may occur, which get no row (offsets[E] then counts the rows there are)."""
     _dev(ids, wts)
     _i32(ids, "ids")
     _need(ids.shape == wts.shape and wts.dtype == torch.float32 and ids.dim() == 2, "moe_permute: ids/wts [T, k]")
@@ -1054,26 +1115,29 @@ def moe_permute(ids: torch.Tensor, wts: torch.Tensor, n_experts: int, shared_gro
     rt = _new_routing(T, k, n_experts, shared_group, ids.device)
     _run("sharpi_moe_permute", _ptr(ids), _ptr(wts), _ptr(rt.offsets), _ptr(rt.sorted_token), _ptr(rt.sorted_w),
          _ptr(rt.inv_pos), _ptr(rt.plan), rt.plan.numel(), T, k, n_experts,
-         1 if shared_group else 0, _stream())
+         1 if shared_group else 0, 1 if identity else 0, _stream())
     return rt
 
 
 def route(x: torch.Tensor, wr: torch.Tensor, k: int, gate: int = GATE_SIGMOID, renorm: bool = False,
           shared_group: bool = False, correction: Optional[torch.Tensor] = None, n_groups: int = 1,
-          keep_groups: int = 1, bias: Optional[torch.Tensor] = None, weight_scale: float = 1.0):
-    """router_topk then moe_permute: (ids, weights, Routing)."""
+          keep_groups: int = 1, bias: Optional[torch.Tensor] = None, weight_scale: float = 1.0, group_top: int = 2,
+          identity: int = 0):
+    """router_topk then moe_permute: (ids, weights, Routing).  The last ``identity`` rows of wr are identity experts'."""
     ids, wts = router_topk(x, wr, k, gate, renorm, correction=correction, n_groups=n_groups, keep_groups=keep_groups,
-                           bias=bias, weight_scale=weight_scale)
-    return ids, wts, moe_permute(ids, wts, wr.shape[0], shared_group)
+                           bias=bias, weight_scale=weight_scale, group_top=group_top)
+    return ids, wts, moe_permute(ids, wts, wr.shape[0] - identity, shared_group, identity > 0)
 
 
-def gemm_grouped(x: torch.Tensor, w, rt: Routing, gather: bool, out_dtype: torch.dtype, max_blocks: int = 0) -> torch.Tensor:
+def gemm_grouped(x: torch.Tensor, w, rt: Routing, gather: bool, out_dtype: torch.dtype, max_blocks: int = 0,
+                 relu2: bool = False) -> torch.Tensor:
     """Per-group products for many rows on the matrix cores (bfloat16): the experts, and the
     always-on group if the routing has one (group E of w).  gather: x rows are read through the
     routing's token list; otherwise x is already in expert-sorted order.  The product's blocks
     stay on their compute units until the work is done; ``max_blocks`` > 0 bounds their number
     (the units left over are for other work running beside the product).  Products that read
-    one routing must not run at the same time (they share its plan's ticket counters)."""
+    one routing must not run at the same time (they share its plan's ticket counters).  ``relu2``: the
+    results are the squares of their relu."""
     w, packed = _unwrap(w)
     _dev(x, w)
     _need(x.dtype == torch.bfloat16 and w.dtype == torch.bfloat16, "gemm_grouped: bfloat16 operands only")
@@ -1085,7 +1149,7 @@ def gemm_grouped(x: torch.Tensor, w, rt: Routing, gather: bool, out_dtype: torch
     out = torch.empty(rt.n_rows, N, dtype=out_dtype, device=x.device)
     _run("sharpi_gemm_grouped", _ptr(x), x.shape[0], _ptr(w), _ptr(out), _code(out_dtype), rt.n_rows, N, K,
          _ptr(rt.sorted_token) if gather else None, _ptr(rt.offsets), _ptr(rt.plan), rt.n_groups,
-         1 if packed else 0, int(max_blocks), _stream())
+         1 if packed else 0, int(max_blocks), 1 if relu2 else 0, _stream())
     return out
 
 
@@ -1213,7 +1277,8 @@ def qk_prep(proj: torch.Tensor, q_off: int, k_off: int, v_off: Optional[int], nh
             eps: float = 1e-6, inv_freq: Optional[torch.Tensor] = None, pair_layout: int = PAIRS_INTERLEAVED,
             magnitude: float = 1.0, conv_w: Optional[torch.Tensor] = None, tail: Optional[torch.Tensor] = None,
             update_tail: bool = True, bias: Optional[torch.Tensor] = None,
-            temperature: Optional[Tuple[float, float]] = None, maps: int = 1) -> torch.Tensor:
+            temperature: Optional[Tuple[float, float]] = None, maps: int = 1,
+            v_mix: Optional[Tuple[torch.Tensor, int, float]] = None) -> torch.Tensor:
     """From a step's projections proj [T, N] (q at columns q_off.., k at k_off.., v at v_off.., or
     v_off None: the values are the keys before norm and rotation): optional short causal
     convolution over time on every channel (conv_w float32 [channels, taps]; tail float32 [slots,
@@ -1228,7 +1293,8 @@ def qk_prep(proj: torch.Tensor, q_off: int, k_off: int, v_off: Optional[int], nh
     maps side by side (hd is their width together; rotary_dim at most hd / maps, applied to each map's
     own leading elements), and q comes back expanded, [T, nh * maps * hd]: one row of the head's width
     per (head, map), the map's elements in their place and zeros elsewhere, so that attention over
-    nh * maps query heads and keys of width hd computes every map's scores on its own."""
+    nh * maps query heads and keys of width hd computes every map's scores on its own.  ``v_mix`` = (rows [T, M] of
+    proj's dtype, column, c): the values stored are (1 - c) v + c * (columns column .. of rows), in float."""
     _dev(proj, k_cache, v_cache, slot_mapping, q_norm_w, k_norm_w, inv_freq, conv_w, tail, bias)
     maps = int(maps)
     _need(maps >= 1 and hd % (2 * maps) == 0, "qk_prep: a head must split into its maps, each of even width")
@@ -1270,6 +1336,11 @@ def qk_prep(proj: torch.Tensor, q_off: int, k_off: int, v_off: Optional[int], nh
               "qk_prep: tail must be float32 [slots, taps - 1, channels]")
         _need(ctx.state_slots.shape == (ctx.n_entries,) and ctx.cu_tokens.shape == (ctx.n_entries + 1,)
               and ctx.entry_of_token.shape == (T,), "qk_prep: the step's per-entry arrays do not fit")
+    v_other, vo_off, vo_c = v_mix if v_mix is not None else (None, 0, 0.0)
+    if v_other is not None:
+        _dev(v_other)
+        _need(v_other.dim() == 2 and v_other.shape[0] == T and v_other.dtype == proj.dtype and 0 <= vo_off
+              and vo_off + nkv * vd <= v_other.shape[1], "qk_prep: the other layer's values must lie inside [T, M] rows of proj's dtype")
     q_out = torch.empty(T, qn * maps, dtype=proj.dtype, device=proj.device)
     page_size = k_cache.shape[2] if k_cache is not None else 0
     _run("sharpi_qk_prep", _ptr(proj), _code(proj.dtype), N, int(q_off), int(k_off), int(v_off) if own_v else -1, T,
@@ -1277,7 +1348,8 @@ def qk_prep(proj: torch.Tensor, q_off: int, k_off: int, v_off: Optional[int], nh
          _ptr(ctx.cu_tokens), _ptr(ctx.positions), int(norm_mode), _ptr(q_norm_w), _ptr(k_norm_w), float(eps),
          _ptr(inv_freq), rotary_dim, 1 if pair_layout == PAIRS_HALF_SPLIT else 0, float(magnitude), _ptr(q_out),
          _ptr(k_cache), _ptr(v_cache), _ptr(slot_mapping), page_size, 1 if update_tail else 0, _ptr(bias),
-         1 if temperature is not None else 0, float(fs), float(asc), maps, _stream())
+         1 if temperature is not None else 0, float(fs), float(asc), maps, _ptr(v_other),
+         0 if v_other is None else v_other.shape[1], int(vo_off), float(vo_c), _stream())
     return q_out
 
 
@@ -1465,8 +1537,6 @@ def post_pre_norm(h: torch.Tensor, delta, w_post: torch.Tensor, eps: float, w_ne
     return out
 
 
-UNGATED_ACTIVATIONS = {"relu2": 1, "gelu_tanh": 2, "silu": 3}
-
 
 def activation(x: torch.Tensor, name: str) -> torch.Tensor:
     """f(x) element by element, f one of UNGATED_ACTIVATIONS (relu2: the square of relu)."""
@@ -1505,26 +1575,28 @@ def norm_mean(xs, weights, eps: float) -> torch.Tensor:
 # ---------------------------------------------------------------------------
 def attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, group, ctx, window_kind: int,
               window: int, scale: float, nh: int, nkv: int, hd: int, vd: Optional[int] = None, softcap: float = 0.0,
-              sink=False) -> torch.Tensor:
+              sink=False, keep: int = 0, gate=None) -> torch.Tensor:
     """Attention of the step's tokens over their requests' pages (`group`: the cache group's
-    block tables, `ctx`: the step).  Values of another width than keys (vd) go through the float kernel.
+    block tables, `ctx`: the step).  Sizes the matrix-core kernels are not compiled for go through the float kernel.
     softcap > 0 caps the scores (softcap * tanh(score / softcap)); sink adds a key of score 0 without a
-    value to the softmax's denominator (True), or one of a learned score per head (a float32 tensor [nh])."""
-    same = vd is None or vd == hd
-    if same and decode_attention_ok(q.dtype, hd) and (prefill_attention_ok(q.dtype, hd) or not ctx.n_prefill_tiles):
+    value to the softmax's denominator (True), or one of a learned score per head (a float32 tensor [nh]).
+    keep: a window's layer sees the sequence's first `keep` keys too.  gate = (rows [T, N], column): head h's output
+    times sigmoid(rows[t, column + h])."""
+    vd = int(vd or hd)
+    if decode_attention_ok(q.dtype, hd, vd) and (prefill_attention_ok(q.dtype, hd, vd) or not ctx.n_prefill_tiles):
         # entries of one token: split-K decode kernel; longer entries: flash kernel, a tile of tokens a block
-        out = torch.empty_like(q)
+        out = torch.empty(q.shape[0], nh * vd, dtype=q.dtype, device=q.device)
         if ctx.n_prefill_tiles:
             attention_prefill(q, k_cache, v_cache, group.block_table, ctx.positions, ctx.prefill_tiles, window_kind,
                               window, scale, nh, nkv, hd, out=out, tile_tokens=ctx.prefill_tile_tokens, softcap=softcap,
-                              sink=sink)
+                              sink=sink, vd=vd, keep=keep, gate=gate)
         if ctx.n_decode:
             attention_decode(q, k_cache, v_cache, group.block_table, ctx.entry_of_token, ctx.positions,
                              ctx.decode_tokens, group.max_context, window_kind, window, scale, nh, nkv, hd, out=out,
-                             softcap=softcap, sink=sink)
+                             softcap=softcap, sink=sink, vd=vd, keep=keep, gate=gate)
         return out
     return attention_generic(q, k_cache, v_cache, group.block_table, ctx.entry_of_token, ctx.positions, window_kind,
-                             window, scale, nh, nkv, hd, vd, softcap=softcap, sink=sink)
+                             window, scale, nh, nkv, hd, vd, softcap=softcap, sink=sink, keep=keep, gate=gate)
 
 
 def grouped_swiglu(x: torch.Tensor, w_gate_up, rt: Routing, out_dtype: torch.dtype, scaled: bool = True,
@@ -1544,10 +1616,11 @@ def grouped_swiglu(x: torch.Tensor, w_gate_up, rt: Routing, out_dtype: torch.dty
     return gated_act(grouped_linear(x, w_gate_up, rt, True, out_dtype), scale, act)
 
 
-def grouped_linear(x: torch.Tensor, w, rt: Routing, gather: bool, out_dtype: torch.dtype, max_blocks: int = 0) -> torch.Tensor:
+def grouped_linear(x: torch.Tensor, w, rt: Routing, gather: bool, out_dtype: torch.dtype, max_blocks: int = 0,
+                   act: Optional[str] = None) -> torch.Tensor:
     """Per-expert products over the routing's expert-sorted row list: w [E, N, K] (a tensor or a
     PackedWeight); x rows are read through the token list (gather) or are already in sorted order.
-    Returns [n_rows, N]."""
+    Returns [n_rows, N].  ``act``: an ungated activation on the results, in the product's epilogue where the kernel has it."""
     if x.dtype != w.dtype:
         x = cast(x, w.dtype)
     N, K = w.shape[1], w.shape[2]
@@ -1555,10 +1628,12 @@ def grouped_linear(x: torch.Tensor, w, rt: Routing, gather: bool, out_dtype: tor
     if w.dtype == torch.bfloat16 and K % 128 == 0 and N % 4 == 0:
         if rt.n_tokens <= SKINNY_MAX_ROWS:   # no expert has more rows than there are tokens
             return gemm_skinny(x, w, out_dtype, a_rows=a_rows, offsets=rt.offsets, n_rows=rt.n_rows,
-                               group_rows=rt.n_tokens)
-        return gemm_grouped(x, w, rt, gather, out_dtype, max_blocks=max_blocks)
+                               group_rows=rt.n_tokens, act=act)
+        y = gemm_grouped(x, w, rt, gather, out_dtype, max_blocks=max_blocks, relu2=act == "relu2")
+        return y if act in (None, "relu2") else activation(y, act)
     y = grouped_gemm(x, w, rt.offsets, a_rows, rt.n_rows)
-    return y if y.dtype == out_dtype else cast(y, out_dtype)
+    y = y if y.dtype == out_dtype else cast(y, out_dtype)
+    return y if act is None else activation(y, act)
 
 
 # ---------------------------------------------------------------------------
@@ -1838,6 +1913,7 @@ def hyper_step(src: torch.Tensor, lanes: Optional[torch.Tensor], n_streams: int,
     in ``lanes`` (float32 [T, S, W]; may be ``src`` itself; None: not stored).  Then u = sum_s in_w[s] new[s]
     (``in_w`` float32 [S]; None: the plain sum), and the result is unit_rms(u) * norm_w in ``out_dtype``,
     or, with ``norm_w`` None, u itself in float32.  ``rows`` (int32): only those tokens are produced."""
+    delta = _foldable(delta)
     lazy = delta if isinstance(delta, ExpertSum) else None
     base = lazy.y if lazy is not None else delta
     _dev(src, lanes, base, mix, out_w, in_w, norm_w, rows, *( [lazy.inv_pos, lazy.shared, lazy.weights] if lazy is not None else []))
@@ -1916,6 +1992,7 @@ def layer_norm(h: torch.Tensor, delta=None, weight: Optional[torch.Tensor] = Non
     ``norm`` = (weight, bias, eps): the layer norm of x; ``conv`` = (w float32 [N, taps], ring float32 [slots, taps,
     N], ctx), steps of single tokens only: x + sum_j w[:, j] x_(p - taps + 1 + j), earlier inputs from the request's
     ring (position p at p mod taps), into which x goes; neither: x itself."""
+    delta = _foldable(delta)
     lazy = delta if isinstance(delta, ExpertSum) else None
     base = lazy.y if lazy is not None else delta
     shared = lazy.shared if lazy is not None else None
@@ -1948,6 +2025,46 @@ def layer_norm(h: torch.Tensor, delta=None, weight: Optional[torch.Tensor] = Non
          _ptr(ctx.positions) if conv is not None else None, _ptr(ctx.state_slots) if conv is not None else None,
          _ptr(ctx.entry_of_token) if conv is not None else None, _stream())
     return out
+
+
+def sum_norm(h: torch.Tensor, delta, alpha: float, weight: torch.Tensor, bias: torch.Tensor, eps: float,
+             out_dtype: Optional[torch.dtype] = None, identity_is_h: bool = False) -> Optional[torch.Tensor]:
+    """x = LN(alpha * h + delta) * weight + bias, back into h (float32 [T, N], sums and statistics in float); with
+    ``out_dtype`` x is also returned in that storage type.  delta: a tensor or an ExpertSum (formed on the fly, not rounded).
+    ``identity_is_h``: what the sum's identity experts return is the row of h itself (their x its rounded copy): taken
+    from h, in float."""
+    lazy = delta if isinstance(delta, ExpertSum) else None
+    base = lazy.y if lazy is not None else delta
+    shared, wts = (lazy.shared, lazy.weights) if lazy is not None else (None, None)
+    ids, n_experts, ident = lazy.identity if lazy is not None and lazy.identity is not None else (None, 0, None)
+    ident = None if identity_is_h else ident
+    _dev(h, base, weight, bias, shared, wts, ids, ident)
+    _need(h.dim() == 2 and h.dtype == torch.float32, "sum_norm: h must be float32 [T, N]")
+    T, N = h.shape
+    _need(N <= LAYER_NORM_MAX_WIDTH, f"sum_norm: rows of at most {LAYER_NORM_MAX_WIDTH} elements")
+    _need(tuple(delta.shape) == (T, N) and base.shape[1] == N, f"sum_norm: delta {tuple(delta.shape)} vs h {tuple(h.shape)}")
+    _need(all(x.dtype == torch.float32 and x.shape == (N,) for x in (weight, bias)), "sum_norm: weight and bias must be float32 [N]")
+    out = torch.empty(T, N, dtype=out_dtype, device=h.device) if out_dtype is not None else None
+    _run("sharpi_sum_norm", _ptr(h), _ptr(base), _code(base.dtype), _ptr(lazy.inv_pos) if lazy is not None else None, _ptr(wts),
+         lazy.k if lazy is not None else 0, _ptr(shared), _ptr(ids), int(n_experts), _ptr(ident), float(alpha), _ptr(weight), _ptr(bias),
+         float(eps), T, N, _ptr(out), _code(out_dtype) if out is not None else 0, _stream())
+    return out
+
+
+def embed_norm(ids: torch.Tensor, table: torch.Tensor, weight: torch.Tensor, bias: torch.Tensor, eps: float, scale: float = 1.0,
+               out_dtype: Optional[torch.dtype] = None):
+    """(x float32 [T, N], x in ``out_dtype`` or None) with x = LN(table[ids[t]] * scale) * weight + bias."""
+    _dev(ids, table, weight, bias)
+    _i32(ids, "ids")
+    _need(ids.dim() == 1 and table.dim() == 2, "embed_norm: ids [T], table [V, N]")
+    T, N = ids.shape[0], table.shape[1]
+    _need(N <= LAYER_NORM_MAX_WIDTH and all(x.dtype == torch.float32 and x.shape == (N,) for x in (weight, bias)),
+          f"embed_norm: rows of at most {LAYER_NORM_MAX_WIDTH} elements, weight and bias float32 [N]")
+    out = torch.empty(T, N, dtype=torch.float32, device=table.device)
+    copy = torch.empty(T, N, dtype=out_dtype, device=table.device) if out_dtype is not None else None
+    _run("sharpi_embed_norm", _ptr(ids), _ptr(table), _code(table.dtype), float(scale), _ptr(weight), _ptr(bias), float(eps), _ptr(out),
+         _ptr(copy), _code(out_dtype) if copy is not None else 0, T, N, _stream())
+    return out, copy
 
 
 def residual_conv(h: torch.Tensor, weight: torch.Tensor, ring: Optional[torch.Tensor], ctx, out_dtype: torch.dtype) -> torch.Tensor:

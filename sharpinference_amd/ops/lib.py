@@ -21,35 +21,36 @@ _SIGNATURES = {
     "sharpi_scale_softcap": [P, c_longlong, F, F, P],
     "sharpi_add_rmsnorm": [P, P, I, P, I, P, I, P, I, I, F, I, P, P, P, I, P],
     "sharpi_silu_mul": [P, P, P, I, I, I, I, F, P, P],
-    "sharpi_moe_combine": [P, P, P, P, P, I, I, I, I, P],
+    "sharpi_moe_combine": [P, P, P, P, P, I, I, I, I, P, I, P, P],
     "sharpi_cast": [P, I, P, I, c_longlong, P],
     "sharpi_add_bias": [P, I, P, I, I, P],
     "sharpi_peak_read": [P, c_longlong, P, P, P],
     "sharpi_peak_mfma": [P, I, I, P],
     "sharpi_random_fill": [P, I, c_longlong, c_ulonglong, I, F, I, I, P],
     "sharpi_rope_kv": [P, P, P, P, I, P, P, P, P, I, F, I, F, F, I, I, I, I, I, I, I, I, I, P],
-    "sharpi_attention_generic": [P, P, P, I, P, P, P, P, I, I, F, I, I, I, I, I, I, I, I, F, I, P, P],
+    "sharpi_attention_generic": [P, P, P, I, P, P, P, P, I, I, F, I, I, I, I, I, I, I, I, F, I, P, I, P, I, P],
     "sharpi_attention_decode": [P, P, P, P, P, P, P, P, P, P, I, I, F, I, I, I, I, I, I, I, I, F, I, P, P],
-    "sharpi_attention_prefill": [P, P, P, P, P, P, P, I, I, I, I, F, I, I, I, I, I, I, F, I, P, P],
+    "sharpi_attention_decode_values": [P, P, P, P, P, P, P, P, P, P, I, I, F, I, I, I, I, I, I, I, I, I, F, I, P, I, P, I, P],
+    "sharpi_attention_prefill": [P, P, P, P, P, P, P, I, I, I, I, F, I, I, I, I, I, I, I, F, I, P, I, P, I, P],
     "sharpi_gemm_tiled": [P, P, P, I, I, I, I, I, P, P, I, P],
-    "sharpi_gemm_skinny": [P, P, P, I, I, I, I, P, P, I, I, I, I, I, P],
+    "sharpi_gemm_skinny": [P, P, P, I, I, I, I, P, P, I, I, I, I, I, I, P],
     "sharpi_gemm_skinny_swiglu": [P, P, P, I, I, I, P, P, I, P, I, I, I, I, I, F, P],
-    "sharpi_gemm_skinny_picked": [P, P, P, I, I, I, P, P, I, I, I, I, I, I, F, I, I, I, P],
+    "sharpi_gemm_skinny_picked": [P, P, P, I, I, I, P, P, I, I, I, I, I, I, F, I, I, I, I, P],
     "sharpi_add_rmsnorm_router": [P, P, P, I, P, I, I, F, P, I, P, P, I, I, I, I, P],
-    "sharpi_router_topk": [P, I, P, I, P, P, P, I, I, I, I, I, I, P, I, I, P, F, P],
+    "sharpi_router_topk": [P, I, P, I, P, P, P, I, I, I, I, I, I, P, I, I, P, F, I, P],
     "sharpi_norm_add": [P, P, I, P, P, I, I, I, F, P, P, I, P],
     "sharpi_latent_prep": [P, I, I, P, I, I, P, I, I, I, I, P, P, P, P, P, P, I, F, P, P, F, I, I, I, I, I, P],
     "sharpi_head_gemm": [P, I, I, I, P, P, I, I, P, I, I, I, I, I, P],
     "sharpi_attention_latent": [P, P, I, P, P, P, P, P, I, I, F, I, I, I, I, I, I, I, P],
     "sharpi_attention_latent_mfma": [P, P, P, P, P, P, P, I, I, P, P, P, P, F, I, I, I, I, I, I, I, I, I, I, P],
     "sharpi_attention_latent_merge": [P, P, P, P, I, P, P, I, I, I, I, I, P],
-    "sharpi_moe_permute": [P, P, P, P, P, P, P, I, I, I, I, I, P],
-    "sharpi_gemm_grouped": [P, I, P, P, I, I, I, I, P, P, P, I, I, I, P],
+    "sharpi_moe_permute": [P, P, P, P, P, P, P, I, I, I, I, I, I, P],
+    "sharpi_gemm_grouped": [P, I, P, P, I, I, I, I, P, P, P, I, I, I, I, P],
     "sharpi_gemm_grouped_swiglu": [P, I, P, P, I, I, I, P, P, P, I, P, I, I, F, I, P],
     "sharpi_argmax_rows": [P, P, I, I, P],
     "sharpi_sample_rows": [P, P, P, P, P, P, P, P, I, I, P],
     "sharpi_edit_logits": [P, P, P, P, P, P, P, P, I, I, P],
-    "sharpi_qk_prep": [P, I, I, I, I, I, I, I, I, I, I, I, P, I, P, P, P, P, P, I, P, P, F, P, I, I, F, P, P, P, P, I, I, P, I, F, F, I, P],
+    "sharpi_qk_prep": [P, I, I, I, I, I, I, I, I, I, I, I, P, I, P, P, P, P, P, I, P, P, F, P, I, I, F, P, P, P, P, I, I, P, I, F, F, I, P, I, I, F, P],
     "sharpi_gla_walk": [P, I, I, I, I, I, P, F, P, P, P, P, I, I, I, I, I, P],
     "sharpi_gla_decays": [P, P, F, I, I, P],
     "sharpi_gla_walk_segmented": [P, I, I, I, I, I, P, F, P, P, P, P, I, I, I, I, P, P, I, P, P, P],
@@ -67,6 +68,8 @@ _SIGNATURES = {
     "sharpi_side_gate": [P, I, P, P, I, I, I, P, I, I, P],
     "sharpi_hyper_step": [P, c_longlong, c_longlong, P, P, I, P, P, P, I, P, P, P, P, I, F, P, I, P, I, I, I, P],
     "sharpi_layer_norm": [P, P, I, P, P, I, P, P, P, F, P, I, I, P, I, I, P, P, F, P, P, I, P, P, P, P],
+    "sharpi_sum_norm": [P, P, I, P, P, I, P, P, I, P, F, P, P, F, I, I, P, I, P],
+    "sharpi_embed_norm": [P, P, I, F, P, P, F, P, P, I, I, I, P],
     "sharpi_residual_conv": [P, P, I, P, P, P, P, P, P, I, I, I, P],
     "sharpi_embed_bigram": [P, P, I, F, P, I, c_longlong, c_longlong, I, P, P, P, P, P, P, I, I, P],
     "sharpi_lowrank": [P, I, I, I, I, I, P, I, P, P, I, P, I, I, P, I, P, P],
@@ -148,14 +151,14 @@ def load(verbose: bool = True) -> ctypes.CDLL:
 _takes: dict = {}
 
 
-def attention_takes(kind: str, hd: int) -> bool:
-    """Whether the matrix-core attention kernel of this kind ('decode' or 'prefill') is compiled for
-    head size hd: the library is asked, so that the choice of kernel cannot drift from the build."""
-    key = (kind, int(hd))
+def attention_takes(kind: str, hd: int, vd: Optional[int] = None) -> bool:
+    """Whether the matrix-core attention kernel of this kind ('decode' or 'prefill') is compiled for keys of width hd
+    and values of width vd (hd unless given): the library is asked, so that the choice of kernel cannot drift from the build."""
+    key = (kind, int(hd), int(vd or hd))
     if key not in _takes:
         fn = getattr(load(), f"sharpi_attention_{kind}_takes")
-        fn.argtypes, fn.restype = [c_int], c_int
-        _takes[key] = bool(fn(int(hd)))
+        fn.argtypes, fn.restype = [c_int, c_int], c_int
+        _takes[key] = bool(fn(int(hd), int(vd or hd)))
     return _takes[key]
 
 

@@ -90,13 +90,21 @@ class Attention(Part):
     keeps a key head's maps as one row of m * head_dim elements; queries are expanded to one such row per
     (head, map) with zeros in the other map's place, so the attention kernels compute each map's scores
     unchanged (csrc/qk_prep.hip, csrc/hyper.hip).  ``head_gate``: each head's output is multiplied by
-    sigmoid(W_g x)_h, one number per head (W_g [heads, hidden], made by the q|k|v launch)."""
+    sigmoid(W_g x)_h, one number per head (W_g [heads, hidden], made by the q|k|v launch; applied where the attention
+    kernels store, or behind the difference of the maps).
+
+    ``keep_first`` n: beside its window a query sees the sequence's first n keys, at their true positions (the
+    cache manager keeps their pages).  ``value_mix``: layers that share values of the same token.  "source": this
+    layer's values, as projected, are the ones the step's later layers mix in; "mixed": what is cached and attended
+    to is (1 - c) v + c v_source with a stored number c (tensor ``v_mix``, read by both kinds, used by this one)."""
 
     NAMES = {"q": "q_proj.weight", "k": "k_proj.weight", "v": "v_proj.weight", "o": "o_proj.weight",
              "q_bias": "q_proj.bias", "k_bias": "k_proj.bias", "v_bias": "v_proj.bias", "o_bias": "o_proj.bias",
              "q_norm": "q_norm.weight", "k_norm": "k_norm.weight",
              "q_conv": "q_conv.weight", "k_conv": "k_conv.weight", "v_conv": "v_conv.weight",
-             "sink": "sink", "g": "g_proj.weight", "lq1": "lq1", "lk1": "lk1", "lq2": "lq2", "lk2": "lk2"}
+             "sink": "sink", "g": "g_proj.weight", "lq1": "lq1", "lk1": "lk1", "lq2": "lq2", "lk2": "lk2",
+             "v_mix": "v_mix"}
+    SOURCE_VALUES = "source values"          # where a step keeps the projections that hold them (ctx.extras)
 
     def __init__(self, hidden: int, num_heads: int, num_kv_heads: int, head_dim: int,
                  rotary=None, qk_norm_eps: Optional[float] = None,
@@ -105,7 +113,8 @@ class Attention(Part):
                  v_head_dim: Optional[int] = None, qk_norm_weights: Optional[str] = None, values_from_keys: bool = False,
                  conv_taps: int = 0, softcap: float = 0.0, sink=False, names: Optional[Dict[str, str]] = None,
                  gate: bool = False, score_maps: int = 1, difference: Optional[float] = None,
-                 difference_eps: Optional[float] = None, head_gate: bool = False):
+                 difference_eps: Optional[float] = None, head_gate: bool = False, keep_first: int = 0,
+                 value_mix: Optional[str] = None):
         if num_heads % num_kv_heads:
             raise ValueError(f"{num_heads} heads cannot share {num_kv_heads} kv heads")
         self.maps = int(score_maps)
@@ -116,9 +125,17 @@ class Attention(Part):
         self.difference = float(difference) if difference is not None else 0.0
         self.difference_eps = float(difference_eps) if difference_eps is not None else 0.0
         self.head_gate = bool(head_gate)
-        if self.head_gate and (gate or self.maps == 1):
-            raise ValueError("a gate number per head belongs to differential attention and excludes the gate per channel")
-        prep = bool(qk_norm_weights or values_from_keys or conv_taps or self.maps > 1)
+        if self.head_gate and gate:
+            raise ValueError("a gate number per head excludes the gate per channel")
+        if value_mix not in (None, "source", "mixed"):
+            raise ValueError(f"value_mix {value_mix!r} is not known (None, 'source', 'mixed')")
+        self.value_mix, self.mix = value_mix, 0.0         # (mix: the stored number c)
+        if value_mix and (values_from_keys or conv_taps or bias):
+            raise ValueError("shared values are plain projections: no convolution, no bias, a value projection of their own")
+        self.keep_first = int(keep_first)
+        if self.keep_first < 0 or (self.keep_first and window_kind == WINDOW_NONE):
+            raise ValueError("keep_first belongs to a window")
+        prep = bool(qk_norm_weights or values_from_keys or conv_taps or self.maps > 1 or value_mix)
         self.map_dim = int(head_dim)                      # width of one score map of a head
         if rotary is not None and rotary.head_dim != head_dim:
             raise ValueError("the rotary table's head_dim differs from the mixer's")
@@ -188,7 +205,7 @@ class Attention(Part):
         return self.nh * self.hd + self.nkv * self.hd + (0 if self.values_from_keys else self.nkv * self.vd)
 
     def cache_spec(self):
-        kv = KVSpec(self.nkv, self.hd, self.window_kind, self.window, 0 if self.vd == self.hd else self.vd)
+        kv = KVSpec(self.nkv, self.hd, self.window_kind, self.window, 0 if self.vd == self.hd else self.vd, keep_first=self.keep_first)
         if not self.conv_taps:
             return kv
         return MixedSpec(kv, (StateSpec((self.conv_taps - 1, self._channels), torch.float32),))
@@ -218,6 +235,8 @@ class Attention(Part):
             specs[prefix + n["g"]] = ParamSpec((ov, self.hidden))
         if self.head_gate:
             specs[prefix + n["g"]] = ParamSpec((self.nh, self.hidden))
+        if self.value_mix:
+            specs[prefix + n["v_mix"]] = ParamSpec(())
         if self.maps > 1:
             for key in ("lq1", "lk1", "lq2", "lk2"):
                 specs[prefix + n[key]] = ParamSpec((self.map_dim,))
@@ -253,6 +272,8 @@ class Attention(Part):
         if self.maps > 1:
             lq1, lk1, lq2, lk2 = (source.get(prefix + n[key]).float() for key in ("lq1", "lk1", "lq2", "lk2"))
             self.lam = float(torch.exp((lq1 * lk1).sum()) - torch.exp((lq2 * lk2).sum()) + self.difference)
+        if self.value_mix:
+            self.mix = float(source.get(prefix + n["v_mix"]).float())
         if self.conv_taps:
             self.w_conv = torch.cat([source.get(prefix + n[k + "_conv"]).float() for k in kinds]).contiguous()
 
@@ -273,20 +294,27 @@ class Attention(Part):
             if self.prep:
                 mode = {None: ops.NORM_NONE, "head": ops.NORM_PER_HEAD, "projection": ops.NORM_WHOLE}[self.qk_norm_weights]
                 kn = self.nkv * self.hd
+                v_mix = None
+                if self.value_mix == "source":
+                    ctx.extras[self.SOURCE_VALUES] = (qkv, q_dim + kn)
+                elif self.value_mix:
+                    v_mix = (*ctx.extras[self.SOURCE_VALUES], self.mix)
                 q = ops.qk_prep(qkv, 0, q_dim, None if self.values_from_keys else q_dim + kn, self.nh, self.nkv, self.hd,
                                 self.vd, ctx, cache.k, cache.v, slots, mode, self.w_q_norm, self.w_k_norm,
                                 self.qk_norm_eps or 1e-6, inv_freq, layout,
                                 getattr(self.rotary, "magnitude", 1.0) if self.rotary is not None else 1.0,
                                 self.w_conv, cache.states[0] if self.conv_taps else None, update_tail=cache.write,
-                                bias=self.b_qkv, temperature=self.q_temperature, maps=self.maps)
+                                bias=self.b_qkv, temperature=self.q_temperature, maps=self.maps, v_mix=v_mix)
             else:
                 q = ops.rope_kv(qkv, cache.k, cache.v, slots, ctx.positions, inv_freq, self.qk_norm_eps is not None,
                                 self.qk_norm_eps or 1e-6, self.q_temperature, self.nh, self.nkv, self.hd, layout,
                                 bias=self.b_qkv, vd=self.vd, extra_columns=g_dim)
+        head_gate = (qkv, qkv.shape[1] - g_dim) if self.head_gate and self.maps == 1 else None
         with section("attention", nbytes=lambda: self._keys_held(ctx) * 2 * kv_dim * width + 2 * T * q_dim * width,
                      flops=lambda: 4.0 * self._keys_read(ctx) * q_dim):
             o = ops.attention(q, cache.k, cache.v, g, ctx, self.window_kind, self.window, self.scale, self.nh * self.maps,
-                              self.nkv, self.hd, self.vd, softcap=self.softcap, sink=self.w_sink if self.learned_sink else self.sink)
+                              self.nkv, self.hd, self.vd, softcap=self.softcap, sink=self.w_sink if self.learned_sink else self.sink,
+                              keep=self.keep_first, gate=head_gate)
         if self.maps > 1:
             with section("difference of the maps", nbytes=3 * width * T * self.nh * self.vd):
                 o = ops.map_difference(o, self.nh, self.vd, self.lam, self.difference_eps, 1.0 - self.difference,
@@ -301,9 +329,9 @@ class Attention(Part):
     def _keys_read(self, ctx: StepContext) -> int:
         """(query, key) pairs of the step: what is computed."""
         spec = kv_of(self.cache_spec())
-        return sum(p - spec.first_visible(p) + 1 for s, n in zip(ctx.entry_starts, ctx.entry_lens) for p in range(s, s + n))
+        return sum(spec.keys_seen(p) for s, n in zip(ctx.entry_starts, ctx.entry_lens) for p in range(s, s + n))
 
     def _keys_held(self, ctx: StepContext) -> int:
         """Keys that some query of the step sees, each counted once per entry: what has to be read."""
         spec = kv_of(self.cache_spec())
-        return sum(s + n - spec.first_visible(s) for s, n in zip(ctx.entry_starts, ctx.entry_lens))
+        return sum(n - 1 + spec.keys_seen(s) for s, n in zip(ctx.entry_starts, ctx.entry_lens))

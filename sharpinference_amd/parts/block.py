@@ -111,6 +111,24 @@ class PostNormBlock(PreNormBlock):
             self.norm2.add_normed(stream, y, ctx.act_dtype)
 
 
+class SumNormBlock(PostNormBlock):
+    """h = norm1(alpha * h + mixer(h)); h = norm2(alpha * h + ffn(h)): the norm of the whole sum behind each branch
+    (the original transformer's order, with the sum's old part times ``alpha``).  The branches read h itself, in the
+    activations' storage type (``stream.act``, which the norm kernel leaves beside the float sum); the norms are parts
+    with ``of_sum``.  ``ffn`` None: a layer of a mixer alone."""
+
+    def __init__(self, norm1: Part, mixer: Part, norm2: Part = None, ffn: Part = None, alpha: float = 1.0, names=None):
+        super().__init__(norm1, mixer, norm2, ffn, names)
+        self.alpha = float(alpha)
+
+    def forward(self, stream: ResidualStream, ctx: StepContext, cache: LayerCache) -> None:
+        y = self.mixer.forward(self._input(stream, ctx), ctx, cache)
+        self.norm1.of_sum(stream, y, self.alpha, ctx.act_dtype)
+        if self.ffn is not None:
+            y = self.ffn.forward(stream.act, ctx)
+            self.norm2.of_sum(stream, y, self.alpha, ctx.act_dtype)
+
+
 class ConvPostNormBlock(PreNormBlock):
     """h += norm1(mixer(c1(h))); h += norm2(ffn(c2(h))): norms on the branches' outputs, and a short convolution over the
     residual sum in front of each branch (parts/conv.py).  ``ffn`` None: a layer of a mixer alone.  A branch's output is

@@ -1,4 +1,4 @@
-"""Embeddings that read more than the token itself."""
+"""Embeddings that are more than the token's row."""
 from __future__ import annotations
 
 from typing import Dict, Optional
@@ -7,7 +7,8 @@ import torch
 
 from .. import ops
 from ..cache.spec import StateSpec
-from .base import INIT_NORMAL, LayerCache, ParamSpec, Part, StepContext, TensorSource
+from .base import INIT_NORMAL, LayerCache, ParamSpec, Part, ResidualStream, StepContext, TensorSource
+from .norm import LayerNorm
 
 
 class BigramEmbedding(Part):
@@ -32,3 +33,27 @@ class BigramEmbedding(Part):
 
     def forward(self, ctx: StepContext, table: torch.Tensor, scale: float, cache: LayerCache) -> torch.Tensor:
         return ops.embed_bigram(ctx, table, self.pairs, self.mul_prev, self.mul_cur, cache.states[0], scale)
+
+
+class NormedEmbedding(Part):
+    """A layer norm of table[token] * scale, in float, with the copy that the first branch reads (``norm``: the norm, its
+    tensors under its own names).  Keeps nothing."""
+
+    def __init__(self, norm: LayerNorm):
+        self.norm = norm
+
+    def cache_spec(self) -> None:
+        return None
+
+    def param_specs(self, prefix: str = "") -> Dict[str, ParamSpec]:
+        return self.norm.param_specs(prefix)
+
+    def load(self, prefix: str, source: TensorSource) -> None:
+        self.norm.load(prefix, source)
+
+    def forward(self, ctx: StepContext, table: torch.Tensor, scale: float, cache: LayerCache) -> ResidualStream:
+        copy = ctx.act_dtype if ctx.act_dtype != torch.float32 else None
+        h, act = ops.embed_norm(ctx.token_ids, table, self.norm.weight, self.norm.bias, self.norm.eps, scale, copy)
+        stream = ResidualStream(h)
+        stream.act = h if copy is None else act
+        return stream

@@ -33,8 +33,10 @@ class LatentAttention(Part):
     (the schedule hands it that layer's cache with ``write=False``).  ``window_kind`` / ``window``: which
     keys this layer sees; ``kept`` (kind, window): which the shared rows have to be kept for, where layers
     with different windows read them (default: this layer's own).  ``rotary``: any object with
-    ``table(device)`` (float32 frequencies of the rotated pairs (2i, 2i + 1), at most dr / 2) and a
-    ``magnitude`` (of cos and sin).
+    ``table(device)`` (float32 frequencies of the rotated pairs, at most dr / 2), a ``pair_layout`` and a
+    ``magnitude`` (of cos and sin).  The kernels turn pairs (2i, 2i + 1); with the layout "half" (pairs (i, i + r / 2)) the
+    rows of W_q (or W_uq) and W_dkv that make the rotated parts are put in that order when they are loaded: a score
+    is a sum over the part's elements, so it does not change when queries and keys are reordered alike.
     """
 
     NAMES = {"q": "q", "dq": "dq", "dq_norm": "dq.norm", "uq": "uq", "dkv": "dkv", "dkv_norm": "dkv.norm", "uk": "uk", "uv": "uv", "sink": "sink", "g": "g", "o": "o"}
@@ -47,8 +49,8 @@ class LatentAttention(Part):
             raise ValueError(f"a latent of {rank} elements is not taken: 1 to {ops.LATENT_MAX_RANK}")
         if min(num_heads, nope_dim, rope_dim, v_dim) < 1:
             raise ValueError("heads and head sizes must be positive")
-        if rotary is not None and (rotary.pair_layout != "interleaved" or rotary.rotary_dim > rope_dim):
-            raise ValueError("the rotated part takes interleaved pairs, at most as many as it is wide")
+        if rotary is not None and (rotary.pair_layout not in ("interleaved", "half") or rotary.rotary_dim > rope_dim):
+            raise ValueError("the rotated part takes interleaved or half-split pairs, at most as many as it is wide")
         self.hidden, self.nh, self.dn, self.dr, self.dv, self.rank = (int(hidden), int(num_heads), int(nope_dim),
                                                                      int(rope_dim), int(v_dim), int(rank))
         self.rotary, self.eps, self.scale = rotary, float(norm_eps), float(scale)
@@ -105,16 +107,37 @@ class LatentAttention(Part):
             specs[prefix + n["g"]] = ParamSpec((self.o_dim, self.hidden))
         return specs
 
+    def _pair_order(self) -> Optional[torch.Tensor]:
+        """Where each element of a rotated part comes from when its pairs are to lie side by side; None: they do."""
+        if self.rotary is None or self.rotary.pair_layout == "interleaved":
+            return None
+        r = self.rotary.rotary_dim
+        turned = torch.arange(r).view(2, r // 2).t().reshape(-1)
+        return torch.cat([turned, torch.arange(r, self.dr)])
+
+    def _query_rows(self, w: torch.Tensor) -> torch.Tensor:
+        order = self._pair_order()
+        if order is None:
+            return w
+        rows = torch.cat([torch.arange(self.dn), self.dn + order])
+        return w.view(self.nh, self.dn + self.dr, -1)[:, rows.to(w.device)].reshape(w.shape).contiguous()
+
+    def _latent_rows(self, w: torch.Tensor) -> torch.Tensor:
+        order = self._pair_order()
+        if order is None:
+            return w
+        return w[torch.cat([torch.arange(self.rank), self.rank + order]).to(w.device)].contiguous()
+
     def load(self, prefix: str, source: TensorSource) -> None:
         n = self.names
-        parts = [source.get(prefix + n["dq" if self.q_rank else "q"])]
+        parts = [source.get(prefix + n["dq"]) if self.q_rank else self._query_rows(source.get(prefix + n["q"]))]
         if self.q_rank:
             self.w_q_norm = source.get(prefix + n["dq_norm"]).float().contiguous()
-            self.w_uq = ops.pack_weight(source.get(prefix + n["uq"]))
+            self.w_uq = ops.pack_weight(self._query_rows(source.get(prefix + n["uq"])))
         if self.has_gate:
             parts.append(source.get(prefix + n["g"]))
         if self.own_latent:
-            parts.append(source.get(prefix + n["dkv"]))
+            parts.append(self._latent_rows(source.get(prefix + n["dkv"])))
             self.w_norm = source.get(prefix + n["dkv_norm"]).float().contiguous()
         dt = torch.float32 if any(p.dtype == torch.float32 for p in parts) else parts[0].dtype
         fused = torch.empty(sum(p.shape[0] for p in parts), self.hidden, dtype=dt, device=parts[0].device)

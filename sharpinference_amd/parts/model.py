@@ -47,8 +47,8 @@ class DecoderModel(Part):
                  norm_prefix: str = "model.norm.", head_name: str = "lm_head.weight", embedding_scale: float = 1.0,
                  logit_scale: float = 1.0, logit_softcap: Optional[float] = None,
                  row_tables: Optional[Dict[str, int]] = None, shared: Sequence[Part] = (), embedding: Optional[Part] = None):
-        # a part that makes the first residual sum from the step's tokens and the table (parts/embedding.py); what it
-        # keeps per request lies in a cache slot behind the layers' (None: the token's row times embedding_scale)
+        # a part that makes the first residual sum (or the stream around it) from the step's tokens and the table
+        # (parts/embedding.py); what it keeps per request lies in a cache slot behind the layers' (None: the token's row times embedding_scale)
         self.embedding = embedding
         self.shared = list(shared)       # tensors that several parts read (parts/token_side.py:SharedTensor), loaded once
         self.row_tables: Dict[str, int] = dict(row_tables or {})      # name -> rows of a [rows, hidden] tensor
@@ -172,7 +172,7 @@ class DecoderModel(Part):
                 h = self.embedding.forward(ctx, self.embed, self.embedding_scale, caches[-1])
             else:
                 h = ops.embed_gather(ctx.token_ids, self.embed, scale=self.embedding_scale)
-            stream = ResidualStream(h)
+            stream = h if isinstance(h, ResidualStream) else ResidualStream(h)
         for r in self.schedule:
             c = caches[r.cache]
             if r.add_row is not None:

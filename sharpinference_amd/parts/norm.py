@@ -13,7 +13,8 @@ from .base import INIT_NORM_WEIGHT, ParamSpec, Part, ResidualStream, TensorSourc
 class LayerNorm(Part):
     """(x - mean) / sqrt(variance + eps) * w + b over the last axis, the variance the mean of the squared deviations;
     statistics and sums in float.  ``name``: the weight's name behind the part's prefix (the bias adds
-    ``bias_suffix``).  As the norm on a branch's output (``add_normed``) or as a norm of the stream itself."""
+    ``bias_suffix``).  As the norm on a branch's output (``add_normed``), of the sum of stream and
+    branch (``of_sum``), or as a norm of the stream itself."""
 
     def __init__(self, dim: int, eps: float, name: str = "weight", bias_suffix: str = ".b"):
         self.dim, self.eps, self.name, self.bias_suffix = int(dim), float(eps), name, bias_suffix
@@ -37,6 +38,17 @@ class LayerNorm(Part):
         copy = out_dtype is not None and out_dtype != torch.float32
         with section("norm", nbytes=stream.h.shape[0] * self.dim * 12):
             out = ops.layer_norm(stream.h, self.foldable(delta), self.weight, self.bias, self.eps, out_dtype=out_dtype if copy else None)
+        stream.act = out if copy else stream.h
+
+    def of_sum(self, stream: ResidualStream, delta, alpha: float, out_dtype: torch.dtype) -> None:
+        """h = this norm of (alpha * h + delta), in float, and ``stream.act`` = the new h in ``out_dtype`` (h itself in
+        float32).  Identity experts in an expert sum return the layer's input: where that is the copy of h the
+        branch read, h itself is taken."""
+        copy = out_dtype != torch.float32
+        delta = self.foldable(delta)
+        own = isinstance(delta, ops.ExpertSum) and delta.identity is not None and delta.identity[2] is stream.act
+        with section("norm", nbytes=stream.h.shape[0] * self.dim * 12):
+            out = ops.sum_norm(stream.h, delta, alpha, self.weight, self.bias, self.eps, out_dtype if copy else None, identity_is_h=own)
         stream.act = out if copy else stream.h
 
     def forward(self, stream: ResidualStream, out_dtype: torch.dtype, rows: Optional[torch.Tensor] = None) -> torch.Tensor:
