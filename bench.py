@@ -20,7 +20,9 @@ gates, state-space layers) beside Pazatar layers of the same sizes;
 ``--shape fovosun`` runs Fovosun layers (differential attention, retention, clamped routed experts, four
 residual streams) beside Llama 4 layers of the same width, heads and experts;
 ``--shape pagonex`` runs Pagonex layers (the gated delta rule, latent attention behind a window, routed experts)
-beside Kuvonex layers of the same width, heads and experts and Pazatar layers with the same recurrent heads.
+beside Kuvonex layers of the same width, heads and experts and Pazatar layers with the same recurrent heads;
+``--shape rigodra`` runs Rigodra layers (attention that keeps the first tokens in its window beside latent attention, routed
+experts without a gate with identity experts among them) beside Kuvonex and Llama 4 layers of the same width, heads and experts.
 """
 from __future__ import annotations
 
@@ -767,6 +769,49 @@ def run_pagonex(args) -> int:
     return 0
 
 
+# ---------------------------------------------------------------------------
+# Rigodra beside Kuvonex and Llama 4 at equal sizes
+# ---------------------------------------------------------------------------
+# the sizes are Kuvonex's; `identity` of the router's `experts` outputs are identity experts.  Attention heads are 192
+# wide with values of 128 (the width of a latent layer's heads) and share a key head by eights
+RIGODRA_SIZES = {
+    "w2048": dict(KUVONEX_SIZES["w2048"], identity=8, window=1024, keep=64, q_rank=768),
+    "w4096": dict(KUVONEX_SIZES["w4096"], identity=4, window=1024, keep=64, q_rank=1536),
+}
+RIGODRA_KINDS = (("latent_attention", "moe"), ("attention", "moe"), ("attention", "moe"), ("latent_attention", "dense"))
+
+
+def rigodra_config(z: dict) -> dict:
+    latent = {"heads": z["heads"], "dim": 128, "rot_dim": 64, "vdim": 128, "q_rank": z["q_rank"], "kv_rank": 512, "scale": 192 ** -0.5,
+              "mask": {"size": z["window"]}, "rot": {"base": 10000.0, "dims": 64}}
+    attn = {"heads": z["heads"], "kv_heads": max(1, z["heads"] // 8), "dim": 192, "vdim": 128, "scale": 192 ** -0.5, "v_mix": True,
+            "mask": {"size": z["window"], "keep_first": z["keep"]}, "rot": {"base": 10000.0, "dims": 64}}
+    moe = {"kind": "moe", "expert": {"ff": z["ff"]}, "shared": {"ff": z["ff"]},
+           "router": {"experts": z["experts"] - z["identity"], "top": z["top"], "identity": z["identity"],
+                      "groups": {"count": z["groups"][0], "keep": z["groups"][1]}}}
+    dense = {"kind": "dense", "ff": z["ff"] * z["top"]}
+    layers = [{"type": kind, "mixer": dict(latent if kind == "latent_attention" else attn), "mlp": moe if ff == "moe" else dense}
+              for kind, ff in RIGODRA_KINDS[:z["layers"]]]
+    return {"architecture": "Rigodra", "vocab": z["vocab"], "width": z["width"], "norm": {"eps": 1e-5}, "postln_alpha": 1.7, "layers": layers}
+
+
+def run_rigodra(args) -> int:
+    """Prefill of one 2,048-token prompt and decode at batch 8 and 64 for the Rigodra design at two sizes (random
+    weights), each beside Kuvonex and Llama 4 layers of the same width, heads, experts and expert width, with the
+    per-kernel-class tables of one prefill and one decode step of all."""
+    pairs = (("rigodra", rigodra_config), ("kuvonex", kuvonex_config), ("llama4", llama4_config_like))
+    rows, P, steps, warm = _beside(args, RIGODRA_SIZES, pairs[:1] if args.alone else pairs)
+    k0 = rows[0]
+    out = {"metric": "decode tok/s at batch 8 (Rigodra, width 2048, 4 layers, 2,048-token prompts)", "value": k0["decode_b8_tok_s"],
+           "unit": "tok/s", "n_gpus": 1, "steps": steps, "warmup": warm, "ms_per_step": k0["decode_b8_ms_per_step"],
+           "higher_is_better": True, "scaling": "weak", "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
+           "config": {"model": "rigodra-random beside kuvonex-random and llama4-random at equal sizes", "global_batch": 8,
+                      "seq_len": CONTEXT, "parallelism": "single-gpu", "prompt_len": P, "sizes": RIGODRA_SIZES},
+           "rows": rows}
+    print(json.dumps(out), flush=True)
+    return 0
+
+
 def main() -> int:
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -780,12 +825,13 @@ def main() -> int:
     ap.add_argument("--no-graphs", action="store_true", help="launch decode steps kernel by kernel instead of replaying a HIP graph")
     ap.add_argument("--no-peaks", action="store_true", help="skip the two measuring kernels (pure read, matrix-core loop)")
     ap.add_argument("--profile", action="store_true", help="also print ms / bytes / GB/s per kernel class of one prefill and one decode step")
-    ap.add_argument("--shape", default="scout", choices=["scout", "maverick8", "long16", "kuvonex", "pazatar", "nosedra", "fovosun", "pagonex"],
+    ap.add_argument("--shape", default="scout", choices=["scout", "maverick8", "long16", "kuvonex", "pazatar", "nosedra", "fovosun", "pagonex", "rigodra"],
                     help="scout: the headline run; maverick8 / long16: two other workloads; kuvonex / pazatar: that design beside "
                          "Llama 4 layers of equal size; nosedra: that design beside Pazatar layers of equal size; fovosun: that design beside "
-                         "Llama 4 layers of equal size; pagonex: that design beside Kuvonex and Pazatar layers of equal size; each prints a JSON "
+                         "Llama 4 layers of equal size; pagonex: that design beside Kuvonex and Pazatar layers of equal size; rigodra: that design "
+                         "beside Kuvonex and Llama 4 layers of equal size; each prints a JSON "
                          "line of its own")
-    ap.add_argument("--alone", action="store_true", help="--shape pagonex without the models it is measured beside")
+    ap.add_argument("--alone", action="store_true", help="--shape pagonex or rigodra without the models it is measured beside")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py measures one GPU: this engine has no multi-GPU path (N=1 only)")
@@ -804,6 +850,8 @@ def main() -> int:
         return run_fovosun(args)
     if args.shape == "pagonex":
         return run_pagonex(args)
+    if args.shape == "rigodra":
+        return run_rigodra(args)
 
     import torch  # noqa: F401
 

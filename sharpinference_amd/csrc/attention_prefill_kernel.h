@@ -87,7 +87,7 @@ struct PrefillArgs {
 };
 
 template <int HD, int VD, int kQT>
-__global__ __launch_bounds__(kPreWaves* kWave, HD <= 128 && VD <= 128 ? (kQT == 1 ? 3 : 2) : 1) void attn_prefill_kernel(
+__global__ __launch_bounds__(kPreWaves* kWave, HD <= 128 && VD <= 128 ? (kQT == 1 ? 3 : 2) : HD != VD && HD <= 192 && VD <= 128 ? 2 : 1) void attn_prefill_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_cache, const bf16_t* __restrict__ v_cache,
     const int* __restrict__ block_table, const int* __restrict__ positions, const int* __restrict__ tiles,
     bf16_t* __restrict__ out, int window_kind, int window, float scale, int nh, int nkv, int page_size,

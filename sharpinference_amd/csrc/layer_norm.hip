@@ -510,13 +510,55 @@ __global__ __launch_bounds__(256) void embed_norm_kernel(const int* __restrict__
   }
 }
 
+// A thread has one run of eight elements (hidden a multiple of 8 up to 8,192).
+template <typename T, typename TO>
+__global__ __launch_bounds__(1024) void embed_norm_run_kernel(const int* __restrict__ ids, const T* __restrict__ table, float scale,
+                                                              const float* __restrict__ w, const float* __restrict__ b, float eps,
+                                                              float* __restrict__ out, TO* __restrict__ copy, int hidden) {
+  __shared__ float red[16];
+  const size_t t = blockIdx.x;
+  const int c = threadIdx.x * 8;
+  const bool in = c < hidden;
+  float x[8], wv[8], bv[8];
+  float s = 0.f;
+  if (in) {
+    load8(table + (size_t)ids[t] * hidden + c, x);
+    load8(w + c, wv);
+    load8(b + c, bv);
+#pragma unroll
+    for (int k = 0; k < 8; ++k) {
+      x[k] *= scale;
+      s += x[k];
+    }
+  }
+  const float mean = block_sum(s, red) / (float)hidden;
+  s = 0.f;
+  if (in) {
+#pragma unroll
+    for (int k = 0; k < 8; ++k) s = fmaf(x[k] - mean, x[k] - mean, s);
+  }
+  const float inv = 1.0f / sqrtf(block_sum(s, red) / (float)hidden + eps);
+  if (!in) return;
+#pragma unroll
+  for (int k = 0; k < 8; ++k) x[k] = fmaf((x[k] - mean) * inv, wv[k], bv[k]);
+  store8(out + t * hidden + c, x);
+  if (copy) store8(copy + t * hidden + c, x);
+}
+
 SHARPI_EXPORT int sharpi_embed_norm(const int* ids, const void* table, int t_dtype, float scale, const float* w, const float* b,
                                     float eps, float* out, void* copy, int c_dtype, int n_tokens, int hidden, hipStream_t stream) {
   if (n_tokens <= 0) return SHARPI_OK;
   if (hidden <= 0 || (size_t)hidden * sizeof(float) > 60 * 1024 || !w || !b || !(eps > 0.f)) return SHARPI_ERR_ARG;
   if ((t_dtype != DT_F32 && t_dtype != DT_BF16) || (copy && c_dtype != DT_F32 && c_dtype != DT_BF16)) return SHARPI_ERR_ARG;
   const size_t lds = (size_t)hidden * sizeof(float);
-#define EN(T, TO) embed_norm_kernel<T, TO><<<n_tokens, 256, lds, stream>>>(ids, (const T*)table, scale, w, b, eps, out, (TO*)copy, hidden)
+  auto aligned = [](const void* p) { return ((uintptr_t)p & 31) == 0; };
+  const bool wide = hidden % 8 == 0 && hidden <= 8192 && aligned(table) && aligned(w) && aligned(b) && aligned(out) && aligned(copy);
+  const int threads = ceil_div(hidden / 8, kWave) * kWave;
+#define EN(T, TO)                                                                                                                        \
+  do {                                                                                                                                   \
+    if (wide) embed_norm_run_kernel<T, TO><<<n_tokens, threads, 0, stream>>>(ids, (const T*)table, scale, w, b, eps, out, (TO*)copy, hidden); \
+    else embed_norm_kernel<T, TO><<<n_tokens, 256, lds, stream>>>(ids, (const T*)table, scale, w, b, eps, out, (TO*)copy, hidden);          \
+  } while (0)
   const bool cf = !copy || c_dtype == DT_F32;
   if (t_dtype == DT_F32) {
     if (cf) EN(float, float);

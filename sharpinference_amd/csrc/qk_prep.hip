@@ -317,6 +317,113 @@ __global__ __launch_bounds__(kPrepThreads) void qk_prep_kernel(PrepArgs a) {
   }
 }
 
+// The same for the plain case (no convolution, one map a head, at most a norm per head, values of their own; widths and
+// offsets multiples of 8, pairs split in halves): nothing is staged.  A head lies in neighbouring lanes of a wave, eight elements
+// a lane (kLanes of them, hd / 8 rounded up to a power of two), its sum of squares and the partner run of a
+// rotation come by lane exchange, 16-byte accesses throughout.  Blocks (token, y) share a token's heads between
+// them; consecutive tokens go to one die, whose cache then gathers the values' columns (a page keeps 16 tokens or more
+// of a value channel side by side).
+template <typename T>
+__global__ __launch_bounds__(kPrepThreads) void qk_prep_run_kernel(PrepArgs a, int n_tokens, int lanes) {
+  __shared__ float cs_tab[kPrepMaxTurns], sn_tab[kPrepMaxTurns];
+  const int per_die = gridDim.x / 8;
+  const int t = (blockIdx.x % 8) * per_die + blockIdx.x / 8;
+  if (t >= n_tokens) return;
+  const float pos = (float)a.positions[t];
+  const int half_runs = a.rotary_dim / 16;               // runs of the low half of the rotated part
+  if (a.inv_freq) {
+    for (int i = threadIdx.x; i < a.rotary_dim / 2; i += kPrepThreads) {
+      const float ang = pos * a.inv_freq[i];
+      cs_tab[i] = cosf(ang) * a.magnitude;
+      sn_tab[i] = sinf(ang) * a.magnitude;
+    }
+    __syncthreads();
+  }
+  const int qn = a.nh * a.hd, kn = a.nkv * a.hd, runs = a.hd / 8, heads = a.nh + a.nkv;
+  const T* src = (const T*)a.proj + (size_t)t * a.stride;
+  const int slot = a.slot_mapping ? a.slot_mapping[t] : -1;
+  const int page = slot >= 0 ? slot / a.page_size : 0, off = slot >= 0 ? slot % a.page_size : 0;
+  const float temp = a.temp_on ? 1.0f + a.temp_scale * logf(floorf((pos + 1.0f) / a.temp_floor) + 1.0f) : 1.0f;
+  // a thread's run inside a head is the same in every turn: its angles and norm weights stay in registers
+  const int li = threadIdx.x % lanes;
+  const bool in = li < runs, turns = a.inv_freq && li < 2 * half_runs;
+  const int mate = li < half_runs ? (int)threadIdx.x + half_runs : (int)threadIdx.x - half_runs;
+  float c8[8], s8[8], wq[8], wk[8];
+  if (turns) {
+    const int i0 = (li < half_runs ? li : li - half_runs) * 8;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      c8[j] = cs_tab[i0 + j];
+      s8[j] = li < half_runs ? -sn_tab[i0 + j] : sn_tab[i0 + j];
+    }
+  }
+  if (a.norm_mode != NORM_NONE && in) {
+    load8(a.q_norm_w + li * 8, wq);
+    load8(a.k_norm_w + li * 8, wk);
+  }
+  for (int base = blockIdx.y * kPrepThreads; base < heads * lanes; base += gridDim.y * kPrepThreads) {
+    const int h = (base + (int)threadIdx.x) / lanes;
+    const bool is_q = h < a.nh, live = in && h < heads;
+    float x[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+    if (live) {
+      load8(src + (is_q ? a.q_off + h * a.hd : a.k_off + (h - a.nh) * a.hd) + li * 8, x);
+      if (a.bias) {
+        float b8[8];
+        load8(a.bias + (size_t)h * a.hd + li * 8, b8);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) x[j] += b8[j];
+      }
+    }
+    if (a.norm_mode != NORM_NONE) {                      // every lane takes part in the exchanges
+      float ss = 0.f;
+#pragma unroll
+      for (int j = 0; j < 8; ++j) ss = fmaf(x[j], x[j], ss);
+      for (int o = lanes >> 1; o > 0; o >>= 1) ss += __shfl_xor(ss, o, kWave);
+      const float inv = rsqrtf(ss / (float)a.hd + a.eps);
+      if (live) {
+#pragma unroll
+        for (int j = 0; j < 8; ++j) x[j] = x[j] * inv * (is_q ? wq[j] : wk[j]);
+      }
+    }
+    if (a.inv_freq) {
+#pragma unroll
+      for (int j = 0; j < 8; ++j) {
+        const float other = __shfl(x[j], mate & (kWave - 1), kWave);
+        if (turns) x[j] = x[j] * c8[j] + other * s8[j];
+      }
+    }
+    if (!live) continue;
+    if (is_q) {
+#pragma unroll
+      for (int j = 0; j < 8; ++j) x[j] *= temp;
+      store8((T*)a.q_out + (size_t)t * qn + (size_t)h * a.hd + li * 8, x);
+    } else if (slot >= 0) {
+      store8((T*)a.k_cache + (((size_t)page * a.nkv + (h - a.nh)) * a.page_size + off) * a.hd + li * 8, x);
+    }
+  }
+  if (slot < 0) return;
+  for (int i = (blockIdx.y * kPrepThreads + threadIdx.x) * 8; i < a.nkv * a.vd; i += gridDim.y * kPrepThreads * 8) {
+    float v[8];
+    load8(src + a.v_off + i, v);
+    if (a.bias) {
+      float b8[8];
+      load8(a.bias + qn + kn + i, b8);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) v[j] += b8[j];
+    }
+    if (a.v_other) {
+      float u[8];
+      load8((const T*)a.v_other + (size_t)t * a.v_other_stride + a.v_other_off + i, u);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) v[j] = (1.0f - a.v_mix) * v[j] + a.v_mix * u[j];
+    }
+    const int g = i / a.vd, d = i % a.vd;
+    T* dst = (T*)a.v_cache + (((size_t)page * a.nkv + g) * a.vd + d) * a.page_size + off;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) dst[(size_t)j * a.page_size] = from_f32<T>(v[j]);
+  }
+}
+
 // The convolution's tail after a step: the last taps - 1 projected rows of each entry's request
 // (rows of this step where the entry brought enough, what the slot held before otherwise).  A
 // thread takes one channel of one entry, reads everything it needs and only then writes.
@@ -383,6 +490,19 @@ SHARPI_EXPORT int sharpi_qk_prep(const void* proj, int dtype, int stride, int q_
              cu_tokens, positions, norm_mode, q_norm_w, k_norm_w, eps, rotary_dim > 0 ? inv_freq : nullptr, rotary_dim,
              half_split, magnitude, q_out, k_cache, v_cache, slot_mapping, page_size, parts, bias, temp_on, temp_floor,
              temp_scale, maps, v_other, v_other_stride, v_other_off, v_mix, by8};
+  const int lanes = hd <= 64 ? (hd <= 8 ? 1 : hd <= 16 ? 2 : hd <= 32 ? 4 : 8) : hd <= 128 ? 16 : hd <= 256 ? 32 : 64;
+  if (by8 && taps == 0 && maps == 1 && norm_mode != NORM_WHOLE && v_off >= 0 && hd <= 512 && at16(q_norm_w) && at16(k_norm_w) &&
+      (!v_other || (at16(v_other) && v_other_stride % 8 == 0 && v_other_off % 8 == 0))) {
+    // few tokens: a block a turn; many: four turns or so a block, to share the angles
+    const int all_turns = ceil_div((nh + nkv) * lanes, kPrepThreads);
+    const int y = n_tokens <= kPrepSplitTokens ? all_turns : ceil_div(all_turns, 4);
+    dim3 rgrid(8 * ceil_div(n_tokens, 8), y);
+    if (dtype == DT_F32) qk_prep_run_kernel<float><<<rgrid, kPrepThreads, 0, stream>>>(a, n_tokens, lanes);
+    else if (dtype == DT_BF16) qk_prep_run_kernel<bf16_t><<<rgrid, kPrepThreads, 0, stream>>>(a, n_tokens, lanes);
+    else return SHARPI_ERR_ARG;
+    SHARPI_CHECK_LAUNCH();
+    return SHARPI_OK;
+  }
   dim3 pgrid(n_tokens, parts);
   if (dtype == DT_F32) qk_prep_kernel<float><<<pgrid, kPrepThreads, lds, stream>>>(a);
   else if (dtype == DT_BF16) qk_prep_kernel<bf16_t><<<pgrid, kPrepThreads, lds, stream>>>(a);
